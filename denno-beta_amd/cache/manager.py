@@ -44,6 +44,7 @@ class GroupLayout:
     n_pages: int = 0
     page_size: int = 1
     window: int = 0      # 0: all keys are kept
+    keep_first: int = 0  # with a window: the first keys, which every query reads and which stay
 
 
 _host = None
@@ -56,7 +57,7 @@ def host_library():
         I, L, P = c_int, c_int64, c_void_p
         IP = POINTER(c_int)
         sig = {
-            "dn_cache_create": (P, [I, IP, IP, IP, IP, I]), "dn_cache_destroy": (None, [P]),
+            "dn_cache_create": (P, [I, IP, IP, IP, IP, IP, I]), "dn_cache_destroy": (None, [P]),
             "dn_cache_add": (I, [P, L]), "dn_cache_release": (I, [P, L]), "dn_cache_reserve": (I, [P, L, I]),
             "dn_cache_commit": (I, [P, L, I]), "dn_cache_length": (I, [P, L]), "dn_cache_slot": (I, [P, L]),
             "dn_cache_state": (I, [P, L, c_void_p]), "dn_cache_set_rng": (I, [P, L, ctypes.c_uint64, ctypes.c_uint64]),
@@ -99,7 +100,8 @@ class CacheManager:
         arr = lambda vals: (c_int * max(n, 1))(*vals)   # noqa: E731
         self._h = self._lib.dn_cache_create(
             n, arr([g.kind for g in self.groups]), arr([g.n_pages for g in self.groups]),
-            arr([g.page_size for g in self.groups]), arr([g.window for g in self.groups]), max_requests)
+            arr([g.page_size for g in self.groups]), arr([g.window for g in self.groups]),
+            arr([g.keep_first for g in self.groups]), max_requests)
         if not self._h:
             raise ValueError(f"cache manager: bad layout {self.groups} for {max_requests} requests")
 

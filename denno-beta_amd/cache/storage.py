@@ -44,7 +44,7 @@ class CacheStorage:
         layouts = []
         for cs in self.group_specs:
             if isinstance(cs, PagedKV):
-                layouts.append(GroupLayout(PAGED, n_pages, page_size, cs.window))
+                layouts.append(GroupLayout(PAGED, n_pages, page_size, cs.window, cs.keep_first))
             elif isinstance(cs, FixedState):
                 layouts.append(GroupLayout(STATE))
             else:

@@ -16,12 +16,12 @@ using denno::StepEntry;
 extern "C" {
 
 void* dn_cache_create(int n_groups, const int* kinds, const int* n_pages, const int* page_size,
-                      const int* window, int max_requests) {
+                      const int* window, const int* keep_first, int max_requests) {
   if (n_groups < 0 || max_requests < 1) return nullptr;
   std::vector<GroupSpec> g(n_groups);
   for (int i = 0; i < n_groups; ++i) {
-    g[i] = GroupSpec{kinds[i], n_pages[i], page_size[i], window[i]};
-    if (kinds[i] == denno::kPaged && (n_pages[i] < 1 || page_size[i] < 1 || window[i] < 0)) return nullptr;
+    g[i] = GroupSpec{kinds[i], n_pages[i], page_size[i], window[i], keep_first[i]};
+    if (kinds[i] == denno::kPaged && (n_pages[i] < 1 || page_size[i] < 1 || window[i] < 0 || keep_first[i] < 0)) return nullptr;
   }
   return new (std::nothrow) CacheManager(g, max_requests);
 }

@@ -55,6 +55,11 @@ int CacheManager::first_needed_block(int g, int len) const {
   return first_key <= 0 ? 0 : first_key / s.page_size;
 }
 
+int CacheManager::kept_blocks(int g) const {
+  const GroupSpec& s = groups_[g];
+  return (s.keep_first + s.page_size - 1) / s.page_size;
+}
+
 int CacheManager::pages_needed(int64_t rid, int from_len, int new_len, int g) const {
   if (g < 0 || g >= n_groups() || groups_[g].kind != kPaged) return 0;
   int have = 0;
@@ -74,9 +79,10 @@ int CacheManager::pages_peak(int g, int total_len, int chunk) const {
   const GroupSpec& s = groups_[g];
   int all = (total_len + s.page_size - 1) / s.page_size;
   if (s.window <= 0) return all;
-  // window keys before the portion, the portion itself, and one page of slack at each edge
+  // window keys before the portion, the portion itself, and one page of slack at each edge; and the pages of the first
+  // keys, which stay
   int span = (s.window + std::max(chunk, 1) + s.page_size - 1) / s.page_size + 1;
-  return std::min(all, span);
+  return std::min(all, span + kept_blocks(g));
 }
 
 int CacheManager::reserve(int64_t rid, int new_len) {
@@ -118,7 +124,7 @@ int CacheManager::commit(int64_t rid, int new_len) {
     if (groups_[g].kind != kPaged) continue;
     int first = std::min(first_needed_block(static_cast<int>(g), new_len),
                          static_cast<int>(r.tables[g].size()));
-    for (int b = r.first_live[g]; b < first; ++b) {
+    for (int b = std::max(r.first_live[g], kept_blocks(static_cast<int>(g))); b < first; ++b) {
       if (r.tables[g][b] >= 0) {
         free_[g].push_back(r.tables[g][b]);
         r.tables[g][b] = -1;

@@ -32,6 +32,7 @@ struct GroupSpec {
   int n_pages;     // pool size (paged groups)
   int page_size;   // tokens in a page
   int window;      // 0: every key is kept; W > 0: a query at position p reads keys in (p - W, p]
+  int keep_first = 0;   // with a window: the first keep_first keys are read by every query and stay
 };
 
 // What a live request keeps beside its pages, in its slot: a record of fixed size, zero when the slot
@@ -102,9 +103,10 @@ class CacheManager {
   struct Request {
     int slot;                                  // index of its SlotState (the position lives there)
     std::vector<std::vector<int32_t>> tables;  // [group][block] -> page, -1 once given back
-    std::vector<int> first_live;               // [group] first block that is still held
+    std::vector<int> first_live;               // [group] first block that is still held (behind the kept ones)
   };
   int first_needed_block(int g, int len) const;
+  int kept_blocks(int g) const;      // blocks at a request's start that a window never gives back
 
   std::vector<GroupSpec> groups_;
   std::vector<std::vector<int32_t>> free_;     // [group] stack of free pages

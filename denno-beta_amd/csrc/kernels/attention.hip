@@ -10,8 +10,9 @@
 //
 // What a layer may add to this (ScoreExtras): chunks (a row reads only the keys of its own run of `chunk` positions, runs
 // counted from the request's position 0), a bias by distance (bias[h][pos - key] is added to the scaled score; distances
-// from `span` on take the last entry) and a sink (a key that every row sees, with score 0 and no value: one more
-// summand, exp(0), under the softmax).
+// from `span` on take the last entry), a sink (a key that every row sees, with a score per head, or 0, and no value: one more
+// summand, exp(score), under the softmax) and, with a window, the request's first `keep` keys, which every row reads as well
+// (their pages stay; those between them and the window are given back, and the kernels step over the gap).
 //
 // The key pool is [n_pages, Hkv, page_size, dh], the value pool [n_pages, Hkv, dh, page_size];
 // query head h reads key head h / (H / Hkv).
@@ -28,6 +29,22 @@ __device__ __forceinline__ int first_key(int pos, int window, int chunk) {
   if (chunk > 0) lo = max(lo, pos / chunk * chunk);
   return lo;
 }
+
+// whether the row at `pos`, whose window begins at `lo`, reads `key`
+__device__ __forceinline__ bool reads_key(int key, int lo, int pos, int keep) { return key <= pos && (key >= lo || key < keep); }
+
+// the score of the sink that head h sees (ex.sink set)
+__device__ __forceinline__ float sink_score(const ScoreExtras& ex, int h) { return ex.sink_at ? ex.sink_at[h] : 0.f; }
+
+// Keys are walked in tiles of `tile` from multiples of `tile`: those that hold the first `keep` keys, then those from the
+// window's first key `lo` on.  The walk starts at first(), goes from kt to next(kt), and ends where the caller's last key is
+// passed; a tile is never visited twice.
+struct TileWalk {
+  int tile, keep_end, rest;
+  __device__ __forceinline__ TileWalk(int tile_, int lo, int keep) : tile(tile_), keep_end((keep + tile_ - 1) / tile_ * tile_), rest(max(lo / tile_ * tile_, keep_end)) {}
+  __device__ __forceinline__ int first() const { return keep_end > 0 ? 0 : rest; }
+  __device__ __forceinline__ int next(int kt) const { return kt + tile == keep_end ? rest : kt + tile; }
+};
 
 namespace plain {
 constexpr int BQ = 16;
@@ -71,8 +88,8 @@ __device__ __forceinline__ float dim_sum(const float* ps, const float* vs, int d
 
 // the scores of one row against the tile in Ks: p[j] to Ps (this row's BK entries), -> m_T, l_T
 __device__ __forceinline__ void tile_scores(const float* qr, const float* Ks, float* ps, int g, int nc, int dh, int kt,
-                                            int lo, int pos, bool row_ok, float scale, const float* bias, int span, float& m_t,
-                                            float& l_t) {
+                                            int lo, int pos, int keep, bool row_ok, float scale, const float* bias, int span,
+                                            float& m_t, float& l_t) {
   const float NEG_INF = -INFINITY;
   float s[4];
   float tmax = NEG_INF;
@@ -83,7 +100,7 @@ __device__ __forceinline__ void tile_scores(const float* qr, const float* Ks, fl
       const int j = g + 16 * c;
       const int key = kt + j;
       const float dot = key_dot(qr, Ks + j * (dh + 1), dh);
-      const bool ok = row_ok && key >= lo && key <= pos;
+      const bool ok = row_ok && reads_key(key, lo, pos, keep);
       s[c] = ok ? (bias ? fmaf(dot, scale, bias[min(pos - key, span - 1)]) : dot * scale) : NEG_INF;
       tmax = fmaxf(tmax, s[c]);
     }
@@ -243,11 +260,13 @@ __global__ __launch_bounds__(THREADS) void attention_kernel(
 #pragma unroll
   for (int i = 0; i < 16; ++i) acc[i] = 0.f;
 
-  for (int kt = (first_lo / BK) * BK; kt <= last_pos; kt += BK) {
+  const TileWalk walk(BK, first_lo, ex.keep);
+  for (int kt = walk.first(); kt <= last_pos; kt = walk.next(kt)) {
     __syncthreads();
     load_tile(Ks, Vs, Kb, Vb, k_pool, v_pool, bt, kt, last_pos, BK, dh, page_size, Hkv, hk, dhp + 1);
     float m_t, l_t, a_t[16];
-    tile_scores(Qs + qi * dhp, Ks, Ps + qi * BK, g, nc, dhp, kt, my_lo, my_pos, row_ok, scale, bias, ex.span, m_t, l_t);
+    tile_scores(Qs + qi * dhp, Ks, Ps + qi * BK, g, nc, dhp, kt, my_lo, my_pos, ex.keep, row_ok, scale, bias, ex.span, m_t,
+                l_t);
     __syncthreads();
     if (m_t > NEG_INF) {                // the same for the 16 threads of a row
       tile_values(Ps + qi * BK, Vs, g, nd, dhp, BK, a_t);
@@ -255,7 +274,7 @@ __global__ __launch_bounds__(THREADS) void attention_kernel(
     }
   }
   if (row_ok) {
-    float inv = 1.0f / (ex.sink ? l + expf(-m) : l);
+    float inv = 1.0f / (ex.sink ? l + expf(sink_score(ex, h) - m) : l);
     T* o = out + static_cast<size_t>(row0 + qi) * ldo + h * dh;
 #pragma unroll
     for (int i = 0; i < 16; ++i)
@@ -289,7 +308,7 @@ __global__ __launch_bounds__(THREADS) void row_tiles_kernel(
   const int kt = ktile * BK;
   const int t = threadIdx.x, g = t % 16;
   float* mine = part + ((static_cast<size_t>(tile) * H + h) * n_key_tiles + ktile) * (dh + 2);
-  if (kt > pos || kt + BK <= lo) {
+  if (kt > pos || (kt + BK <= lo && kt >= ex.keep)) {
     if (t == 0) mine[0] = -INFINITY;
     return;
   }
@@ -306,7 +325,7 @@ __global__ __launch_bounds__(THREADS) void row_tiles_kernel(
     if (t < BK) {
       const int key = kt + t;
       const float dot = key_dot(Qs, Ks + t * (dh + 1), dh);
-      s = (key >= lo && key <= pos) ? (bias ? fmaf(dot, scale, bias[min(pos - key, ex.span - 1)]) : dot * scale) : NEG_INF;
+      s = reads_key(key, lo, pos, ex.keep) ? (bias ? fmaf(dot, scale, bias[min(pos - key, ex.span - 1)]) : dot * scale) : NEG_INF;
     }
     const float tmax = wave_max(s);
     if (t < BK) Ps[t] = s > NEG_INF ? expf(s - tmax) : 0.f;
@@ -364,7 +383,7 @@ __global__ __launch_bounds__(64) void row_tile64_kernel(
   const int kt = ktile * BK;
   const int lane = threadIdx.x;
   float* mine = part + ((static_cast<size_t>(tile) * H + h) * n_key_tiles + ktile) * (DH + 2);
-  if (kt > pos || kt + BK <= lo) {
+  if (kt > pos || (kt + BK <= lo && kt >= ex.keep)) {
     if (lane == 0) mine[0] = -INFINITY;
     return;
   }
@@ -409,7 +428,7 @@ __global__ __launch_bounds__(64) void row_tile64_kernel(
     dot = fmaf(a.w, b.w, dot);
   }
   const int key = kt + lane;
-  const float sc = (key >= lo && key <= pos) ? (bias ? fmaf(dot, scale, bias[min(pos - key, ex.span - 1)]) : dot * scale) : NEG_INF;
+  const float sc = reads_key(key, lo, pos, ex.keep) ? (bias ? fmaf(dot, scale, bias[min(pos - key, ex.span - 1)]) : dot * scale) : NEG_INF;
   const float tmax = wave_max(sc);
   Ps[lane] = sc > NEG_INF ? expf(sc - tmax) : 0.f;
   __syncthreads();
@@ -438,7 +457,7 @@ __global__ __launch_bounds__(64) void row_tile64_kernel(
 
 template <typename T>
 __global__ void row_join_kernel(const float* __restrict__ part, T* __restrict__ out, int ldo,
-                                const int32_t* __restrict__ tile_seq, int n_key_tiles, int H, int dh, int sink) {
+                                const int32_t* __restrict__ tile_seq, int n_key_tiles, int H, int dh, ScoreExtras ex) {
   const int tile = blockIdx.x, h = blockIdx.y;
   if (tile_seq[tile] < 0) return;
   const int g = threadIdx.x;           // 16 threads, the dims g + 16 i each, as in the kernels above
@@ -468,7 +487,7 @@ __global__ void row_join_kernel(const float* __restrict__ part, T* __restrict__ 
       join_tile(m, l, acc, m_t[u], l_t[u], a_t, nd);
     }
   }
-  const float inv = 1.0f / (sink ? l + expf(-m) : l);
+  const float inv = 1.0f / (ex.sink ? l + expf(sink_score(ex, h) - m) : l);
   T* o = out + static_cast<size_t>(tile) * ldo + h * dh;
 #pragma unroll
   for (int i = 0; i < 16; ++i)
@@ -479,23 +498,27 @@ __global__ void row_join_kernel(const float* __restrict__ part, T* __restrict__ 
 static int tile_keys(int dh) { return dh <= 64 ? 64 : (dh <= 128 ? 32 : 16); }
 }  // namespace plain
 
+// kept first keys go with a window, and not with chunks (a page behind a chunk is not told from one behind a window)
+static bool keep_ok(int keep, int window, int chunk) { return keep == 0 || (keep > 0 && window > 0 && chunk == 0); }
+
 extern "C" int dn_attention(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                             const int32_t* block_tables, int max_blocks, const int32_t* tile_seq,
                             const int32_t* tile_row0, const int32_t* tile_nrows, const int32_t* tile_pos0,
                             int n_tiles, int H, int Hkv, int dh, int page_size, float scale, int window, int dtype,
                             hipStream_t stream) {
   return dn_attention_extras(q, ldq, out, ldo, k_pool, v_pool, block_tables, max_blocks, tile_seq, tile_row0, tile_nrows, tile_pos0,
-                             n_tiles, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, dtype, stream);
+                             n_tiles, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, nullptr, 0, dtype, stream);
 }
 
 extern "C" int dn_attention_extras(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                                    const int32_t* block_tables, int max_blocks, const int32_t* tile_seq,
                                    const int32_t* tile_row0, const int32_t* tile_nrows, const int32_t* tile_pos0,
                                    int n_tiles, int H, int Hkv, int dh, int page_size, float scale, int window, int chunk,
-                                   const float* bias, int span, int sink, int dtype, hipStream_t stream) {
+                                   const float* bias, int span, int sink, const float* sink_at, int keep, int dtype,
+                                   hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  if (chunk < 0 || (bias && span < 1)) return DN_ERR_SHAPE;
-  const ScoreExtras ex{chunk, bias, span, sink};
+  if (chunk < 0 || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
+  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep};
   // (any head size up to 256: one that is no multiple of 16 is padded to the next inside the kernel)
   if (dh < 1 || dh > 256 || Hkv < 1 || H % Hkv != 0 || page_size < 1 || max_blocks < 1) return DN_ERR_SHAPE;
   const int dhp = (dh + 15) / 16 * 16;
@@ -528,17 +551,17 @@ extern "C" int dn_attention_rows(const void* q, int ldq, void* out, int ldo, con
                                  const int32_t* tile_pos0, int n_tiles, float* part, int max_context, int H, int Hkv,
                                  int dh, int page_size, float scale, int window, int dtype, hipStream_t stream) {
   return dn_attention_rows_extras(q, ldq, out, ldo, k_pool, v_pool, block_tables, max_blocks, tile_seq, tile_pos0, n_tiles, part,
-                                  max_context, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, dtype, stream);
+                                  max_context, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, nullptr, 0, dtype, stream);
 }
 
 extern "C" int dn_attention_rows_extras(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                                         const int32_t* block_tables, int max_blocks, const int32_t* tile_seq,
                                         const int32_t* tile_pos0, int n_tiles, float* part, int max_context, int H, int Hkv,
                                         int dh, int page_size, float scale, int window, int chunk, const float* bias, int span,
-                                        int sink, int dtype, hipStream_t stream) {
+                                        int sink, const float* sink_at, int keep, int dtype, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  if (chunk < 0 || (bias && span < 1)) return DN_ERR_SHAPE;
-  const ScoreExtras ex{chunk, bias, span, sink};
+  if (chunk < 0 || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
+  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep};
   if (dh < 16 || dh > 256 || dh % 16 != 0 || Hkv < 1 || H % Hkv != 0 || page_size < 1 || max_blocks < 1 ||
       max_context < 1 || !part || n_tiles > 65535 || H > 65535)
     return DN_ERR_SHAPE;
@@ -558,7 +581,7 @@ extern "C" int dn_attention_rows_extras(const void* q, int ldq, void* out, int l
                        static_cast<const T*>(k_pool), static_cast<const T*>(v_pool), block_tables, max_blocks,       \
                        tile_seq, tile_pos0, part, n_key_tiles, H, Hkv, dh, page_size, BK, scale, window, ex);        \
   hipLaunchKernelGGL(plain::row_join_kernel<T>, dim3(n_tiles, H), dim3(16), 0, stream, part, static_cast<T*>(out), ldo, \
-                     tile_seq, n_key_tiles, H, dh, sink)
+                     tile_seq, n_key_tiles, H, dh, ex)
   if (dtype == DN_F32) {
     DN_ROWS(float);
   } else if (dtype == DN_BF16) {
@@ -621,7 +644,7 @@ typedef __attribute__((__vector_size__(4 * sizeof(uint32_t)))) uint32_t u32x4;
 // POW2: the page size is a power of two (page_size = 1 << page_shift), so that a key's page and its place in
 // the page are a shift and a mask: a tile's keys need four such pairs a step, and a division by a number
 // known only at run time is some twenty-five vector instructions.
-// EXTRAS: chunks, a bias by distance and a sink (ScoreExtras).  A score is then the scaled product plus the bias, both
+// EXTRAS: chunks, a bias by distance, a sink and kept first keys (ScoreExtras).  A score is then the scaled product plus the bias, both
 // in units of log2(e), made before the maximum is taken (the largest product is no longer the largest score).
 template <int DH16, int GROUPS, int TPS, bool POW2, bool EXTRAS = false>     // head size / 16; groups of 4 waves; tiles a wave takes per step
 __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH16 > 12 && GROUPS == 1 ? 1 : 2))) void kernel(
@@ -673,6 +696,7 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
   const int lo_g = first_key(pos0, window, chunk);              // the workgroup's
   const int hi_g = pos0 + nrows - 1;
   const float* bias = EXTRAS && ex.bias ? ex.bias + static_cast<size_t>(h) * ex.span : nullptr;
+  const int keep = EXTRAS ? ex.keep : 0;
   const float NEG_INF = -INFINITY;
   const float scale2 = scale * 1.44269504088896340736f;    // log2(e)
   const u32x4 zero4 = {0u, 0u, 0u, 0u};
@@ -735,33 +759,36 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
     }
   };
 
-  // Step kt first puts the tiles of step kt + STEP (asked for during the step before) from
+  // Step kt first puts the tiles of the step after it (asked for during the step before) from
   // registers into the half of LDS that the step before read (every wave has left it: the
-  // barrier), then asks for the tiles of step kt + 2 STEP, then multiplies.
-  const int kt0 = (lo_g / STEP) * STEP;
+  // barrier), then asks for the tiles of the step after that, then multiplies.
+  const TileWalk walk(STEP, lo_g, keep);
+  const int kt0 = walk.first(), kt1 = walk.next(kt0), kt2 = walk.next(kt1);
   const int mine = 32 * TPS * ti;            // this thread carries the tiles at kt + mine + 32 c
   Pages pg_now[TPS], pg_reg[TPS], pg_far[TPS];    // pages of the tiles in registers and of those to ask for next
 #pragma clang loop unroll(full)
   for (int c = 0; c < TPS; ++c) {
     pg_now[c] = pages_of(kt0 + mine + 32 * c);
     fetch(kt0 + mine + 32 * c, pg_now[c], kregs[c], vregs[c]);
-    pg_reg[c] = pages_of(kt0 + STEP + mine + 32 * c);
+    pg_reg[c] = pages_of(kt1 + mine + 32 * c);
   }
 #pragma clang loop unroll(full)
   for (int c = 0; c < TPS; ++c) {
     stash(pg_now[c], tiles_lds + (ti * TPS + c) * TSZ, kregs[c], vregs[c]);
-    fetch(kt0 + STEP + mine + 32 * c, pg_reg[c], kregs[c], vregs[c]);
-    pg_far[c] = pages_of(kt0 + 2 * STEP + mine + 32 * c);
+    fetch(kt1 + mine + 32 * c, pg_reg[c], kregs[c], vregs[c]);
+    pg_far[c] = pages_of(kt2 + mine + 32 * c);
   }
   __syncthreads();
   int buf = 0;
-  for (int kt = kt0; kt <= hi_g; kt += STEP, buf ^= 1) {
+  int kn1 = kt1, kn2 = kt2;      // the steps behind kt
+  for (int kt = kt0; kt <= hi_g; buf ^= 1) {
+    const int kn3 = walk.next(kn2);
 #pragma clang loop unroll(full)
     for (int c = 0; c < TPS; ++c) {
-      if (kt + STEP <= hi_g) stash(pg_reg[c], tiles_lds + (((buf ^ 1) * GROUPS + ti) * TPS + c) * TSZ, kregs[c], vregs[c]);
-      if (kt + 2 * STEP <= hi_g) fetch(kt + 2 * STEP + mine + 32 * c, pg_far[c], kregs[c], vregs[c]);
+      if (kn1 <= hi_g) stash(pg_reg[c], tiles_lds + (((buf ^ 1) * GROUPS + ti) * TPS + c) * TSZ, kregs[c], vregs[c]);
+      if (kn2 <= hi_g) fetch(kn2 + mine + 32 * c, pg_far[c], kregs[c], vregs[c]);
       pg_reg[c] = pg_far[c];
-      pg_far[c] = pages_of(kt + 3 * STEP + mine + 32 * c);
+      pg_far[c] = pages_of(kn3 + mine + 32 * c);
     }
 
     // this wave's tiles of the step: kw0 + 32 c.  They share one maximum, one sum and one rescaling:
@@ -771,7 +798,7 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
     bool act[TPS], any = false;
 #pragma unroll
     for (int c = 0; c < TPS; ++c) {
-      act[c] = has_rows && kw0 + 32 * c <= hi_w && kw0 + 32 * c + 31 >= lo_w;     // the same for the whole wave
+      act[c] = has_rows && kw0 + 32 * c <= hi_w && (kw0 + 32 * c + 31 >= lo_w || kw0 + 32 * c < keep);     // the same for the whole wave
       any = any || act[c];
     }
     if (any) {
@@ -802,13 +829,13 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
 #pragma unroll
       for (int c = 0; c < TPS; ++c) {
         const int kw = kw0 + 32 * c;
-        const bool edge = kw + 31 > pos0 + wrow0 || kw < lo_last;
+        const bool edge = kw + 31 > pos0 + wrow0 || (kw < lo_last && kw + 31 >= keep);
         if (!act[c]) continue;
         if constexpr (EXTRAS) {
 #pragma unroll
           for (int i = 0; i < 16; ++i) {
             const int key = kw + 8 * (i / 4) + 4 * g + (i % 4);
-            const bool ok = key >= my_lo && key <= my_pos;
+            const bool ok = reads_key(key, my_lo, my_pos, keep);
             float sc = s[c][i] * scale2;
             if (bias) sc = fmaf(bias[min(max(my_pos - key, 0), ex.span - 1)], 1.44269504088896340736f, sc);
             s[c][i] = (!edge || ok) ? sc : NEG_INF;
@@ -882,6 +909,7 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
       }
     }
     __syncthreads();      // the other half of LDS is written and this one has been read by every wave
+    kt = kn1, kn1 = kn2, kn2 = kn3;
   }
   if constexpr (GROUPS > 1) {
     // the second group hands its maxima, sums and weighted values to the first, lane to lane (both
@@ -909,7 +937,7 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
       for (int i = 0; i < 16; ++i) o[db][i] = o[db][i] * f0 + join[2 + 16 * db + i] * f1;
   }
   if (has_rows && row_ok) {
-    if (EXTRAS && ex.sink) l += __builtin_amdgcn_exp2f(-m);      // (a key with score 0 and no value)
+    if (EXTRAS && ex.sink) l += __builtin_amdgcn_exp2f(fmaf(sink_score(ex, h), 1.44269504088896340736f, -m));      // (a key without a value)
     const float inv = 1.0f / l;
     // rows, or packed rows (ldo == 0): four dims from a multiple of 4 are 8 bytes side by side in both
     const int orow_i = row0 + my_row;
@@ -936,19 +964,19 @@ extern "C" int dn_attention_flash(const void* q, int ldq, void* out, int ldo, co
                                   int n_tiles, int H, int Hkv, int dh, int page_size, float scale, int window,
                                   hipStream_t stream) {
   return dn_attention_flash_extras(q, ldq, out, ldo, k_pool, v_pool, block_tables, max_blocks, tile_seq, tile_row0, tile_nrows,
-                                   tile_pos0, n_tiles, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, stream);
+                                   tile_pos0, n_tiles, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, nullptr, 0, stream);
 }
 
-// With chunks, a bias by distance or a sink: pages of a power of two only.
+// With any of ScoreExtras: pages of a power of two only.
 extern "C" int dn_attention_flash_extras(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                                          const int32_t* block_tables, int max_blocks, const int32_t* tile_seq,
                                          const int32_t* tile_row0, const int32_t* tile_nrows, const int32_t* tile_pos0,
                                          int n_tiles, int H, int Hkv, int dh, int page_size, float scale, int window, int chunk,
-                                         const float* bias, int span, int sink, hipStream_t stream) {
+                                         const float* bias, int span, int sink, const float* sink_at, int keep, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  const bool extras = chunk > 0 || bias != nullptr || sink != 0;
-  if (chunk < 0 || (bias && span < 1)) return DN_ERR_SHAPE;
-  const ScoreExtras ex{chunk, bias, span, sink};
+  const bool extras = chunk > 0 || bias != nullptr || sink != 0 || keep > 0;
+  if (chunk < 0 || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
+  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep};
   // ldo == 0: out is a packed matrix of H * dh columns (a multiple of 32); the kernel takes the largest score
   // for the largest product of a query and a key, so the scale is positive
   if (!(scale > 0.f)) return DN_ERR_SHAPE;
@@ -1064,10 +1092,11 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
   const int pos = tile_pos0[tile];
   const int lo = first_key(pos, window, EXTRAS ? ex.chunk : 0);
   const float* bias = EXTRAS && ex.bias ? ex.bias + static_cast<size_t>(h) * ex.span : nullptr;
+  const int keep = EXTRAS ? ex.keep : 0;
   const int key0 = split * chunks * CHUNK;
   const float NEG_INF = -INFINITY;
   float* mypart = part + ((static_cast<size_t>(tile) * H + h) * n_splits + split) * (DH + 2);
-  if (key0 > pos || key0 + chunks * CHUNK <= lo) {
+  if (key0 > pos || (key0 + chunks * CHUNK <= lo && key0 >= keep)) {
     if (n_splits > 1 && threadIdx.x == 0) {
       mypart[0] = NEG_INF;     // the join skips it
       mypart[1] = 0.f;
@@ -1085,7 +1114,7 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
 
   for (int c = 0; c < chunks; ++c) {
     const int kbase = key0 + c * CHUNK + wave * 64;
-    if (kbase > pos || kbase + 64 <= lo) continue;     // the same for the whole wave; no barrier in this loop
+    if (kbase > pos || (kbase + 64 <= lo && kbase >= keep)) continue;     // the same for the whole wave; no barrier in this loop
     // values: lane = dim; 16 keys of one page at a time.  They are asked for first, before the keys
     // (whose use would otherwise stand between them and memory): keys and values then make one trip
     bf16x8 v0[4][DPL], v1[4][DPL];
@@ -1093,7 +1122,7 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
 #pragma unroll
     for (int blk = 0; blk < 4; ++blk) {
       const int kb = kbase + blk * 16;
-      live[blk] = kb <= pos && kb + 16 > lo;
+      live[blk] = kb <= pos && (kb + 16 > lo || kb < keep);
       const int kk = live[blk] ? kb : (pos / 16) * 16;
       const int page = bt[page_index(kk)];
       live[blk] = live[blk] && page >= 0;
@@ -1114,7 +1143,7 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
 #pragma unroll
       for (int u = 0; u < GROUP; ++u) {
         const int key = kbase + (it0 + u) * KPI + grp;
-        const int kk = (key >= lo && key <= pos) ? key : pos;     // a key that surely has a page
+        const int kk = reads_key(key, lo, pos, keep) ? key : pos;     // a key that surely has a page
         const int page = bt[page_index(kk)];
         kv[u] = bf16x8{};
         if (holds)
@@ -1129,7 +1158,7 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
         for (int i = 0; i < 8; ++i) dot = fmaf(qr[i], static_cast<float>(kv[u][i]), dot);
         dot = group_reduce<LPK>(dot, SumOp());
         if (EXTRAS && bias) dot += bias[min(max(pos - key, 0), ex.span - 1)];
-        sc[it0 + u] = (key >= lo && key <= pos) ? dot : NEG_INF;
+        sc[it0 + u] = reads_key(key, lo, pos, keep) ? dot : NEG_INF;
       }
     }
     float m_c = NEG_INF;
@@ -1186,7 +1215,7 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
       }
     }
     if (n_splits == 1) {
-      if (EXTRAS && ex.sink) L += __expf(-M);      // (a key with score 0 and no value)
+      if (EXTRAS && ex.sink) L += __expf(sink_score(ex, h) - M);      // (a key without a value)
       out[ldo > 0 ? static_cast<size_t>(row) * ldo + h * DH + d : packed_index(row, h * DH + d, H * DH / 32)] =
           from_float<bf16_t>(A / L);
     } else {
@@ -1201,7 +1230,7 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
 
 __global__ void join_kernel(const float* __restrict__ part, bf16_t* __restrict__ out, int ldo,
                             const int32_t* __restrict__ tile_seq, const int32_t* __restrict__ tile_row0, int n_splits,
-                            int H, int DH, int sink) {
+                            int H, int DH, ScoreExtras ex) {
   const int tile = blockIdx.x, h = blockIdx.y;
   if (tile_seq[tile] < 0) return;
   const float* base = part + (static_cast<size_t>(tile) * H + h) * n_splits * (DH + 2);
@@ -1217,7 +1246,7 @@ __global__ void join_kernel(const float* __restrict__ part, bf16_t* __restrict__
         A += ps[2 + d] * f;
       }
     }
-    if (sink) L += __expf(-M);
+    if (ex.sink) L += __expf(sink_score(ex, h) - M);
     out[ldo > 0 ? static_cast<size_t>(tile) * ldo + h * DH + d : packed_index(tile, h * DH + d, H * DH / 32)] =
         from_float<bf16_t>(A / L);
   }
@@ -1235,20 +1264,20 @@ extern "C" int dn_attention_decode(const void* q, int ldq, void* out, int ldo, c
                                    float scale, int window, hipStream_t stream) {
   return dn_attention_decode_extras(q, ldq, out, ldo, k_pool, v_pool, block_tables, max_blocks, tile_seq, tile_row0, tile_pos0,
                                     n_tiles, part, n_splits, chunks, waves, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0,
-                                    stream);
+                                    nullptr, 0, stream);
 }
 
-// With chunks, a bias by distance or a sink: pages of a power of two only.
+// With any of ScoreExtras: pages of a power of two only.
 extern "C" int dn_attention_decode_extras(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                                           const int32_t* block_tables, int max_blocks, const int32_t* tile_seq,
                                           const int32_t* tile_row0, const int32_t* tile_pos0, int n_tiles, float* part,
                                           int n_splits, int chunks, int waves, int H, int Hkv, int dh, int page_size,
                                           float scale, int window, int chunk, const float* bias, int span, int sink,
-                                          hipStream_t stream) {
+                                          const float* sink_at, int keep, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  const bool extras = chunk > 0 || bias != nullptr || sink != 0;
-  if (chunk < 0 || (bias && span < 1)) return DN_ERR_SHAPE;
-  const ScoreExtras ex{chunk, bias, span, sink};
+  const bool extras = chunk > 0 || bias != nullptr || sink != 0 || keep > 0;
+  if (chunk < 0 || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
+  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep};
   if (Hkv < 1 || H % Hkv != 0 || page_size % 16 != 0 || max_blocks < 1 || n_splits < 1 || chunks < 1 ||
       ldq % 8 != 0 || ldo < 0 || (ldo == 0 && (H * dh) % 32 != 0) || reinterpret_cast<uintptr_t>(q) % 16 != 0 || reinterpret_cast<uintptr_t>(k_pool) % 16 != 0 ||
       reinterpret_cast<uintptr_t>(v_pool) % 16 != 0)
@@ -1304,7 +1333,7 @@ extern "C" int dn_attention_decode_extras(const void* q, int ldq, void* out, int
 #undef DN_DECODE_P
   if (n_splits > 1)
     hipLaunchKernelGGL(decode::join_kernel, dim3(n_tiles, H), dim3(64), 0, stream, part, static_cast<bf16_t*>(out),
-                       ldo, tile_seq, tile_row0, n_splits, H, dh, sink);
+                       ldo, tile_seq, tile_row0, n_splits, H, dh, ex);
   return dn_launch_status();
 }
 

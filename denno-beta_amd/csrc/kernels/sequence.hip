@@ -1172,11 +1172,11 @@ __global__ __launch_bounds__(WAVES * 64) void selective_scan_runs_kernel(Selecti
 
 // ---- queries and keys normed as whole vectors, keys and values to the cache -----------------------------------------
 // A row of z is [q: qw | k: kw].  q_out[t] = q / rms(q) * wq; the key that goes to the cache is k / rms(k) * wk, the value
-// k as it is (pools [page][key head][offset][dim] and [page][key head][dim][offset], the row's place from slot_map; a
-// negative place: nothing is written).  One workgroup a row, the sums as in rmsnorm_kernel.
+// k as it is, or (value_normed) the same as the key: a latent that serves as both (pools [page][key head][offset][dim] and
+// [page][key head][dim][offset], the row's place from slot_map; a negative place: nothing is written).  One workgroup a row, the sums as in rmsnorm_kernel.
 __global__ __launch_bounds__(256) void norm_pair_write_kernel(const float* z, size_t ldz, int qw, int kw, const float* wq, const float* wk,
                                                               float eps, void* q_out, size_t ldq, const int* slot_map, void* k_pool,
-                                                              void* v_pool, int dh, int page_size, int dt, int write) {
+                                                              void* v_pool, int dh, int page_size, int dt, int write, int value_normed) {
   __shared__ float sh[4];
   const size_t t = blockIdx.x;
   const float* row = z + t * ldz;
@@ -1193,9 +1193,195 @@ __global__ __launch_bounds__(256) void norm_pair_write_kernel(const float* z, si
   for (int c = threadIdx.x; c < kw; c += 256) {
     const int h = c / dh, d = c % dh;
     const size_t base = (static_cast<size_t>(page) * Hkv + h) * page_size * dh;
-    const float k = row[qw + c];
-    store_as(k_pool, base + static_cast<size_t>(off) * dh + d, dt, k * ik * wk[c]);
-    store_as(v_pool, base + static_cast<size_t>(d) * page_size + off, dt, k);
+    const float k = row[qw + c], kn = k * ik * wk[c];
+    store_as(k_pool, base + static_cast<size_t>(off) * dh + d, dt, kn);
+    store_as(v_pool, base + static_cast<size_t>(d) * page_size + off, dt, value_normed ? kn : k);
+  }
+}
+
+// ---- heads' queries, keys and values: normed, turned, to their places ------------------------------------------------
+// A row of z is [q: H x dk | k: G x dk | v: G x dv].  Each query and key is divided by its root mean square (eps inside the
+// root; eps < 0: it is not) and weighed entry by entry (wq, wk: dk numbers shared by the heads), then its first `dims` entries are turned in
+// neighbouring pairs by position * freq; a value's first v_dims entries are turned by position * v_freq.  A query times
+// q_scale[head] goes to q_out (heads `kept` columns wide), keys and values to the cache's pools (heads `kept` wide, the row's
+// place from slot_map; a negative place: nothing is written); columns a vector does not have are zeros.  A wave a vector: a
+// lane holds the pairs lane and lane + 64, the squares are summed over the wave in one order.
+struct NormTurnArgs {
+  const float* z;
+  size_t ldz;
+  int H, G, dk, dv;
+  const float *wq, *wk, *q_scale;      // (each may be none)
+  float eps;
+  const float* freq;
+  int dims;
+  const float* v_freq;
+  int v_dims;
+  const int* positions;
+  void* q_out;
+  size_t ldq;
+  int kept;
+  const int* slot_map;
+  void *k_pool, *v_pool;
+  int page_size, dt, write;
+};
+
+// two neighbours from an even place
+__device__ __forceinline__ void store_pair(void* p, size_t i, int dt, float a, float b) {
+  if (dt == DN_F32) {
+    typedef __attribute__((__vector_size__(2 * sizeof(float)))) float f32x2;
+    *reinterpret_cast<f32x2*>(static_cast<float*>(p) + i) = f32x2{a, b};
+  } else {
+    *reinterpret_cast<uint32_t*>(static_cast<bf16_t*>(p) + i) =
+        static_cast<uint32_t>(from_float<bf16_t>(a).bits) | (static_cast<uint32_t>(from_float<bf16_t>(b).bits) << 16);
+  }
+}
+
+__global__ __launch_bounds__(256) void norm_turn_write_kernel(NormTurnArgs a) {
+  __shared__ float cs[256], sn[256];      // the row's angles: the keys' pairs, then the values' (at most 128 each)
+  const size_t t = blockIdx.x;
+  const int lane = threadIdx.x & 63;
+  const int half = a.dims / 2, v_half = a.v_dims / 2, n_vec = a.H + 2 * a.G;
+  const float p = static_cast<float>(a.positions[t]);
+  if (threadIdx.x < half + v_half) {
+    const float ang = p * (threadIdx.x < half ? a.freq[threadIdx.x] : a.v_freq[threadIdx.x - half]);
+    cs[threadIdx.x] = cosf(ang), sn[threadIdx.x] = sinf(ang);
+  }
+  __syncthreads();
+  const int slot = a.slot_map[t];
+  const bool writes = a.write && slot >= 0;
+  const int page = writes ? slot / a.page_size : 0, off = writes ? slot % a.page_size : 0;
+  for (int vec = blockIdx.y * 4 + (threadIdx.x >> 6); vec < n_vec; vec += gridDim.y * 4) {      // (the whole wave)
+    const bool is_q = vec < a.H, is_v = vec >= a.H + a.G;
+    if (!is_q && !writes) continue;
+    const int n = is_q ? vec : (is_v ? vec - a.H - a.G : vec - a.H);      // the head's number among its kind
+    const int width = is_v ? a.dv : a.dk, turned = is_v ? v_half : half, base = is_v ? half : 0;
+    const float* src = a.z + t * a.ldz + (is_v ? static_cast<size_t>(a.H + a.G) * a.dk + static_cast<size_t>(n) * a.dv
+                                               : static_cast<size_t>(vec) * a.dk);
+    const float* w = is_q ? a.wq : (is_v ? nullptr : a.wk);
+    float lo[2], hi[2], ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      const int e = 2 * (lane + 64 * j);
+      lo[j] = e < width ? src[e] : 0.f;
+      hi[j] = e + 1 < width ? src[e + 1] : 0.f;
+      ss = fmaf(lo[j], lo[j], ss);
+      ss = fmaf(hi[j], hi[j], ss);
+    }
+    const float inv = is_v || a.eps < 0.f ? 1.0f : 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(width) + a.eps);
+    const float times = is_q && a.q_scale ? a.q_scale[n] : 1.0f;
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      const int i = lane + 64 * j, e = 2 * i;
+      if (e >= a.kept) continue;
+      float x = lo[j], y = hi[j];
+      if (!is_v) {
+        x *= inv, y *= inv;
+        if (w) {
+          if (e < width) x *= w[e];
+          if (e + 1 < width) y *= w[e + 1];
+        }
+      }
+      if (i < turned) {
+        const float c = cs[base + i], s = sn[base + i];
+        const float u = x * c - y * s;
+        y = y * c + x * s;
+        x = u;
+      }
+      if (is_q) {
+        store_pair(a.q_out, t * a.ldq + static_cast<size_t>(n) * a.kept + e, a.dt, x * times, y * times);
+      } else {
+        const size_t head = (static_cast<size_t>(page) * a.G + n) * a.page_size * a.kept;
+        if (is_v) {
+          store_as(a.v_pool, head + static_cast<size_t>(e) * a.page_size + off, a.dt, x);
+          store_as(a.v_pool, head + static_cast<size_t>(e + 1) * a.page_size + off, a.dt, y);
+        } else {
+          store_pair(a.k_pool, head + static_cast<size_t>(off) * a.kept + e, a.dt, x, y);
+        }
+      }
+    }
+  }
+}
+
+// An attention's result on its way to the output projection: head h of row t (head_stride columns apart, dv of them used) has
+// its neighbouring pairs turned back by position * freq (freq: dv / 2 numbers, or none) and is multiplied entry by entry with
+// sigmoid(gate[t, h * dv + d]) (gate: or none); the heads lie side by side in out.
+__global__ __launch_bounds__(256) void turn_back_gate_kernel(const void* o, int o_dt, size_t ldo, int head_stride, const float* gate,
+                                                             size_t ldg, const float* freq, const int* positions, void* out, int out_dt,
+                                                             size_t ldout, int n_heads, int dv) {
+  __shared__ float cs[128], sn[128];
+  const size_t t = blockIdx.x;
+  const int per = (dv + 1) / 2;      // pairs of a head (the last of an odd one is a single entry: nothing is turned then)
+  if (freq) {
+    if (threadIdx.x < per) {
+      const float ang = static_cast<float>(positions[t]) * freq[threadIdx.x];
+      cs[threadIdx.x] = cosf(ang), sn[threadIdx.x] = sinf(ang);
+    }
+    __syncthreads();
+  }
+  for (int i = blockIdx.y * 256 + threadIdx.x; i < n_heads * per; i += gridDim.y * 256) {
+    const int h = i / per, m = i % per, d = 2 * m;
+    const bool two = d + 1 < dv;
+    const size_t src = t * ldo + static_cast<size_t>(h) * head_stride + d;
+    float x = load_as(o, src, o_dt), y = two ? load_as(o, src + 1, o_dt) : 0.f;
+    if (freq) {
+      const float c = cs[m], s = sn[m];
+      const float u = x * c + y * s;
+      y = y * c - x * s;
+      x = u;
+    }
+    const size_t col = static_cast<size_t>(h) * dv + d;
+    if (gate) {
+      const float* g = gate + t * ldg + col;
+      x *= 1.0f / (1.0f + expf(-g[0]));
+      if (two) y *= 1.0f / (1.0f + expf(-g[1]));
+    }
+    store_as(out, t * ldout + col, out_dt, x);
+    if (two) store_as(out, t * ldout + col + 1, out_dt, y);
+  }
+}
+
+// ---- a polynomial of normed powers ----------------------------------------------------------------------------------
+// out = a N(z) + b N(z^2) + c N(z^3) + e with (a, b, c, e) the four numbers, powers entry by entry, N the division of a row by its
+// root mean square (eps inside the root).  One workgroup a row; up to 256 NC columns a thread holds its share of the row (NC 0:
+// it reads it twice); a thread sums its own columns in ascending order, waves are joined in order.
+template <int NC>
+__global__ __launch_bounds__(256) void poly_norm_kernel(const float* z, size_t ldz, const float* numbers, float eps, void* out, int out_dt,
+                                                        size_t ldo, int n) {
+  __shared__ float sh[3][4];
+  const float* row = z + static_cast<size_t>(blockIdx.x) * ldz;
+  constexpr int HELD = NC > 0 ? NC : 1;
+  float v[HELD];
+  float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+  auto add = [&](float x) {
+    const float x2 = x * x, x3 = x2 * x;
+    s1 = fmaf(x, x, s1), s2 = fmaf(x2, x2, s2), s3 = fmaf(x3, x3, s3);
+  };
+  if constexpr (NC > 0) {
+#pragma unroll
+    for (int k = 0; k < NC; ++k) {
+      const int c = threadIdx.x + 256 * k;
+      v[k] = c < n ? row[c] : 0.f;
+    }
+#pragma unroll
+    for (int k = 0; k < NC; ++k) add(v[k]);
+  } else {
+    for (int c = threadIdx.x; c < n; c += 256) add(row[c]);
+  }
+  s1 = wave_sum(s1), s2 = wave_sum(s2), s3 = wave_sum(s3);
+  const int wave = threadIdx.x >> 6;
+  if ((threadIdx.x & 63) == 0) sh[0][wave] = s1, sh[1][wave] = s2, sh[2][wave] = s3;
+  __syncthreads();
+  const float len = static_cast<float>(n);
+  auto factor = [&](int i) { return numbers[i] / sqrtf(((sh[i][0] + sh[i][1]) + (sh[i][2] + sh[i][3])) / len + eps); };
+  const float f1 = factor(0), f2 = factor(1), f3 = factor(2), e = numbers[3];
+  const size_t dst = static_cast<size_t>(blockIdx.x) * ldo;
+  auto put = [&](int c, float x) { store_as(out, dst + c, out_dt, fmaf(x, fmaf(x, fmaf(x, f3, f2), f1), e)); };
+  if constexpr (NC > 0) {
+#pragma unroll
+    for (int k = 0; k < NC; ++k)
+      if (threadIdx.x + 256 * k < n) put(threadIdx.x + 256 * k, v[k]);
+  } else {
+    for (int c = threadIdx.x; c < n; c += 256) put(c, row[c]);
   }
 }
 
@@ -1669,12 +1855,61 @@ int dn_streams_write(float* xs, long long plane, int n, const float* mix, const 
 
 int dn_norm_pair_write(const float* z, long long ldz, int qw, int kw, const float* wq, const float* wk, float eps, void* q_out,
                        long long ldq, const int* slot_map, void* k_pool, void* v_pool, int T, int Hkv, int dh, int page_size,
-                       int dt, int write, hipStream_t stream) {
+                       int dt, int write, int value_normed, hipStream_t stream) {
   if (!float_kind(dt)) return DN_ERR_DTYPE;
   if (qw < 1 || kw != Hkv * dh || page_size < 1 || ldz < qw + kw || ldq < qw) return DN_ERR_SHAPE;
   if (T == 0) return 0;
   hipLaunchKernelGGL(norm_pair_write_kernel, dim3(T), dim3(256), 0, stream, z, static_cast<size_t>(ldz), qw, kw, wq, wk, eps, q_out,
-                     static_cast<size_t>(ldq), slot_map, k_pool, v_pool, dh, page_size, dt, write);
+                     static_cast<size_t>(ldq), slot_map, k_pool, v_pool, dh, page_size, dt, write, value_normed);
+  return dn_launch_status();
+}
+
+int dn_norm_turn_write(const float* z, long long ldz, int H, int G, int dk, int dv, const float* wq, const float* wk, const float* q_scale,
+                       float eps, const float* freq, int dims, const float* v_freq, int v_dims, const int* positions, void* q_out,
+                       long long ldq, int kept, const int* slot_map, void* k_pool, void* v_pool, int T, int page_size, int dt, int write,
+                       hipStream_t stream) {
+  if (!float_kind(dt)) return DN_ERR_DTYPE;
+  if (H < 1 || G < 1 || dk < 1 || dv < 1 || kept > 256 || kept % 2 != 0 || dk > kept || dv > kept || dims < 0 || dims % 2 != 0 || dims > dk ||
+      v_dims < 0 || v_dims % 2 != 0 || v_dims > dv || (dims > 0 && !freq) || (v_dims > 0 && !v_freq) || page_size < 1 ||
+      ldz < static_cast<long long>(H + G) * dk + static_cast<long long>(G) * dv || ldq < static_cast<long long>(H) * kept || ldq % 2 != 0 ||
+      reinterpret_cast<uintptr_t>(q_out) % 8 != 0 || reinterpret_cast<uintptr_t>(k_pool) % 8 != 0)
+    return DN_ERR_SHAPE;
+  if (T == 0) return 0;
+  const NormTurnArgs a{z, static_cast<size_t>(ldz), H, G, dk, dv, wq, wk, q_scale, eps, freq, dims, v_freq, v_dims, positions, q_out,
+                       static_cast<size_t>(ldq), kept, slot_map, k_pool, v_pool, page_size, dt, write};
+  // (few rows: four vectors a workgroup, so that a step of decoded tokens is more than a handful of workgroups; many rows: one
+  // workgroup a row, whose angles are made once)
+  const int groups = (H + 2 * G + 3) / 4;
+  hipLaunchKernelGGL(norm_turn_write_kernel, dim3(T, T <= 256 ? groups : 1), dim3(256), 0, stream, a);
+  return dn_launch_status();
+}
+
+int dn_turn_back_gate(const void* o, int o_dt, long long ldo, int head_stride, const float* gate, long long ldg, const float* freq,
+                      const int* positions, void* out, int out_dt, long long ldout, int T, int n_heads, int dv, hipStream_t stream) {
+  if (!float_kind(o_dt) || !float_kind(out_dt)) return DN_ERR_DTYPE;
+  if (n_heads < 1 || dv < 1 || dv > 256 || (freq && dv % 2 != 0) || head_stride < dv || ldo < static_cast<long long>(n_heads - 1) * head_stride + dv ||
+      (gate && ldg < static_cast<long long>(n_heads) * dv) || ldout < static_cast<long long>(n_heads) * dv)
+    return DN_ERR_SHAPE;
+  if (T == 0) return 0;
+  const int total = n_heads * ((dv + 1) / 2);
+  hipLaunchKernelGGL(turn_back_gate_kernel, dim3(T, T <= 256 ? (total + 255) / 256 : 1), dim3(256), 0, stream, o, o_dt,
+                     static_cast<size_t>(ldo), head_stride, gate, static_cast<size_t>(ldg), freq, positions, out, out_dt,
+                     static_cast<size_t>(ldout), n_heads, dv);
+  return dn_launch_status();
+}
+
+int dn_poly_norm(const float* z, long long ldz, const float* numbers, float eps, void* out, int out_dt, long long ldo, int T, int n,
+                 hipStream_t stream) {
+  if (!float_kind(out_dt)) return DN_ERR_DTYPE;
+  if (n < 1 || ldz < n || ldo < n) return DN_ERR_SHAPE;
+  if (T == 0) return 0;
+#define DN_POLY(NC)                                                                                                     \
+  hipLaunchKernelGGL(poly_norm_kernel<NC>, dim3(T), dim3(256), 0, stream, z, static_cast<size_t>(ldz), numbers, eps, out, out_dt, \
+                     static_cast<size_t>(ldo), n)
+  if (n <= 1024) DN_POLY(4);
+  else if (n <= 4096) DN_POLY(16);
+  else DN_POLY(0);
+#undef DN_POLY
   return dn_launch_status();
 }
 

@@ -120,10 +120,10 @@ def _declare(name, lib):
             "dn_attention": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P],
             "dn_attention_rows": [P, I, P, I, P, P, P, I, P, P, I, P, I, I, I, I, I, F, I, I, P],
             "dn_attention_rows_tile": [I],
-            "dn_attention_extras": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P, I, I, I, P],
-            "dn_attention_rows_extras": [P, I, P, I, P, P, P, I, P, P, I, P, I, I, I, I, I, F, I, I, P, I, I, I, P],
-            "dn_attention_flash_extras": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P, I, I, P],
-            "dn_attention_decode_extras": [P, I, P, I, P, P, P, I, P, P, P, I, P, I, I, I, I, I, I, I, F, I, I, P, I, I, P],
+            "dn_attention_extras": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P, I, I, P, I, I, P],
+            "dn_attention_rows_extras": [P, I, P, I, P, P, P, I, P, P, I, P, I, I, I, I, I, F, I, I, P, I, I, P, I, I, P],
+            "dn_attention_flash_extras": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P, I, I, P, I, P],
+            "dn_attention_decode_extras": [P, I, P, I, P, P, P, I, P, P, P, I, P, I, I, I, I, I, I, I, F, I, I, P, I, I, P, I, P],
             "dn_attention_flash": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, P],
             "dn_attention_decode": [P, I, P, I, P, P, P, I, P, P, P, I, P, I, I, I, I, I, I, I, F, I, P],
         },
@@ -148,7 +148,10 @@ def _declare(name, lib):
             "dn_gate_scan": [P, c_longlong, P, c_longlong, P, c_longlong, P, P, P, c_longlong, P, P, I, I, I, P, I, c_longlong, P],
             "dn_streams_read": [P, c_longlong, I, P, P, F, P, I, c_longlong, P, I, I, P],
             "dn_streams_write": [P, c_longlong, I, P, P, P, c_longlong, P, c_longlong, P, P, F, P, P, F, P, I, c_longlong, I, I, P],
-            "dn_norm_pair_write": [P, c_longlong, I, I, P, P, F, P, c_longlong, P, P, P, I, I, I, I, I, I, P],
+            "dn_norm_pair_write": [P, c_longlong, I, I, P, P, F, P, c_longlong, P, P, P, I, I, I, I, I, I, I, P],
+            "dn_norm_turn_write": [P, c_longlong, I, I, I, I, P, P, P, F, P, I, P, I, P, P, c_longlong, I, P, P, P, I, I, I, I, P],
+            "dn_turn_back_gate": [P, I, c_longlong, I, P, c_longlong, P, P, P, I, c_longlong, I, I, I, P],
+            "dn_poly_norm": [P, c_longlong, P, F, P, I, c_longlong, I, I, P],
             "dn_head_gate": [P, I, c_longlong, I, P, c_longlong, P, I, c_longlong, I, I, I, P],
             "dn_token_input": [P, c_longlong, P, P, I, P, I, c_longlong, I, P, I, P, I, I, I, F, P, F, P, I, c_longlong, P],
             "dn_rows_times_table": [P, I, c_longlong, P, I, c_longlong, I, P, I, P, I, c_longlong, I, I, P],
@@ -619,7 +622,7 @@ def attention_writes_packed(dtype, page_size, head_dim, single_rows, max_context
 
 
 def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, window=0, tiles_wide=None,
-              single_rows=False, max_context=0, decode_waves=None, chunk=0, bias=None, sink=False):
+              single_rows=False, max_context=0, decode_waves=None, chunk=0, bias=None, sink=False, keep_first=0):
     """Causal attention of the batch's rows over the paged cache.
 
     q: [T, >= H*dh] rows contiguous, head h at columns h*dh..; out: [T, H*dh];
@@ -632,7 +635,9 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
 
     chunk > 0: the row at position p reads only the keys from p // chunk * chunk on (runs of `chunk` positions counted from
     the request's first); bias: 32-bit [H, span], bias[h, p - key] is added to the scaled score (distances from span on
-    take the last entry); sink: one more summand exp(0) under the softmax (a key with score 0 and no value).
+    take the last entry); sink: True: one more summand exp(0) under the softmax (a key with score 0 and no value), or 32-bit [H]:
+    head h's summand is exp(sink[h]), which nothing scales; keep_first: with a window, the request's first so many keys are
+    read by every row as well.
 
     Three kernels: 32-bit takes the plain one; bfloat16 takes the MFMA kernel over tiles_wide, or,
     for a pure decode step, the split kernel (with both, out may be packed rows); a head size that
@@ -656,7 +661,11 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
     _need(1 <= dh <= 256, lambda: f"attention: head size {dh} must be at most 256")
     _need(n_heads % Hkv == 0, lambda: f"attention: {n_heads} heads over {Hkv} key heads")
     ldq, ldo = _rows(q, "q"), (0 if out_packed else _rows(out, "out"))
-    extras = chunk > 0 or bias is not None or bool(sink)
+    sink_at, sink = (sink, True) if isinstance(sink, torch.Tensor) else (None, bool(sink))
+    _f32vec(sink_at, "sink", n_heads)
+    keep_first = int(keep_first) if window > 0 else 0      # (without a window every key is read anyway)
+    _need(keep_first >= 0 and not (keep_first and chunk), "attention: kept first keys go with a window and not with chunks")
+    extras = chunk > 0 or bias is not None or sink or keep_first > 0
     span = 0
     if bias is not None:
         _dev(bias, "bias", (torch.float32,), 2)
@@ -665,7 +674,7 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
     _need(chunk >= 0, "attention: chunk")
     lib = _lib("attention")
     # (the kernel for portions takes the largest score for the largest product: a scale that is not positive goes the plain way)
-    # (with chunks, a bias or a sink the two bfloat16 kernels take pages of a power of two)
+    # (with chunks, a bias, a sink or kept first keys the two bfloat16 kernels take pages of a power of two)
     fast = (q.dtype == torch.bfloat16 and ps % 16 == 0 and ldq % 8 == 0 and q.data_ptr() % 16 == 0 and scale > 0
             and (not extras or ps & (ps - 1) == 0))
     decode = fast and decode_attention_applies(q.dtype, ps, dh, single_rows, max_context)
@@ -703,8 +712,8 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
         _ok(lib.dn_attention_decode_extras(
             q.data_ptr(), ldq, out.data_ptr(), ldo, k_pool.data_ptr(), v_pool.data_ptr(), block_tables.data_ptr(),
             block_tables.shape[1], base, base + 4 * n_tiles, base + 12 * n_tiles, n_tiles, part.data_ptr(), n_splits,
-            chunks, waves, n_heads, Hkv, dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(bool(sink)),
-            _stream()), "attention (decode)")
+            chunks, waves, n_heads, Hkv, dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(sink),
+            _ptr(sink_at), keep_first, _stream()), "attention (decode)")
         return out
     if fast and tiles_wide is not None and dh in FLASH_HEAD_DIMS:
         _dev(tiles_wide, "tiles_wide", _I32, 2)
@@ -714,8 +723,8 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
         _ok(lib.dn_attention_flash_extras(
             q.data_ptr(), ldq, out.data_ptr(), ldo, k_pool.data_ptr(), v_pool.data_ptr(), block_tables.data_ptr(),
             block_tables.shape[1], base, base + 4 * n_tiles, base + 8 * n_tiles, base + 12 * n_tiles, n_tiles,
-            n_heads, Hkv, dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(bool(sink)), _stream()),
-            "attention (flash)")
+            n_heads, Hkv, dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(sink), _ptr(sink_at),
+            keep_first, _stream()), "attention (flash)")
         return out
     n_tiles = tiles.shape[1]
     base = tiles.data_ptr()
@@ -729,14 +738,14 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
         _ok(lib.dn_attention_rows_extras(
             q.data_ptr(), ldq, out.data_ptr(), ldo, k_pool.data_ptr(), v_pool.data_ptr(), block_tables.data_ptr(),
             block_tables.shape[1], base, base + 12 * n_tiles, n_tiles, part.data_ptr(), int(max_context), n_heads, Hkv,
-            dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(bool(sink)), _CODE[q.dtype], _stream()),
-            "attention (single rows)")
+            dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(sink), _ptr(sink_at), keep_first, _CODE[q.dtype],
+            _stream()), "attention (single rows)")
         return out
     _ok(lib.dn_attention_extras(
         q.data_ptr(), ldq, out.data_ptr(), ldo, k_pool.data_ptr(), v_pool.data_ptr(), block_tables.data_ptr(),
         block_tables.shape[1], base, base + 4 * n_tiles, base + 8 * n_tiles, base + 12 * n_tiles, n_tiles,
-        n_heads, Hkv, dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(bool(sink)), _CODE[q.dtype],
-        _stream()), "attention")
+        n_heads, Hkv, dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(sink), _ptr(sink_at), keep_first,
+        _CODE[q.dtype], _stream()), "attention")
     return out
 
 
@@ -1441,10 +1450,10 @@ def streams_write(xs, y, mix, w_out, next_in=None, weight=None, eps=0.0, out=Non
     return out
 
 
-def norm_pair_write(z, q_width, wq, wk, eps, q_out, slot_map, k_pool, v_pool, write=True):
+def norm_pair_write(z, q_width, wq, wk, eps, q_out, slot_map, k_pool, v_pool, write=True, value_normed=False):
     """A row of z (32-bit) is [q: q_width | k: the rest].  q_out = q / sqrt(mean(q^2) + eps) * wq; the key that goes to the cache
     (k_pool [pages, Hkv, page, dh]) is k / sqrt(mean(k^2) + eps) * wk, each normed as one vector over all heads; the value
-    (v_pool [pages, Hkv, dh, page]) is k as it is.  slot_map: int32 [T], page * page_size + offset, negative: not written."""
+    (v_pool [pages, Hkv, dh, page]) is k as it is, or (value_normed) the key over again.  slot_map: int32 [T], page * page_size + offset, negative: not written."""
     _dev(z, "z", (torch.float32,), 2), _dev(q_out, "q_out", _FLOATS, 2), _dev(slot_map, "slot_map", _I32, 1)
     _dev(k_pool, "k_pool", (q_out.dtype,), 4), _dev(v_pool, "v_pool", (q_out.dtype,), 4)
     T = z.shape[0]
@@ -1456,9 +1465,67 @@ def norm_pair_write(z, q_width, wq, wk, eps, q_out, slot_map, k_pool, v_pool, wr
     _f32vec(wq, "wq", q_width), _f32vec(wk, "wk", kw)
     _ok(_lib("sequence").dn_norm_pair_write(z.data_ptr(), _rows(z, "z"), q_width, kw, wq.data_ptr(), wk.data_ptr(), float(eps),
                                             q_out.data_ptr(), _rows(q_out, "q_out"), slot_map.data_ptr(), k_pool.data_ptr(),
-                                            v_pool.data_ptr(), T, Hkv, dh, ps, _CODE[q_out.dtype], int(bool(write)), _stream()),
-        "norm_pair_write")
+                                            v_pool.data_ptr(), T, Hkv, dh, ps, _CODE[q_out.dtype], int(bool(write)), int(bool(value_normed)),
+                                            _stream()), "norm_pair_write")
     return q_out
+
+
+def norm_turn_write(z, n_heads, n_kv, dk, dv, positions, q_out, slot_map, k_pool, v_pool, wq=None, wk=None, eps=None, q_scale=None,
+                    freq=None, v_freq=None, write=True):
+    """A row of z (32-bit) begins with [q: n_heads x dk | k: n_kv x dk | v: n_kv x dv].  Every query and key is x / sqrt(mean(x^2) + eps)
+    (eps None: x) times wq or wk (dk numbers shared by the heads, or None), then its first 2 len(freq) entries are turned in pairs (2i, 2i + 1) by
+    positions[t] * freq[i]; a value's first 2 len(v_freq) entries likewise.  Queries times q_scale[head] go to q_out (heads side by
+    side, as wide as the pools' keys), keys to k_pool [pages, n_kv, page, width], values to v_pool [pages, n_kv, width, page];
+    the columns a vector does not have are zeros.  slot_map as in norm_pair_write.  One launch."""
+    _dev(z, "z", (torch.float32,), 2), _dev(q_out, "q_out", _FLOATS, 2), _dev(slot_map, "slot_map", _I32, 1), _dev(positions, "positions", _I32, 1)
+    _dev(k_pool, "k_pool", (q_out.dtype,), 4), _dev(v_pool, "v_pool", (q_out.dtype,), 4)
+    T = z.shape[0]
+    n_pages, Hkv, ps, kept = k_pool.shape
+    _need(Hkv == n_kv and z.shape[1] >= (n_heads + n_kv) * dk + n_kv * dv and tuple(q_out.shape) == (T, n_heads * kept)
+          and max(dk, dv) <= kept <= 256 and kept % 2 == 0, "norm_turn_write: shapes")
+    _need(slot_map.is_contiguous() and slot_map.shape[0] == T and positions.is_contiguous() and positions.shape[0] == T, "norm_turn_write: rows")
+    _need(k_pool.is_contiguous() and v_pool.is_contiguous() and tuple(v_pool.shape) == (n_pages, Hkv, kept, ps), "norm_turn_write: pools")
+    _f32vec(wq, "wq", dk), _f32vec(wk, "wk", dk), _f32vec(q_scale, "q_scale", n_heads), _f32vec(freq, "freq"), _f32vec(v_freq, "v_freq")
+    dims, v_dims = (0 if f is None else 2 * f.numel() for f in (freq, v_freq))
+    _need(dims <= dk and v_dims <= dv, "norm_turn_write: more turned entries than a vector has")
+    _ok(_lib("sequence").dn_norm_turn_write(z.data_ptr(), _rows(z, "z"), n_heads, n_kv, dk, dv, _ptr(wq), _ptr(wk), _ptr(q_scale),
+                                            -1.0 if eps is None else float(eps), _ptr(freq), dims, _ptr(v_freq), v_dims, positions.data_ptr(), q_out.data_ptr(),
+                                            _rows(q_out, "q_out"), kept, slot_map.data_ptr(), k_pool.data_ptr(), v_pool.data_ptr(), T, ps,
+                                            _CODE[q_out.dtype], int(bool(write)), _stream()), "norm_turn_write")
+    return q_out
+
+
+def turn_back_gate(o, n_heads, dv, out, positions=None, freq=None, gate=None, head_stride=None):
+    """out[t, h * dv + d] = r[d] * sigmoid(gate[t, h * dv + d]), r being o's head h of row t (head_stride columns apart, None: dv) with
+    its pairs (2m, 2m + 1) turned by -positions[t] * freq[m] (freq: dv / 2 numbers, None: as it is; gate: 32-bit, None: none)."""
+    _dev(o, "o", _FLOATS, 2), _dev(out, "out", _FLOATS, 2)
+    T = o.shape[0]
+    hs = dv if head_stride is None else head_stride
+    _need(1 <= dv <= 256 and hs >= dv and n_heads >= 1 and o.shape[1] >= (n_heads - 1) * hs + dv and tuple(out.shape) == (T, n_heads * dv),
+          "turn_back_gate: shapes")
+    if gate is not None:
+        _dev(gate, "gate", (torch.float32,), 2)
+        _need(tuple(gate.shape) == (T, n_heads * dv), "turn_back_gate: gate")
+    if freq is not None:
+        _dev(positions, "positions", _I32, 1)
+        _f32vec(freq, "freq", dv // 2)
+        _need(dv % 2 == 0 and positions.is_contiguous() and positions.shape[0] == T, "turn_back_gate: pairs or rows")
+    _ok(_lib("sequence").dn_turn_back_gate(o.data_ptr(), _CODE[o.dtype], _rows(o, "o"), hs, _ptr(gate), _rows(gate, "gate") if gate is not None else 0,
+                                           _ptr(freq), _ptr(positions) if freq is not None else 0, out.data_ptr(), _CODE[out.dtype],
+                                           _rows(out, "out"), T, n_heads, dv, _stream()), "turn_back_gate")
+    return out
+
+
+def poly_norm(z, numbers, eps, out):
+    """out = a N(z) + b N(z^2) + c N(z^3) + e with (a, b, c, e) = numbers (32-bit), powers entry by entry, N(v) = v / sqrt(mean(v^2) + eps)
+    over the row; z 32-bit."""
+    _dev(z, "z", (torch.float32,), 2), _dev(out, "out", _FLOATS, 2)
+    T, n = z.shape
+    _need(tuple(out.shape) == (T, n), "poly_norm: shapes")
+    _f32vec(numbers, "numbers", 4)
+    _ok(_lib("sequence").dn_poly_norm(z.data_ptr(), _rows(z, "z"), numbers.data_ptr(), float(eps), out.data_ptr(), _CODE[out.dtype],
+                                      _rows(out, "out"), T, n, _stream()), "poly_norm")
+    return out
 
 
 # -- a matrix per head, a matrix per expert (csrc/kernels/grouped.hip) -----------------------------------------------------

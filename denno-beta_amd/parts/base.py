@@ -35,7 +35,8 @@ from ..weights.spec import ParamSpec
 
 @dataclass(frozen=True)
 class PagedKV:
-    """A mixer that keeps keys and values of `window` last positions (0: all) in pages.
+    """A mixer that keeps keys and values of `window` last positions (0: all) in pages; keep_first: and those of the first
+    so many positions, for as long as the request lives.
     dtype: what the pages hold ("bfloat16", "float32"); None: the engine's activation dtype.
     head_dim is the width of a key; value_dim that of a value (None: the same).  The pools are laid out for
     both ([.., Hkv, page, head_dim] and [.., Hkv, value_dim, page]); the attention kernels of this package
@@ -46,6 +47,7 @@ class PagedKV:
     window: int = 0
     dtype: Optional[str] = None
     value_dim: Optional[int] = None
+    keep_first: int = 0
 
     @property
     def v_dim(self) -> int:

@@ -10,7 +10,7 @@ from .linear import Linear
 
 ACTIVATION_EPILOGUES = {"gelu_tanh": "gelu_tanh", "gelu_erf": "gelu_erf"}
 # activations with numbers of their own in a tensor: a kernel between the two products, on the first one's 32-bit result
-ACTIVATION_KERNELS = ("xielu",)
+ACTIVATION_KERNELS = {"xielu": 2, "poly_norm": 4}      # -> how many numbers
 F32 = torch.float32
 
 
@@ -21,32 +21,38 @@ class DenseMLP(Part):
     product's epilogue, in 32-bit, before the rounding to the activation dtype.
 
     activation "xielu": z > 0: softplus(p) z^2 + z / 2; else (1/2 + softplus(q)) (e^z - 1 - z) + z / 2, with (p, q) the two
-    numbers of the tensor `activation_params`; it runs as a kernel of its own on the first product's 32-bit result."""
+    numbers of the tensor `activation_params`; it runs as a kernel of its own on the first product's 32-bit result.
+    activation "poly_norm": a N(z) + b N(z^2) + c N(z^3) + e over the row of `inner` values, (a, b, c, e) the tensor's four numbers,
+    powers entry by entry, N(v) = v / sqrt(mean(v^2) + eps); likewise a kernel of its own."""
     graph_safe = True
     returns_rows = True
 
     def __init__(self, width: int, inner: int, activation: str, up_weight: str, up_bias, down_weight: str,
-                 down_bias, stored_in_out: bool = False, down_init_std: float = 0.02, activation_params=None):
+                 down_bias, stored_in_out: bool = False, down_init_std: float = 0.02, activation_params=None, eps: float = 0.0):
         if activation not in ACTIVATION_EPILOGUES and activation not in ACTIVATION_KERNELS:
             raise ValueError(f"activation {activation!r}; known: {sorted(ACTIVATION_EPILOGUES) + list(ACTIVATION_KERNELS)}")
         if (activation in ACTIVATION_KERNELS) != (activation_params is not None):
             raise ValueError(f"activation {activation!r}: the tensor of its numbers is " +
                              ("missing" if activation_params is None else "not used"))
         self.width, self.inner, self.activation, self.activation_params = width, inner, activation, activation_params
+        self.eps = float(eps)
         if activation in ACTIVATION_KERNELS:
             self.libraries = ("sequence",)
         self.up = Linear(width, inner, up_weight, up_bias, stored_in_out)
         self.down = Linear(inner, width, down_weight, down_bias, stored_in_out, down_init_std)
 
     def param_specs(self):
-        own = [ParamSpec(self.activation_params, (2,), "vector", ("normal", 0.3, 0.3))] if self.activation_params else []
+        n = ACTIVATION_KERNELS.get(self.activation)
+        own = [ParamSpec(self.activation_params, (n,), "vector", ("normal", 0.3, 0.3))] if self.activation_params else []
         return self.up.param_specs() + self.down.param_specs() + own
 
     def bind(self, tensors, runtime):
         super().bind(tensors, runtime)
         self.up.bind(tensors)
         self.down.bind(tensors)
-        if self.activation_params:
+        if self.activation == "poly_norm":
+            self.act_numbers = tensors[self.activation_params].contiguous()
+        elif self.activation_params:
             pq = tensors[self.activation_params].to(F32)
             sp = torch.nn.functional.softplus(pq)
             self.act_numbers = torch.stack([sp[0], 0.5 + sp[1]]).contiguous()      # (softplus(p), 1/2 + softplus(q)), once
@@ -70,8 +76,11 @@ class DenseMLP(Part):
         n = h.shape[0]
         if self.activation in ACTIVATION_KERNELS:
             z = self.up(h, out_dtype=F32)
-            f = ops.activate(z, self.activation, torch.empty(z.shape, dtype=self.runtime.act_dtype, device=z.device),
-                             lower=self.act_numbers)
+            f = torch.empty(z.shape, dtype=self.runtime.act_dtype, device=z.device)
+            if self.activation == "poly_norm":
+                ops.poly_norm(z, self.act_numbers, self.eps, f)
+            else:
+                ops.activate(z, self.activation, f, lower=self.act_numbers)
         else:
             f = self.up(h, out_dtype=self.runtime.act_dtype, epilogue=ACTIVATION_EPILOGUES[self.activation],
                         packed_out=self.up.few_rows(n) and self.down.packed_input(n) and accumulate_into is not None)
@@ -140,14 +149,15 @@ class RoutedExperts(Part):
     shared: an expert of the same form that every token uses, dict(inner, gate, up, down, token_gate): its result is
     added, times sigmoid(w . h) with w the vector `token_gate` (a name, or None: as it is); groups and keep: the experts are
     `groups` equal runs of neighbours, a group's score is the sum of its two largest s + correction, and only the experts
-    of the `keep` best groups can be chosen; route_scale multiplies the weights."""
+    of the `keep` best groups can be chosen; route_scale multiplies the weights; router_bias: a vector's name, added to W_router h
+    (score "softmax" with renorm: the weights are then the softmax over the chosen logits alone)."""
     graph_safe = True
     returns_rows = True
     libraries = ("grouped", "sequence")
 
     def __init__(self, width: int, inner: int, n_experts: int, top: int, router: str, correction, gate: str, up: str, down: str,
                  limit: float = 0.0, alpha: float = 1.0, score: str = "softmax", renorm: bool = True, weigh: str = "output",
-                 act: str = "clamped", shared=None, groups: int = 1, keep: int = 1, route_scale: float = 1.0):
+                 act: str = "clamped", shared=None, groups: int = 1, keep: int = 1, route_scale: float = 1.0, router_bias=None):
         """gate, up, down: tensor names with {e} for the expert's number; correction: a name or None."""
         if not 1 <= top <= n_experts:
             raise ValueError(f"routed_experts: {top} of {n_experts} experts")
@@ -170,10 +180,12 @@ class RoutedExperts(Part):
         self.token_gate = self.shared.get("token_gate") if self.shared else None
         # the router, and behind its rows the shared expert's gate: one product for both
         if self.token_gate:
+            if router_bias:
+                raise ValueError("routed_experts: a router's bias beside a shared expert's token gate is not built")
             self.router = Linear(width, n_experts + 1, router + "+gate", None, init_std=width ** -0.5,
                                  weight_sources=((router, n_experts), (self.token_gate, 1)))
         else:
-            self.router = Linear(width, n_experts, router, None)
+            self.router = Linear(width, n_experts, router, router_bias)
         if self.shared:
             sh = self.shared
             if self.gated:

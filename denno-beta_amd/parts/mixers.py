@@ -31,21 +31,44 @@ class CausalSelfAttention(Part):
     which add nothing to a score or a result).  unit_eps: behind the turn every head's q and k are divided by their root
     mean square, x / sqrt(mean(x^2) + unit_eps) over the head's entries (None: they stay).  head_gate: the name of a matrix
     [n_heads, width]: head a's result is multiplied by sigmoid(W_g h)_a before the output projection (its rows ride behind
-    the fused projection's; qkv_weight_sources then names the pieces of q, k and v).  Both go the 32-bit way of exact_turn."""
+    the fused projection's; qkv_weight_sources then names the pieces of q, k and v).  Both go the 32-bit way of exact_turn.
+    sink: the name of a number per head: a key without a value that every row sees with that score (nothing scales it).
+    keep_first: with a window, the first so many positions are read by every row as well; their pages stay.
+    qk_norm: dict(q, k, eps): before the turn every head's q and k are x / sqrt(mean(x^2) + eps) * w, w the named vector of
+    head_dim numbers that all heads share.  temp: the name of a number per head that multiplies its scores.  turn_values: the
+    value of a position is turned by it over all its pairs (by position * base^(-2m/value_dim), base the encoding's, whatever
+    scaling the keys' has) and kept so; a head's result is turned back by its own position.  entry_gate: the name of a matrix
+    [n_heads * value_dim, width]: the heads' results are multiplied entry by entry with sigmoid(W h).  Any of these four: one
+    kernel makes queries, keys and values from the projection's 32-bit result and puts keys and values into the cache
+    (ops.norm_turn_write), one turns the result back and gates it (ops.turn_back_gate)."""
     graph_safe = True
     returns_rows = True
 
     def __init__(self, width: int, n_heads: int, n_kv_heads: int, head_dim: int, scale: float,
                  qkv_weight: str, qkv_bias, out_weight: str, out_bias, stored_in_out: bool = False,
                  window: int = 0, out_init_std: float = 0.02, position=None, qkv_weight_sources=None,
-                 qkv_bias_sources=None, value_dim=None, exact_turn: bool = False, unit_eps=None, head_gate=None):
+                 qkv_bias_sources=None, value_dim=None, exact_turn: bool = False, unit_eps=None, head_gate=None, sink=None,
+                 keep_first: int = 0, qk_norm=None, temp=None, turn_values: bool = False, entry_gate=None):
         self.width, self.n_heads, self.n_kv_heads, self.head_dim = width, n_heads, n_kv_heads, head_dim
         self.value_dim = head_dim if value_dim is None else int(value_dim)
         self.unit_eps = None if unit_eps is None else float(unit_eps)
-        self.head_gate = head_gate
-        self.split = bool(exact_turn) or self.value_dim != head_dim or self.unit_eps is not None or head_gate is not None
-        if head_gate is not None and (qkv_bias is not None or not qkv_weight_sources or stored_in_out):
-            raise ValueError("causal_attention: a gate per head rides behind a projection without a bias that is stored [out, in] "
+        self.head_gate, self.entry_gate = head_gate, entry_gate
+        self.sink_name, self.temp_name, self.qk_norm, self.turn_values = sink, temp, (dict(qk_norm) if qk_norm else None), bool(turn_values)
+        self.keep_first = int(keep_first) if window > 0 else 0
+        self.prepared = qk_norm is not None or temp is not None or self.turn_values or entry_gate is not None
+        self.split = (bool(exact_turn) or self.value_dim != head_dim or self.unit_eps is not None or head_gate is not None
+                      or self.prepared)
+        if self.prepared:
+            self.libraries = ("sequence",)
+            if unit_eps is not None or head_gate is not None:
+                raise ValueError("causal_attention: unit_eps and head_gate do not go with qk_norm, temp, turn_values or entry_gate")
+            if self.turn_values and (self.value_dim % 2 != 0 or position is None or position[0] != "rotary_pairs"):
+                raise ValueError(f"causal_attention: values of {self.value_dim} numbers are turned in pairs, by the base of a rotary_pairs "
+                                 "encoding of the layer's own")
+        gate = head_gate if head_gate is not None else entry_gate
+        gate_rows = 0 if gate is None else n_heads if head_gate is not None else n_heads * self.value_dim
+        if gate is not None and (qkv_bias is not None or not qkv_weight_sources or stored_in_out):
+            raise ValueError("causal_attention: a gate rides behind a projection without a bias that is stored [out, in] "
                              "and whose pieces qkv_weight_sources names")
         # (the split way keeps keys and values in one width that every attention kernel takes)
         self.kept_dim = -(-max(head_dim, self.value_dim) // 16) * 16 if self.split else head_dim
@@ -60,10 +83,10 @@ class CausalSelfAttention(Part):
         self.kv_width = n_kv_heads * head_dim
         self.v_width = n_kv_heads * self.value_dim
         # (a checkpoint that stores q, k and v apart names them in qkv_*_sources: joined at load, one product here)
-        if head_gate is not None:
-            qkv_weight_sources = tuple(qkv_weight_sources) + ((head_gate, n_heads),)
+        if gate is not None:
+            qkv_weight_sources = tuple(qkv_weight_sources) + ((gate, gate_rows),)
         self.gate_col = self.q_width + self.kv_width + self.v_width
-        self.qkv = Linear(width, self.gate_col + (n_heads if head_gate is not None else 0), qkv_weight, qkv_bias, stored_in_out,
+        self.qkv = Linear(width, self.gate_col + gate_rows, qkv_weight, qkv_bias, stored_in_out,
                           weight_sources=qkv_weight_sources, bias_sources=qkv_bias_sources)
         self.out = Linear(n_heads * self.value_dim, width, out_weight, out_bias, stored_in_out, out_init_std)
         self.position = POSITIONS.make(position) if position is not None else None
@@ -72,10 +95,16 @@ class CausalSelfAttention(Part):
 
     def param_specs(self):
         own = self.position.param_specs() if self.position is not None else []
+        if self.qk_norm:
+            own += [ParamSpec(self.qk_norm[s], (self.head_dim,), "vector", ("normal", 1.0, 0.1)) for s in ("q", "k")]
+        if self.temp_name:
+            own.append(ParamSpec(self.temp_name, (self.n_heads,), "vector", ("normal", 1.0, 0.2)))
+        if self.sink_name:
+            own.append(ParamSpec(self.sink_name, (self.n_heads,), "vector", ("normal", 0.0, 1.0)))
         return self.qkv.param_specs() + self.out.param_specs() + own
 
     def cache_spec(self):
-        return PagedKV(self.n_kv_heads, self.kept_dim, self.window)
+        return PagedKV(self.n_kv_heads, self.kept_dim, self.window, keep_first=self.keep_first)
 
     def bind(self, tensors, runtime):
         super().bind(tensors, runtime)
@@ -84,6 +113,13 @@ class CausalSelfAttention(Part):
         if self.position is not None:
             self.position.bind(tensors, runtime)
         self.no_freq = torch.empty(0, dtype=torch.float32, device=runtime.device)
+        self.wq, self.wk = (tensors[self.qk_norm[s]] for s in ("q", "k")) if self.qk_norm else (None, None)
+        self.temp = tensors[self.temp_name] if self.temp_name else None
+        self.sink = tensors[self.sink_name] if self.sink_name else False
+        self.v_freq = None
+        if self.turn_values:
+            turn = POSITIONS.make(("rotary_pairs", dict(dims=self.value_dim, base=self.position.base)))
+            self.v_freq = turn.frequencies().to(torch.float32).to(runtime.device)
 
     def packed_input(self, n_rows):
         return self.qkv.packed_input(n_rows)
@@ -126,7 +162,7 @@ class CausalSelfAttention(Part):
             ops.kv_write(kv, 0, G * hw, g.slot_map, cache.k, cache.v)
         o = torch.empty((T, H * hw), dtype=act, device=dev)
         ops.attention(q, o, cache.k, cache.v, g.block_tables, g.tiles, H, self.scale, self.window, tiles_wide=g.tiles_wide,
-                      single_rows=g.single_rows, max_context=g.max_context)
+                      single_rows=g.single_rows, max_context=g.max_context, sink=self.sink, keep_first=self.keep_first)
         if self.head_gate is not None:      # (the gate per head, and the heads' first value_dim columns on, in one launch)
             o = ops.head_gate(o, z[:, self.gate_col:self.gate_col + H], H, dv, torch.empty((T, H * dv), dtype=act, device=dev),
                               head_stride=hw)
@@ -138,10 +174,34 @@ class CausalSelfAttention(Part):
             return self.out(o, out_dtype=torch.float32)
         self.out(o, residual=accumulate_into)
 
+    def _forward_prepared(self, h, ctx, cache, g, position, accumulate_into):
+        """The projection's result in 32-bit; one kernel norms and turns what it holds and puts keys and values into the cache;
+        behind the attention one kernel turns the heads' results back and gates them."""
+        act, T, dev = self.runtime.act_dtype, h.shape[0], h.device
+        H, G, dv, hw = self.n_heads, self.n_kv_heads, self.value_dim, self.kept_dim
+        turns = position is not None and getattr(position, "rotates", False)
+        if turns and (not hasattr(position, "freq") or position.mag != 1.0):
+            raise TypeError(f"{type(position).__name__}: this turn needs a table of frequencies and no factor on cos and sin (rotary_pairs)")
+        z = self.qkv(h, out_dtype=torch.float32)
+        q = ops.norm_turn_write(z, H, G, self.head_dim, dv, ctx.positions, torch.empty((T, H * hw), dtype=act, device=dev), g.slot_map,
+                                cache.k, cache.v, wq=self.wq, wk=self.wk, eps=self.qk_norm["eps"] if self.qk_norm else None,
+                                q_scale=self.temp, freq=position.freq if turns else None, v_freq=self.v_freq, write=cache.writes)
+        o = torch.empty((T, H * hw), dtype=act, device=dev)
+        ops.attention(q, o, cache.k, cache.v, g.block_tables, g.tiles, H, self.scale, self.window, tiles_wide=g.tiles_wide,
+                      single_rows=g.single_rows, max_context=g.max_context, sink=self.sink, keep_first=self.keep_first)
+        if hw != dv or self.v_freq is not None or self.entry_gate is not None:
+            o = ops.turn_back_gate(o, H, dv, torch.empty((T, H * dv), dtype=act, device=dev), positions=ctx.positions, freq=self.v_freq,
+                                   gate=z[:, self.gate_col:self.gate_col + H * dv] if self.entry_gate is not None else None, head_stride=hw)
+        if accumulate_into is None:
+            return self.out(o, out_dtype=torch.float32)
+        self.out(o, residual=accumulate_into)
+
     def forward(self, h, ctx, cache, accumulate_into, stats=None, deferred=None):
         act = self.runtime.act_dtype
         g = ctx.groups[cache.group]
         position = self.position if self.position is not None else self.runtime.position
+        if self.prepared:
+            return self._forward_prepared(h, ctx, cache, g, position, accumulate_into)
         if self.split:
             return self._forward_split(h, ctx, cache, g, position, accumulate_into)
         if position is not None and getattr(position, "rotates", False):
@@ -164,7 +224,7 @@ class CausalSelfAttention(Part):
             o = torch.empty((h.shape[0], self.q_width), dtype=act, device=h.device)
         ops.attention(q, o, cache.k, cache.v, g.block_tables, g.tiles, self.n_heads,
                       self.scale, self.window, tiles_wide=g.tiles_wide, single_rows=g.single_rows,
-                      max_context=g.max_context)
+                      max_context=g.max_context, sink=self.sink, keep_first=self.keep_first)
         if accumulate_into is None:
             return self.out(o, out_dtype=torch.float32)
         self.out(o, residual=accumulate_into, stats=stats, deferred=deferred)
@@ -182,13 +242,19 @@ class LatentAttention(Part):
     Only c and the turned key part are kept, as one key of kv_rank + rot_dim numbers per token that every head reads:
     q_plain . (W_uk c) = (W_uk^T q_plain) . c, so the query is carried to the latent's space once per token, the
     attention kernels run with one key head of that width (the same rows serve as values), and W_uv is applied to
-    the weighted sum of latents.  position: the arguments of a "rotary_pairs" encoding for the turned parts."""
+    the weighted sum of latents.  position: the arguments of a "rotary_pairs" encoding for the turned parts (rot_dim 0: there
+    are none, and it is not read).
+
+    q_rank > 0: the queries come through a small normed vector of their own, q = W_uq norm(W_dq h) (names dq, dq_norm, uq in q's
+    place).  A name "sink": a number per head, the score of a key without a value that every row sees."""
     graph_safe = True
+    returns_rows = True
     libraries = ("sequence", "grouped")
 
     def __init__(self, width: int, n_heads: int, head_dim: int, rot_dim: int, value_dim: int, kv_rank: int, scale: float,
-                 eps: float, position: dict, names: dict, keep: str = None, window: int = 0):
-        """names: q, dkv, g, uk, uv, o (matrices; without "g" the heads' results go on ungated); dkv_norm (vector).
+                 eps: float, position: dict, names: dict, keep: str = None, window: int = 0, q_rank: int = 0):
+        """names: q (or dq, uq), dkv, g, uk, uv, o (matrices; without "g" the heads' results go on ungated); dkv_norm (and dq_norm,
+        sink) (vectors).
         window > 0: a query at position p reads the keys p - window + 1 .. p only.
         keep: "latent" (the form above), "heads" (every head's own key [W_uk c | turned part] and value W_uv c are kept,
         as an ordinary attention does: more cache, and the way out where kv_rank + rot_dim is beyond the attention kernels'
@@ -207,19 +273,24 @@ class LatentAttention(Part):
         self.o_width = n_heads * value_dim
         self.window = int(window)
         self.gated = "g" in names
-        # one product for everything that reads h: q | dkv | g
-        if self.gated:
-            self.proj = Linear(width, self.q_width + self.key_dim + self.o_width, names["q"] + "+dkv+g", None,
-                               weight_sources=((names["q"], self.q_width), (names["dkv"], self.key_dim), (names["g"], self.o_width)))
-        else:
-            self.proj = Linear(width, self.q_width + self.key_dim, names["q"] + "+dkv", None,
-                               weight_sources=((names["q"], self.q_width), (names["dkv"], self.key_dim)))
+        self.q_rank = int(q_rank)
+        # one product for everything that reads h: q (or its small vector) | dkv | g
+        first = (names["dq"], self.q_rank) if self.q_rank else (names["q"], self.q_width)
+        self.low = first[1]                    # where dkv's columns begin
+        pieces = (first, (names["dkv"], self.key_dim)) + (((names["g"], self.o_width),) if self.gated else ())
+        self.proj = Linear(width, sum(n for _, n in pieces), first[0] + "+dkv" + ("+g" if self.gated else ""), None, weight_sources=pieces)
+        self.up_q = Linear(self.q_rank, self.q_width, names["uq"], None, init_std=self.q_rank ** -0.5) if self.q_rank else None
         self.out = Linear(self.o_width, width, names["o"], None)
-        self.position = POSITIONS.make(("rotary_pairs", dict(position, head_dim=rot_dim)))
+        self.position = POSITIONS.make(("rotary_pairs", dict(position, head_dim=rot_dim))) if rot_dim else None
 
     def param_specs(self):
         H, r = self.n_heads, self.kv_rank
-        return self.proj.param_specs() + self.out.param_specs() + [
+        own = []
+        if self.q_rank:
+            own += self.up_q.param_specs() + [ParamSpec(self.names["dq_norm"], (self.q_rank,), "vector", ("normal", 1.0, 0.1))]
+        if "sink" in self.names:
+            own.append(ParamSpec(self.names["sink"], (H,), "vector", ("normal", 0.0, 1.0)))
+        return own + self.proj.param_specs() + self.out.param_specs() + [
             ParamSpec(self.names["uk"], (H * self.head_dim, r), "matrix", ("normal", 0.0, r ** -0.5)),
             ParamSpec(self.names["uv"], (H * self.value_dim, r), "matrix", ("normal", 0.0, r ** -0.5)),
             ParamSpec(self.names["dkv_norm"], (r,), "vector", ("normal", 1.0, 0.1))]
@@ -231,7 +302,12 @@ class LatentAttention(Part):
     def bind(self, tensors, runtime):
         super().bind(tensors, runtime)
         self.proj.bind(tensors), self.out.bind(tensors)
-        self.position.bind(tensors, runtime)
+        if self.position is not None:
+            self.position.bind(tensors, runtime)
+        if self.q_rank:
+            self.up_q.bind(tensors)
+            self.q_norm = tensors[self.names["dq_norm"]]
+        self.sink = tensors[self.names["sink"]] if "sink" in self.names else False
         self.no_freq = torch.empty(0, dtype=torch.float32, device=runtime.device)
         H, r = self.n_heads, self.kv_rank
         # W_uk per head, transposed once: [heads, kv_rank, dim], so that both per-head products are out = W[h] a
@@ -245,22 +321,31 @@ class LatentAttention(Part):
         dn, dr, r, kd = self.head_dim, self.rot_dim, self.kv_rank, self.key_dim
         g = ctx.groups[cache.group]
         z = self.proj(h, out_dtype=torch.float32)
-        low, gate = self.q_width, self.q_width + kd
+        low, gate = self.low, self.low + kd
         if self.keep == "heads":
             return self._forward_heads(z, ctx, cache, g, accumulate_into)
-        # the token's key: [c | turned part]
-        key = torch.empty((T, kd), dtype=act, device=h.device)
-        ops.rmsnorm(z[:, low:low + r], self.c_norm, self.eps, key[:, :r])
-        self.position.turn(z, key, ctx.positions, 1, dr, src_off=low + r, dst_off=r)
-        if cache.writes:
-            ops.kv_write(key, 0, 0, g.slot_map, cache.k, cache.v)
+        if self.q_rank and dr == 0:
+            # one kernel: both small vectors normed, the latent to its place in the cache as key and value
+            cq = ops.norm_pair_write(z[:, :gate], low, self.q_norm, self.c_norm, self.eps, torch.empty((T, low), dtype=act, device=h.device),
+                                     g.slot_map, cache.k, cache.v, write=cache.writes, value_normed=True)
+            plain = self.up_q(cq, out_dtype=act)
+        else:
+            # the token's key: [c | turned part]
+            key = torch.empty((T, kd), dtype=act, device=h.device)
+            ops.rmsnorm(z[:, low:low + r], self.c_norm, self.eps, key[:, :r])
+            if dr:
+                self.position.turn(z, key, ctx.positions, 1, dr, src_off=low + r, dst_off=r)
+            if cache.writes:
+                ops.kv_write(key, 0, 0, g.slot_map, cache.k, cache.v)
+            plain = self._queries(z)
         # the queries in the latent's space: [W_uk^T q_plain | turned part] per head
         q = torch.empty((T, H * kd), dtype=act, device=h.device)
-        ops.heads_linear(z, self.uk_t, q, a_off=0, a_stride=dn + dr, o_off=0, o_stride=kd)
-        self.position.turn(z, q, ctx.positions, H, dr, src_off=dn, src_stride=dn + dr, dst_off=r, dst_stride=kd)
+        ops.heads_linear(plain, self.uk_t, q, a_off=0, a_stride=dn + dr, o_off=0, o_stride=kd)
+        if dr:
+            self.position.turn(plain, q, ctx.positions, H, dr, src_off=dn, src_stride=dn + dr, dst_off=r, dst_stride=kd)
         o_lat = torch.empty((T, H * kd), dtype=act, device=h.device)
         ops.attention(q, o_lat, cache.k, cache.v, g.block_tables, g.tiles, H, self.scale, self.window, tiles_wide=g.tiles_wide,
-                      single_rows=g.single_rows, max_context=g.max_context)
+                      single_rows=g.single_rows, max_context=g.max_context, sink=self.sink)
         if self.gated:
             o = torch.empty((T, self.o_width), dtype=torch.float32, device=h.device)
             ops.heads_linear(o_lat, self.uv, o, a_off=0, a_stride=kd)
@@ -273,27 +358,39 @@ class LatentAttention(Part):
             return self.out(og, out_dtype=torch.float32)
         self.out(og, residual=accumulate_into)
 
+    def _queries(self, z):
+        """Rows whose first columns are the heads' queries, 32-bit where something is still turned: the projection's own, or made
+        from its small vector."""
+        if not self.q_rank:
+            return z
+        act = self.runtime.act_dtype
+        cq = ops.rmsnorm(z[:, :self.q_rank], self.q_norm, self.eps, torch.empty((z.shape[0], self.q_rank), dtype=act, device=z.device))
+        return self.up_q(cq, out_dtype=torch.float32 if self.rot_dim else act)
+
     def _forward_heads(self, z, ctx, cache, g, accumulate_into):
         """Every head's key [W_uk c | turned part | zeros] and value [W_uv c | zeros], `head_width` wide, go to the cache;
         the queries are [q_plain | turned part | zeros]: the zeros add nothing to a score or a result."""
         act, T, H, dev = self.runtime.act_dtype, z.shape[0], self.n_heads, z.device
         dn, dr, r, dv, hw = self.head_dim, self.rot_dim, self.kv_rank, self.value_dim, self.head_width
-        low, gate = self.q_width, self.q_width + self.key_dim
+        low, gate = self.low, self.low + self.key_dim
+        plain = self._queries(z)
         copy = lambda src, dst, width, **layout: ops.rotary(src, dst, ctx.positions, self.no_freq, H, 0, width, **layout)   # noqa: E731
         c = torch.empty((T, r), dtype=act, device=dev)
         ops.rmsnorm(z[:, low:low + r], self.c_norm, self.eps, c)
         kv = torch.zeros((T, 2 * H * hw), dtype=act, device=dev)      # keys at column 0, values at H * hw
         ops.heads_linear(c, self.uk, kv, a_off=0, a_stride=0, o_off=0, o_stride=hw)
-        self.position.turn(z, kv, ctx.positions, H, dr, src_off=low + r, src_stride=0, dst_off=dn, dst_stride=hw)
+        if dr:
+            self.position.turn(z, kv, ctx.positions, H, dr, src_off=low + r, src_stride=0, dst_off=dn, dst_stride=hw)
         ops.heads_linear(c, self.uv, kv, a_off=0, a_stride=0, o_off=H * hw, o_stride=hw)
         if cache.writes:
             ops.kv_write(kv, 0, H * hw, g.slot_map, cache.k, cache.v)
         q = torch.zeros((T, H * hw), dtype=act, device=dev)
-        copy(z, q, dn, src_off=0, src_stride=dn + dr, dst_off=0, dst_stride=hw)
-        self.position.turn(z, q, ctx.positions, H, dr, src_off=dn, src_stride=dn + dr, dst_off=dn, dst_stride=hw)
+        copy(plain, q, dn, src_off=0, src_stride=dn + dr, dst_off=0, dst_stride=hw)
+        if dr:
+            self.position.turn(plain, q, ctx.positions, H, dr, src_off=dn, src_stride=dn + dr, dst_off=dn, dst_stride=hw)
         o = torch.empty((T, H * hw), dtype=act, device=dev)
         ops.attention(q, o, cache.k, cache.v, g.block_tables, g.tiles, H, self.scale, self.window, tiles_wide=g.tiles_wide,
-                      single_rows=g.single_rows, max_context=g.max_context)
+                      single_rows=g.single_rows, max_context=g.max_context, sink=self.sink)
         if hw != dv:
             packed = torch.empty((T, self.o_width), dtype=act, device=dev)
             copy(o, packed, dv, src_off=0, src_stride=hw, dst_off=0, dst_stride=dv)

@@ -81,7 +81,12 @@ class RotaryPairs(Part):
     d(t) = dims * ln(original / (2 pi t)) / (2 ln base), the pair index whose pair makes t turns over `original` positions,
     lo = max(floor(d(fast)), 0), hi = min(ceil(d(slow)), dims - 1) and ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1),
     pair i turns by p * (f_i / factor * ramp_i + f_i * (1 - ramp_i)): fast pairs stay, slow ones are slowed down by `factor`;
-    and cos and sin are multiplied by `mag` = 0.1 ln(factor) + 1."""
+    and cos and sin are multiplied by `mag` = 0.1 ln(factor) + 1.
+
+    scaling = dict(factor, original, low, high) is another way to the same end: a pair is judged by n_i = original f_i / (2 pi), the
+    turns it makes over `original` positions.  With ramp_i = clamp((n_i - low) / (high - low), 0, 1) pair i turns by
+    p * (ramp_i f_i + (1 - ramp_i) f_i / factor): pairs of more than `high` turns stay, those of fewer than `low` are slowed down
+    by `factor`; cos and sin stay as they are."""
     graph_safe = True
     rotates = True
     libraries = ("sequence",)
@@ -94,10 +99,15 @@ class RotaryPairs(Part):
             raise ValueError(f"rotary_pairs: {dims} dimensions in vectors of {self.head_dim}")
         self.scaling = dict(scaling) if scaling else None
         self.mag = 1.0
+        self.by_turns = bool(self.scaling) and "low" in self.scaling
         if self.scaling:
-            missing = [k for k in ("factor", "original", "fast", "slow") if k not in self.scaling]
+            missing = [k for k in ("factor", "original") + (("low", "high") if self.by_turns else ("fast", "slow")) if k not in self.scaling]
             if missing or not self.scaling["factor"] > 0 or not self.scaling["original"] > 0 or self.base <= 1:
-                raise ValueError(f"rotary_pairs: scaling needs factor, original, fast and slow (and a base above 1); got {self.scaling}")
+                raise ValueError("rotary_pairs: scaling needs factor, original and either fast and slow or low and high (and a base "
+                                 f"above 1); got {self.scaling}")
+            if self.by_turns and not self.scaling["high"] >= self.scaling["low"]:
+                raise ValueError(f"rotary_pairs: scaling's high is below its low: {self.scaling}")
+        if self.scaling and not self.by_turns:
             self.mag = 0.1 * math.log(float(self.scaling["factor"])) + 1.0
 
     def frequencies(self):
@@ -108,6 +118,10 @@ class RotaryPairs(Part):
             return f
         sc = self.scaling
         factor, original = float(sc["factor"]), float(sc["original"])
+        if self.by_turns:
+            turns, low, high = original * f / (2.0 * math.pi), float(sc["low"]), float(sc["high"])
+            ramp = torch.clamp((turns - low) / (high - low), 0.0, 1.0) if high > low else (turns >= low).to(torch.float64)
+            return ramp * f + (1.0 - ramp) * f / factor
 
         def pair_of(turns):
             return self.dims * math.log(original / (2.0 * math.pi * float(turns))) / (2.0 * math.log(self.base))

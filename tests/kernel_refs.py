@@ -133,7 +133,7 @@ def linear_norm_in(copy, stats, c1, c2, eps, w, out, epilogue="none", kv=None, n
 
 
 def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, window=0, tiles_wide=None,
-              single_rows=False, max_context=0, decode_waves=None, chunk=0, bias=None, sink=False):
+              single_rows=False, max_context=0, decode_waves=None, chunk=0, bias=None, sink=False, keep_first=0):
     n_pages, hkv, ps, dh = k_pool.shape
     group = n_heads // hkv
     tl = tiles.cpu().tolist()
@@ -147,7 +147,7 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
             lo = max(0, pos - window + 1) if window > 0 else 0
             if chunk > 0:
                 lo = max(lo, pos // chunk * chunk)
-            keys = torch.arange(lo, pos + 1)
+            keys = torch.tensor([j for j in range(pos + 1) if j >= lo or (window > 0 and j < keep_first)])
             pages = bt[seq][keys // ps].long()
             offs = keys % ps
             assert (pages >= 0).all(), "attention reads a page that was given back"
@@ -158,8 +158,9 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
                 sc = (k @ qv) * scale
                 if bias is not None:
                     sc = sc + bias[h][torch.clamp(pos - keys, max=bias.shape[1] - 1)]
-                if sink:      # (a key with score 0 and no value)
-                    p = torch.softmax(torch.cat([sc, sc.new_zeros(1)]), dim=0)[:-1]
+                if sink is not False:      # (a key without a value: score 0, or the head's own)
+                    at = sink[h:h + 1].to(sc) if isinstance(sink, torch.Tensor) else sc.new_zeros(1)
+                    p = torch.softmax(torch.cat([sc, at]), dim=0)[:-1]
                 else:
                     p = torch.softmax(sc, dim=0)
                 out[row0 + i, h * dh:(h + 1) * dh] = (p @ v).to(out.dtype)
@@ -536,7 +537,7 @@ def streams_write(xs, y, mix, w_out, next_in=None, weight=None, eps=0.0, out=Non
     return out
 
 
-def norm_pair_write(z, q_width, wq, wk, eps, q_out, slot_map, k_pool, v_pool, write=True):
+def norm_pair_write(z, q_width, wq, wk, eps, q_out, slot_map, k_pool, v_pool, write=True, value_normed=False):
     n_pages, hkv, ps, dh = k_pool.shape
     unit = lambda v: v.double() / torch.sqrt((v.double() ** 2).mean(dim=-1, keepdim=True) + eps)      # noqa: E731
     q_out.copy_(unit(z[:, :q_width]) * wq.double())
@@ -545,8 +546,60 @@ def norm_pair_write(z, q_width, wq, wk, eps, q_out, slot_map, k_pool, v_pool, wr
         for t, slot in enumerate(slot_map.tolist()):
             if slot >= 0:
                 k_pool[slot // ps, :, slot % ps, :] = keys[t].view(hkv, dh)
-                v_pool[slot // ps, :, :, slot % ps] = z[t, q_width:].view(hkv, dh).to(v_pool.dtype)
+                v_pool[slot // ps, :, :, slot % ps] = keys[t].view(hkv, dh) if value_normed else z[t, q_width:].view(hkv, dh).to(v_pool.dtype)
     return q_out
+
+
+def _turned(x, positions, freq, sign=1.0):
+    """x [T, n, d]: its first 2 len(freq) entries in pairs (2i, 2i + 1), turned by sign * position * freq[i]."""
+    out = x.clone()
+    if freq is not None and freq.numel():
+        k = 2 * freq.numel()
+        ang = sign * (positions.to(torch.float32)[:, None] * freq.to(torch.float32)[None, :]).to(x.dtype)[:, None, :]
+        a, b = x[..., 0:k:2], x[..., 1:k:2]
+        out[..., 0:k:2] = a * torch.cos(ang) - b * torch.sin(ang)
+        out[..., 1:k:2] = b * torch.cos(ang) + a * torch.sin(ang)
+    return out
+
+
+def norm_turn_write(z, n_heads, n_kv, dk, dv, positions, q_out, slot_map, k_pool, v_pool, wq=None, wk=None, eps=None, q_scale=None,
+                    freq=None, v_freq=None, write=True):
+    T, kept, ps = z.shape[0], k_pool.shape[3], k_pool.shape[2]
+    zd = z.double()
+    q = zd[:, :n_heads * dk].reshape(T, n_heads, dk)
+    k = zd[:, n_heads * dk:(n_heads + n_kv) * dk].reshape(T, n_kv, dk)
+    v = zd[:, (n_heads + n_kv) * dk:(n_heads + n_kv) * dk + n_kv * dv].reshape(T, n_kv, dv)
+    if eps is not None:
+        q, k = (x / torch.sqrt((x * x).mean(dim=-1, keepdim=True) + eps) for x in (q, k))
+    q, k = (x if w is None else x * w.double() for x, w in ((q, wq), (k, wk)))
+    q, k, v = _turned(q, positions, freq), _turned(k, positions, freq), _turned(v, positions, v_freq)
+    if q_scale is not None:
+        q = q * q_scale.double()[:, None]
+    pad = lambda x: torch.nn.functional.pad(x, (0, kept - x.shape[-1]))      # noqa: E731
+    q_out.copy_(pad(q).reshape(T, n_heads * kept))
+    if write:
+        for t, slot in enumerate(slot_map.tolist()):
+            if slot >= 0:
+                k_pool[slot // ps, :, slot % ps, :] = pad(k[t]).to(k_pool.dtype)
+                v_pool[slot // ps, :, :, slot % ps] = pad(v[t]).to(v_pool.dtype)
+    return q_out
+
+
+def turn_back_gate(o, n_heads, dv, out, positions=None, freq=None, gate=None, head_stride=None):
+    hs = dv if head_stride is None else head_stride
+    T = o.shape[0]
+    x = torch.stack([o[:, h * hs:h * hs + dv].double() for h in range(n_heads)], dim=1)
+    x = _turned(x, positions, freq, -1.0).reshape(T, n_heads * dv)
+    out.copy_(x if gate is None else x * torch.sigmoid(gate.double()))
+    return out
+
+
+def poly_norm(z, numbers, eps, out):
+    a, b, c, e = numbers.double().tolist()
+    N = lambda v: v / torch.sqrt((v * v).mean(dim=-1, keepdim=True) + eps)      # noqa: E731
+    z = z.double()
+    out.copy_(a * N(z) + b * N(z ** 2) + c * N(z ** 3) + e)
+    return out
 
 
 def pair_rows(tokens, positions, row_start, slots, last, mul_prev, mul_cur, buckets, out, write=True):
