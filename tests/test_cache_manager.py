@@ -151,11 +151,31 @@ def test_groups_have_pools_of_their_own():
     assert m.pages_peak(0, 100, 32) == 7 and m.pages_peak(1, 100, 32) == 4 and m.pages_peak(2, 100, 32) == 0
 
 
+def test_a_window_that_keeps_the_first_pages():
+    m = CacheManager([GroupLayout(PAGED, 12, 8, 20, 11), GroupLayout(PAGED, 12, 8, 20)], 2)      # 11 first keys: two pages of 8
+    m.add(1)
+    for n in (5, 12, 19, 20, 21, 28, 29, 36, 40, 61, 77):
+        m.reserve(1, n)
+        m.commit(1, n)
+        first = max(0, n - 20 + 1) // 8      # the first block that the next row's window reaches
+        held = [p >= 0 for p in m.block_table(1, 0).tolist()]
+        assert held == [b < 2 or b >= first for b in range(-(-n // 8))], n
+        assert [p >= 0 for p in m.block_table(1, 1).tolist()] == [b >= first for b in range(-(-n // 8))], n
+        m.check()
+    assert m.pages_held(1, 0) == m.pages_held(1, 1) + 2
+    assert m.pages_peak(0, 400, 16) == m.pages_peak(1, 400, 16) + 2 and m.pages_peak(0, 24, 16) == 3
+    assert m.release(1)
+    m.check()
+    assert m.free_pages(0) == 12 and m.free_pages(1) == 12
+    with pytest.raises(ValueError):
+        CacheManager([GroupLayout(PAGED, 4, 8, 20, -1)], 1)
+
+
 @pytest.mark.parametrize("seed", range(6))
 def test_random_orders_keep_every_page_accounted(seed):
     rng = random.Random(seed)
     window = [0, 0, 24, 5, 0, 40][seed]
-    m = CacheManager([GroupLayout(PAGED, 24, 8, 0), GroupLayout(PAGED, 12, 8, window)], 5)
+    m = CacheManager([GroupLayout(PAGED, 24, 8, 0), GroupLayout(PAGED, 12, 8, window, [0, 3, 0, 9, 0, 16][seed])], 5)
     live, next_rid = {}, 0
     for _ in range(600):
         op = rng.random()

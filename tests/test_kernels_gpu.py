@@ -1097,3 +1097,52 @@ def test_attention_in_chunks_with_a_bias_by_distance_and_a_sink(dtype, H, Hkv, d
         rows = torch.zeros(T, H * dh, dtype=dtype, device=DEV)
         ops().attention(qs, rows, k, v, bt, tiles, H, scale, 0, **kw)
         assert torch.equal(rows, out)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("H,Hkv,dh,ps,window,keep", [(4, 2, 16, 16, 24, 5), (8, 8, 96, 16, 200, 64), (3, 1, 24, 8, 13, 16), (2, 2, 64, 16, 1, 1),
+                                                     (2, 1, 128, 32, 64, 33), (5, 5, 80, 16, 300, 17), (2, 2, 64, 16, 40, 0), (6, 1, 112, 16, 72, 65),
+                                                     (4, 4, 64, 16, 100, 128), (2, 2, 256, 16, 100, 700), (1, 1, 48, 64, 31, 32)])
+def test_attention_in_a_window_that_keeps_first_keys_with_a_sink_per_head(dtype, H, Hkv, dh, ps, window, keep):
+    """Every kernel that `attention` may take, with the pages that no row of a request reads given back: prompts, portions that start
+    deep in a context, before and behind the window's and the kept keys' edges, decoded tokens."""
+    sink = torch.randn(H, generator=torch.Generator().manual_seed(keep)).to(DEV) * 2
+    scale = 1 / math.sqrt(dh)
+
+    def case(seq_lens, new_rows, seed):
+        q, k, v, bt, tiles, T = paged_case(seq_lens, new_rows, H, Hkv, dh, ps, dtype, seed=seed)
+        bt = bt.clone()
+        for s, (total, new) in enumerate(zip(seq_lens, new_rows)):
+            for b in range(-(-keep // ps), max(0, total - new - window + 1) // ps):
+                bt[s, b] = -1
+        return q[:, :H * dh], k, v, bt, tiles, T
+    seq_lens, new_rows = [300, 70, 133, 1, 430, 900], [1, 70, 21, 1, 300, 40]
+    q, k, v, bt, tiles, T = case(seq_lens, new_rows, H + dh + window)
+    for kw in (dict(sink=sink, keep_first=keep), dict(keep_first=keep), dict(sink=sink)):
+        if "keep_first" not in kw:
+            for s, (total, new) in enumerate(zip(seq_lens, new_rows)):      # (what is not kept may be gone)
+                bt[s, :max(0, total - new - window + 1) // ps] = -1
+        want = R.attention(q, torch.zeros(T, H * dh, device=DEV), k, v, bt, tiles, H, scale, window, **kw)
+        for wide in (None, paged_case.wide):
+            out = torch.zeros(T, H * dh, dtype=dtype, device=DEV)
+            ops().attention(q, out, k, v, bt, tiles, H, scale, window, tiles_wide=wide, **kw)
+            assert torch.allclose(out.float(), want, **TOL[dtype]), ("portions", wide is not None, kw.keys())
+    # a step of single rows: contexts on both sides of the window's edge, the kept keys', a page's and a split's
+    seq_lens = [1, window, window + 1, max(keep, 1), keep + 1, keep + window, keep + window + 1, 256, 257, 1024]
+    q, k, v, bt, tiles, T = case(seq_lens, [1] * len(seq_lens), dh)
+    kw = dict(sink=sink, keep_first=keep)
+    want = R.attention(q, torch.zeros(T, H * dh, device=DEV), k, v, bt, tiles, H, scale, window, **kw)
+    out = torch.zeros(T, H * dh, dtype=dtype, device=DEV)
+    ops().attention(q, out, k, v, bt, tiles, H, scale, window, tiles_wide=paged_case.wide, single_rows=True, max_context=1024, **kw)
+    assert torch.allclose(out.float(), want, **TOL[dtype]), "single rows"
+    if dtype == torch.bfloat16 and dh % 16 == 0 and ps % 16 == 0:
+        for waves in (4, 8, 16):
+            if waves <= (16 if dh <= 64 else 8 if dh <= 128 else 4):
+                out = torch.zeros(T, H * dh, dtype=dtype, device=DEV)
+                ops().attention(q, out, k, v, bt, tiles, H, scale, window, tiles_wide=paged_case.wide, single_rows=True, max_context=1024,
+                                decode_waves=waves, **kw)
+                assert torch.allclose(out.float(), want, **TOL[dtype]), waves
+    if dtype == torch.float32 and dh % 16 == 0:      # the kernels for single rows and for portions: the same bits
+        rows = torch.zeros(T, H * dh, dtype=dtype, device=DEV)
+        ops().attention(q, rows, k, v, bt, tiles, H, scale, window, **kw)
+        assert torch.equal(rows, out)

@@ -753,3 +753,68 @@ def test_a_product_that_ends_in_a_squared_relu(dtype, M, N, K):
     close(ops.linear(a, w, None, torch.zeros(M, N, dtype=dtype, device=DEV), epilogue="relu2"), want, dtype, "rows")
     if dtype == torch.bfloat16:
         close(ops.linear(a, ops.pack_matrix(w), None, torch.zeros(M, N, dtype=dtype, device=DEV), epilogue="relu2"), want, dtype, "packed")
+
+
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("T", [9, 300])
+@pytest.mark.parametrize("H,G,dk,dv,dims,ps", [(4, 2, 16, 8, 8, 16), (3, 1, 24, 40, 24, 8), (2, 2, 10, 6, 4, 16), (5, 5, 256, 32, 64, 16),
+                                               (1, 1, 3, 2, 2, 4), (6, 3, 64, 128, 0, 32), (16, 4, 128, 256, 128, 16)])
+def test_queries_keys_and_values_normed_turned_and_kept_in_one_launch(dtype, T, H, G, dk, dv, dims, ps):
+    kept = -(-max(dk, dv) // 16) * 16
+    z = torch.randn(T, (H + G) * dk + G * dv + 5, device=DEV) * 2
+    pos = torch.randint(0, 5000, (T,), dtype=torch.int32, device=DEV)
+    n_pages = T // ps + 3
+    slot_map = torch.randperm(n_pages * ps, device=DEV)[:T].int()
+    slot_map[T // 2] = -1
+    angles = lambda n: (10000.0 ** (-torch.arange(n, dtype=torch.float64) / max(n, 1))).float().to(DEV)      # noqa: E731
+    wq, wk, temp = torch.randn(dk, device=DEV), torch.randn(dk, device=DEV), torch.randn(H, device=DEV)
+    for kw in (dict(wq=wq, wk=wk, eps=1e-5, q_scale=temp, freq=angles(dims // 2), v_freq=angles(dv // 2)), dict(eps=1e-3, wk=wk),
+               dict(q_scale=temp, v_freq=angles(dv // 2)), dict(wq=wq, eps=1e-5, freq=angles(dims // 2), write=False)):
+        q = torch.full((T, H * kept), 7.0, dtype=dtype, device=DEV)
+        k, v = (torch.full(s, 5.0, dtype=dtype, device=DEV) for s in ((n_pages, G, ps, kept), (n_pages, G, kept, ps)))
+        hq, hk, hv = q.cpu().clone(), k.cpu().clone(), v.cpu().clone()
+        ops.norm_turn_write(z, H, G, dk, dv, pos, q, slot_map, k, v, **kw)
+        ref.norm_turn_write(z.cpu(), H, G, dk, dv, pos.cpu(), hq, slot_map.cpu(), hk, hv,
+                            **{n: a.cpu() if isinstance(a, torch.Tensor) else a for n, a in kw.items()})
+        close(q, hq, dtype, "queries"), close(k, hk, dtype, "keys"), close(v, hv, dtype, "values")
+    with pytest.raises(Exception):
+        ops.norm_turn_write(z, H, G, dk, dv, pos, q, slot_map, k, v, freq=angles(dk // 2 + 1))
+
+
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("T,H,dv,hs", [(9, 4, 8, 16), (300, 3, 40, 48), (7, 5, 256, 256), (2, 1, 2, 16), (270, 16, 128, 128)])
+def test_results_turned_back_and_gated(dtype, T, H, dv, hs):
+    o = torch.randn(T, H * hs, device=DEV).to(dtype)
+    gate = torch.randn(T, H * dv + 6, device=DEV)[:, 3:3 + H * dv] * 2
+    pos = torch.randint(0, 5000, (T,), dtype=torch.int32, device=DEV)
+    freq = (10000.0 ** (-torch.arange(dv // 2, dtype=torch.float64) * 2 / dv)).float().to(DEV)
+    out = lambda: torch.zeros(T, H * dv, dtype=dtype, device=DEV)      # noqa: E731
+    for f, g in ((freq, gate), (freq, None), (None, gate), (None, None)):
+        both("turn_back_gate", lambda: (o, H, dv, out(), pos, f, g, hs), [3], dtype)
+    # an odd width, gated only
+    both("turn_back_gate", lambda: (o, H, dv - 1, out()[:, :H * (dv - 1)], None, None, gate[:, :H * (dv - 1)], hs), [3], dtype)
+    # what a value was turned by and a result is turned back by cancel at one position
+    if hs == dv:
+        v = torch.randn(T, H * dv, device=DEV)
+        turned = ops.rotary(v, torch.empty_like(v), pos, freq, H, dv, dv)
+        close(ops.turn_back_gate(turned, H, dv, torch.empty_like(v), pos, freq), v, torch.float32)
+
+
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("n", [1, 37, 256, 1024, 1025, 4096, 5000])
+def test_a_polynomial_of_normed_powers(dtype, n):
+    z = torch.randn(11, n + 3, device=DEV)[:, :n] * torch.logspace(-2, 2, 11, device=DEV)[:, None]
+    numbers = torch.tensor([0.7, -0.4, 1.3, 0.2], device=DEV)
+    both("poly_norm", lambda: (z, numbers, 1e-5, torch.zeros(11, n + 1, dtype=dtype, device=DEV)[:, :n]), [3], dtype)
+    both("poly_norm", lambda: (z, torch.tensor([0.0, 0.0, 1.0, 0.0], device=DEV), 1e-2, torch.zeros(11, n, dtype=dtype, device=DEV)), [3], dtype)
+
+
+@pytest.mark.parametrize("dtype", DT)
+def test_a_normed_latent_kept_as_key_and_value(dtype):
+    T, qw, dh, ps = 21, 30, 44, 8
+    z = torch.randn(T, qw + dh + 3, device=DEV)[:, :qw + dh]
+    wq, wk = torch.randn(qw, device=DEV), torch.randn(dh, device=DEV)
+    slot_map = torch.randperm(5 * ps, device=DEV)[:T].int()
+    k, v = torch.zeros(5, 1, ps, dh, dtype=dtype, device=DEV), torch.zeros(5, 1, dh, ps, dtype=dtype, device=DEV)
+    both("norm_pair_write", lambda: (z, qw, wq, wk, 1e-5, torch.zeros(T, qw, dtype=dtype, device=DEV), slot_map, k, v, True, True), [5, 7, 8], dtype)
+    assert torch.equal(k[:, 0], v[:, 0].transpose(1, 2)) and float(k.float().abs().sum()) > 0
