@@ -30,6 +30,10 @@ decode steps and prefill (`fp32`).  Peaks are the published ones of MI355X.
                                                              sixteen experts and a shared one; gated sublayers, a token input behind
                                                              every layer) beside four Pafivik layers of the same width and feed-forward
                                                              sizes (lightning, attention, attention, lightning): prefill and decode
+    python bench.py --only fikupel [--width 1024] [--kernel-times]   four Fikupel layers (attention in a window that keeps first tokens,
+                                                             latent attention in a window, both again; a dense feed-forward, then
+                                                             sixteen experts; the stream in four copies) beside four Nigilorn layers
+                                                             of the same kinds and sizes: prefill and decode
 """
 import argparse
 import json
@@ -199,8 +203,8 @@ def main():
     ap.add_argument("--shape", choices=["xl", "large", "medium"], default=None,
                     help="--only decode / prefill / replay: the layer sizes of BASELINE.json's configs[2], [3] or [4] "
                          "(default xl; for replay medium)")
-    ap.add_argument("--width", type=int, default=0, help="--only ridopel, pafivik, dogalorn, nigilorn: one width instead of 1,024 and 2,048")
-    ap.add_argument("--only", choices=["decode", "prefill", "serving", "replay", "ridopel", "pafivik", "dogalorn", "nigilorn"], default=None,
+    ap.add_argument("--width", type=int, default=0, help="--only ridopel, pafivik, dogalorn, nigilorn, fikupel: one width instead of 1,024 and 2,048")
+    ap.add_argument("--only", choices=["decode", "prefill", "serving", "replay", "ridopel", "pafivik", "dogalorn", "nigilorn", "fikupel"], default=None,
                     help="run one workload and print a short line (decode, prefill: for profiling; serving: "
                          "BASELINE.json's configs[3], GPT-2 Large shape, 64 requests through the scheduler; replay: "
                          "configs[4], GPT-2 Medium shape, against the plain implementation)")
@@ -218,6 +222,8 @@ def main():
         return dogalorn(a)
     if a.only == "nigilorn":
         return nigilorn(a)
+    if a.only == "fikupel":
+        return fikupel(a)
     if a.only == "replay":
         a.shape = a.shape or "medium"      # (configs[4] as written; --shape xl: the same replay at configs[2]'s sizes)
         return replay(a)
@@ -370,6 +376,43 @@ def nigilorn_configs(width, layers=4, vocab=32000, positions=2048):
     paf = dict(architecture="Pafivik", vocab=vocab, width=width, norm=dict(eps=1e-5), embedding=dict(scale=1.0), residual_mult=0.5,
                layers=[kinds[i % 4] for i in range(layers)], max_positions=positions, n_positions=positions, vocab_size=vocab)
     return nig, paf
+
+
+def fikupel_configs(width, layers=4, vocab=32000, positions=2048):
+    """-> (a Fikupel config, a Nigilorn config) of the same width, layers, vocabulary and positions, without Nigilorn's scan and
+    token input, so that both have the same kinds of layers in the same order: attention (heads of 64, a key head for every
+    four, half of a head turned with a stretched encoding, a window of 256; Fikupel's keeps 16 first tokens) and latent attention
+    (heads with values of 128, a kept key of 256 numbers, a window of 256; queries of 64 plain dimensions through a vector of
+    half the width, or of 64 + 32 from the stream), again both.  The first layer has a dense feed-forward of four times the width
+    (one product up, or a gated one), the others sixteen experts of the model's width of which a token uses two (gated with silu,
+    or one product and a squared relu).  Fikupel's stream is four copies."""
+    H, Hl = width // 64, width // 128
+    ff = dict(kind="dense", ff=4 * width)
+
+    def moe(**router):
+        return dict(kind="moe", expert=dict(ff=width), router=dict(experts=16, top=2, **router))
+
+    def att(scaling, **mask):
+        return dict(type="attention", mixer=dict(heads=H, kv_heads=max(1, H // 4), dim=64, vdim=64, scale=0.125, mask=dict(size=256, **mask),
+                                                 rot=dict(base=10000.0, dims=32, scaling=scaling)))
+
+    def four(a, b, experts):
+        kinds = [dict(a, mlp=ff), dict(b, mlp=experts), dict(a, mlp=experts), dict(b, mlp=experts)]
+        return dict(vocab=vocab, width=width, norm=dict(eps=1e-5), layers=[kinds[i % 4] for i in range(layers)], max_positions=positions,
+                    n_positions=positions, vocab_size=vocab)
+    lat = dict(type="latent_attention", mixer=dict(heads=Hl, dim=64, vdim=128, kv_rank=256, q_rank=width // 2, scale=0.125, mask=dict(size=256)))
+    fik = dict(four(att(dict(factor=4.0, original=512, low=1.0, high=4.0), keep_first=16), lat, moe()), architecture="Fikupel", streams=4)
+    stretch = dict(factor=4.0, original=512, fast=32.0, slow=1.0)
+    nlat = dict(type="latent_attention", mixer=dict(heads=Hl, dim=64, rot_dim=32, vdim=128, kv_rank=224, scale=96 ** -0.5, mask=dict(size=256),
+                                                    rot=dict(base=10000.0, dims=32, scaling=stretch)))
+    nig = dict(four(att(stretch), nlat, moe(scale=2.5, groups=dict(count=4, keep=2))), architecture="Nigilorn")
+    return fik, nig
+
+
+def fikupel(a):
+    """Prefill and decode steps of four Fikupel layers beside four Nigilorn layers of the same kinds and sizes (the closest of the
+    framework's models: attention and latent attention in a window, experts); with --kernel-times each model's kernels."""
+    return side_by_side(a, ("fikupel", "nigilorn"), fikupel_configs)
 
 
 def nigilorn(a):

@@ -31,7 +31,7 @@ struct EmbedTables {
 };
 
 template <typename TW>
-__global__ void embed_kernel(EmbedTables tb, float* __restrict__ x, int T, int E, int wide) {
+__global__ void embed_kernel(EmbedTables tb, float* __restrict__ x, int T, int E, int copies, int wide) {
   int t = blockIdx.x;
   if (t >= T) return;
   int id[EMBED_TABLES_MAX];
@@ -72,9 +72,11 @@ __global__ void embed_kernel(EmbedTables tb, float* __restrict__ x, int T, int E
 #pragma unroll
         for (int k = 0; k < VEC; ++k) v[k] = nan;
       }
-      float* dst = x + static_cast<size_t>(t) * E + e;
+      for (int c = 0; c < copies; ++c) {
+        float* dst = x + (static_cast<size_t>(c) * T + t) * E + e;
 #pragma unroll
-      for (int k = 0; k < VEC; k += 4) *reinterpret_cast<float4*>(dst + k) = float4{v[k], v[k + 1], v[k + 2], v[k + 3]};
+        for (int k = 0; k < VEC; k += 4) *reinterpret_cast<float4*>(dst + k) = float4{v[k], v[k + 1], v[k + 2], v[k + 3]};
+      }
     }
     return;
   }
@@ -89,16 +91,17 @@ __global__ void embed_kernel(EmbedTables tb, float* __restrict__ x, int T, int E
         v += a;
       }
     }
-    x[static_cast<size_t>(t) * E + e] = v;
+    for (int c = 0; c < copies; ++c) x[(static_cast<size_t>(c) * T + t) * E + e] = v;
   }
 }
 
-// tables, indices, rows, scales: n <= 4 entries each (host arrays); every table [rows_i, E] of table_dtype
+// tables, indices, rows, scales: n <= 4 entries each (host arrays); every table [rows_i, E] of table_dtype; the rows are
+// stored `copies` times, x [copies, T, E]
 extern "C" int dn_embed_sum(const void* const* tables, const int32_t* const* indices, const int* rows,
-                            const float* scales, int n, float* x, int T, int E, int table_dtype,
+                            const float* scales, int n, float* x, int T, int E, int copies, int table_dtype,
                             hipStream_t stream) {
   if (T <= 0) return 0;
-  if (n < 1 || n > EMBED_TABLES_MAX || E < 1) return DN_ERR_SHAPE;
+  if (n < 1 || n > EMBED_TABLES_MAX || E < 1 || copies < 1) return DN_ERR_SHAPE;
   EmbedTables tb{};
   tb.n = n;
   const int vec = table_dtype == DN_F32 ? 4 : 8;
@@ -110,9 +113,9 @@ extern "C" int dn_embed_sum(const void* const* tables, const int32_t* const* ind
   }
   dim3 grid(T), block(256);
   if (table_dtype == DN_F32)
-    hipLaunchKernelGGL(embed_kernel<float>, grid, block, 0, stream, tb, x, T, E, wide);
+    hipLaunchKernelGGL(embed_kernel<float>, grid, block, 0, stream, tb, x, T, E, copies, wide);
   else if (table_dtype == DN_BF16)
-    hipLaunchKernelGGL(embed_kernel<bf16_t>, grid, block, 0, stream, tb, x, T, E, wide);
+    hipLaunchKernelGGL(embed_kernel<bf16_t>, grid, block, 0, stream, tb, x, T, E, copies, wide);
   else
     return DN_ERR_DTYPE;
   return dn_launch_status();
@@ -120,13 +123,13 @@ extern "C" int dn_embed_sum(const void* const* tables, const int32_t* const* ind
 
 // the token table and, unless it is null, the position table
 extern "C" int dn_embed(const int32_t* tokens, const int32_t* positions, const void* wte, const void* wpe,
-                        float* x, int T, int E, int vocab, int n_pos, int table_dtype, float token_scale,
+                        float* x, int T, int E, int copies, int vocab, int n_pos, int table_dtype, float token_scale,
                         hipStream_t stream) {
   const void* tables[2] = {wte, wpe};
   const int32_t* indices[2] = {tokens, positions};
   const int rows[2] = {vocab, n_pos};
   const float scales[2] = {token_scale, 1.0f};
-  return dn_embed_sum(tables, indices, rows, scales, wpe ? 2 : 1, x, T, E, table_dtype, stream);
+  return dn_embed_sum(tables, indices, rows, scales, wpe ? 2 : 1, x, T, E, copies, table_dtype, stream);
 }
 
 // ---------------------------------------------------------------------------------------

@@ -1199,6 +1199,51 @@ __global__ __launch_bounds__(256) void norm_pair_write_kernel(const float* z, si
   }
 }
 
+// norm_pair_write_kernel for rows of up to 256 NC numbers: a thread's share of the row is asked for at once and stays in
+// registers, both sums meet in one exchange.
+template <int NC>
+__global__ __launch_bounds__(256) void norm_pair_write_held_kernel(const float* z, size_t ldz, int qw, int kw, const float* wq, const float* wk,
+                                                                   float eps, void* q_out, size_t ldq, const int* slot_map, void* k_pool,
+                                                                   void* v_pool, int dh, int page_size, int dt, int write, int value_normed) {
+  __shared__ float sh[2][4];
+  const size_t t = blockIdx.x;
+  const float* row = z + t * ldz;
+  const int slot = slot_map[t], all = qw + kw;
+  float v[NC], w[NC], sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int j = 0; j < NC; ++j) {
+    const int c = threadIdx.x + 256 * j;
+    v[j] = c < all ? row[c] : 0.f;
+    w[j] = c < qw ? wq[c] : (c < all ? wk[c - qw] : 0.f);
+  }
+#pragma unroll
+  for (int j = 0; j < NC; ++j) {
+    if (static_cast<int>(threadIdx.x) + 256 * j < qw) sq = fmaf(v[j], v[j], sq);
+    else sk = fmaf(v[j], v[j], sk);
+  }
+  sq = wave_sum(sq), sk = wave_sum(sk);
+  const int wave = threadIdx.x >> 6;
+  if ((threadIdx.x & 63) == 0) sh[0][wave] = sq, sh[1][wave] = sk;
+  __syncthreads();
+  sq = (sh[0][0] + sh[0][1]) + (sh[0][2] + sh[0][3]), sk = (sh[1][0] + sh[1][1]) + (sh[1][2] + sh[1][3]);
+  const float iq = 1.0f / sqrtf(sq / static_cast<float>(qw) + eps), ik = 1.0f / sqrtf(sk / static_cast<float>(kw) + eps);
+  const bool writes = write && slot >= 0;
+  const int page = writes ? slot / page_size : 0, off = writes ? slot % page_size : 0, Hkv = kw / dh;
+#pragma unroll
+  for (int j = 0; j < NC; ++j) {
+    const int c = threadIdx.x + 256 * j;
+    if (c < qw) {
+      store_as(q_out, t * ldq + c, dt, v[j] * iq * w[j]);
+    } else if (c < all && writes) {
+      const int h = (c - qw) / dh, d = (c - qw) % dh;
+      const size_t base = (static_cast<size_t>(page) * Hkv + h) * page_size * dh;
+      const float kn = v[j] * ik * w[j];
+      store_as(k_pool, base + static_cast<size_t>(off) * dh + d, dt, kn);
+      store_as(v_pool, base + static_cast<size_t>(d) * page_size + off, dt, value_normed ? kn : v[j]);
+    }
+  }
+}
+
 // ---- heads' queries, keys and values: normed, turned, to their places ------------------------------------------------
 // A row of z is [q: H x dk | k: G x dk | v: G x dv].  Each query and key is divided by its root mean square (eps inside the
 // root; eps < 0: it is not) and weighed entry by entry (wq, wk: dk numbers shared by the heads), then its first `dims` entries are turned in
@@ -1427,10 +1472,17 @@ __global__ __launch_bounds__(256) void streams_read_kernel(const float* xs, size
 // next_in given: the same workgroup then reads the new copies for the next sublayer, as streams_read_kernel does, into `out`.
 // y2 given: the result is the mean of two branches, each normed over the width first with a weight of its own:
 // y = (y / rms(y) * by + y2 / rms(y2) * by2) / 2 (the sums as rmsnorm_add_kernel makes them, one branch after the other).
+// top > 0: the result is a weighted sum of `top` rows of y, those of experts: sum_c weigh[row, c] * y[row * top + c], c ascending.
+__device__ __forceinline__ float weighed_rows(const float* y, size_t ldy, const float* weigh, size_t row, int top, int c) {
+  float acc = 0.f;
+  for (int q = 0; q < top; ++q) acc = fmaf(weigh[row * top + q], y[(row * top + q) * ldy + c], acc);
+  return acc;
+}
+
 __global__ __launch_bounds__(256) void streams_write_kernel(float* xs, size_t plane, int n, const float* mix, const float* w_out, const float* y,
                                                             size_t ldy, const float* y2, size_t ldy2, const float* by, const float* by2,
-                                                            float beps, const float* next_in, const float* g, float eps, void* out,
-                                                            int out_dt, size_t ldo, int width) {
+                                                            float beps, const float* weigh, int top, const float* next_in, const float* g,
+                                                            float eps, void* out, int out_dt, size_t ldo, int width) {
   __shared__ float sh[4];
   __shared__ float sm[STREAMS_MAX * STREAMS_MAX + 2 * STREAMS_MAX];
   const size_t row = blockIdx.x;
@@ -1458,7 +1510,7 @@ __global__ __launch_bounds__(256) void streams_write_kernel(float* xs, size_t pl
     float old[STREAMS_MAX];
 #pragma unroll
     for (int s = 0; s < STREAMS_MAX; ++s) old[s] = s < n ? xs[s * plane + row * width + c] : 0.f;
-    float yc = y[row * ldy + c];
+    float yc = top > 0 ? weighed_rows(y, ldy, weigh, row, top, c) : y[row * ldy + c];
     if (y2) yc = fmaf(0.5f, y2[row * ldy2 + c] * inv2 * by2[c], fmaf(0.5f, yc * inv1 * by[c], 0.f));
     float u = 0.f;
 #pragma unroll
@@ -1493,7 +1545,8 @@ __global__ __launch_bounds__(256) void streams_write_kernel(float* xs, size_t pl
 template <int NS, int NC>
 __global__ __launch_bounds__(256) void streams_write_held_kernel(float* xs, size_t plane, int n, const float* mix, const float* w_out,
                                                                  const float* y, size_t ldy, const float* y2, size_t ldy2, const float* by,
-                                                                 const float* by2, float beps, const float* next_in, const float* g,
+                                                                 const float* by2, float beps, const float* weigh, int top,
+                                                                 const float* next_in, const float* g,
                                                                  float eps, void* out, int out_dt, size_t ldo, int width) {
   __shared__ float sh[4];
   __shared__ float sm[STREAMS_MAX * STREAMS_MAX + 2 * STREAMS_MAX];
@@ -1504,12 +1557,21 @@ __global__ __launch_bounds__(256) void streams_write_held_kernel(float* xs, size
     const int c = threadIdx.x + 256 * k;
     const bool ok = c < width;
     const int cc = ok ? c : 0;
-    yv[k] = ok ? y[row * ldy + cc] : 0.f;
+    yv[k] = ok && top == 0 ? y[row * ldy + cc] : 0.f;
     y2v[k] = (y2 && ok) ? y2[row * ldy2 + cc] : 0.f;
     b1[k] = y2 ? by[cc] : 0.f, b2[k] = y2 ? by2[cc] : 0.f;
     gv[k] = (next_in && g) ? g[cc] : 1.0f;
 #pragma unroll
     for (int s = 0; s < NS; ++s) old[s][k] = (s < n && ok) ? xs[s * plane + row * width + cc] : 0.f;
+  }
+  for (int q = 0; q < top; ++q) {
+    const float wq = weigh[row * top + q];
+    const float* yq = y + (row * top + q) * ldy;
+#pragma unroll
+    for (int k = 0; k < NC; ++k) {
+      const int c = threadIdx.x + 256 * k;
+      yv[k] = fmaf(wq, c < width ? yq[c] : 0.f, yv[k]);
+    }
   }
   if (threadIdx.x < n * n) sm[threadIdx.x] = mix[threadIdx.x];
   if (threadIdx.x < n) {
@@ -1830,15 +1892,17 @@ int dn_streams_read(const float* xs, long long plane, int n, const float* w_in, 
 }
 
 int dn_streams_write(float* xs, long long plane, int n, const float* mix, const float* w_out, const float* y, long long ldy,
-                     const float* y2, long long ldy2, const float* by, const float* by2, float beps, const float* next_in,
-                     const float* g, float eps, void* out, int out_dt, long long ldo, int T, int width, hipStream_t stream) {
+                     const float* y2, long long ldy2, const float* by, const float* by2, float beps, const float* weigh, int top,
+                     const float* next_in, const float* g, float eps, void* out, int out_dt, long long ldo, int T, int width, hipStream_t stream) {
   if (next_in && !float_kind(out_dt)) return DN_ERR_DTYPE;
-  if (n < 1 || n > STREAMS_MAX || width < 1 || (next_in && !out) || (y2 && (!by || !by2))) return DN_ERR_SHAPE;
+  if (n < 1 || n > STREAMS_MAX || width < 1 || (next_in && !out) || (y2 && (!by || !by2)) || top < 0 ||
+      (top > 0 && (!weigh || y2)))
+    return DN_ERR_SHAPE;
   if (T == 0) return 0;
 #define DN_STREAMS_HELD(NS, NC)                                                                                              \
   hipLaunchKernelGGL((streams_write_held_kernel<NS, NC>), dim3(T), dim3(256), 0, stream, xs, static_cast<size_t>(plane), n, mix,    \
-                     w_out, y, static_cast<size_t>(ldy), y2, static_cast<size_t>(ldy2), by, by2, beps, next_in, g, eps, out, out_dt, \
-                     static_cast<size_t>(ldo), width)
+                     w_out, y, static_cast<size_t>(ldy), y2, static_cast<size_t>(ldy2), by, by2, beps, weigh, top, next_in, g, eps, out, \
+                     out_dt, static_cast<size_t>(ldo), width)
   // (up to 4 copies of rows up to 4,096 wide: a thread holds its share of the row; by the sizes alone, the same bits either way)
   if (n <= 2 && width <= 1024) DN_STREAMS_HELD(2, 4);
   else if (n <= 2 && width <= 2048) DN_STREAMS_HELD(2, 8);
@@ -1847,7 +1911,7 @@ int dn_streams_write(float* xs, long long plane, int n, const float* mix, const 
   else if (n <= 4 && width <= 4096) DN_STREAMS_HELD(4, 16);
   else
     hipLaunchKernelGGL(streams_write_kernel, dim3(T), dim3(256), 0, stream, xs, static_cast<size_t>(plane), n, mix, w_out, y,
-                       static_cast<size_t>(ldy), y2, static_cast<size_t>(ldy2), by, by2, beps, next_in, g, eps, out, out_dt,
+                       static_cast<size_t>(ldy), y2, static_cast<size_t>(ldy2), by, by2, beps, weigh, top, next_in, g, eps, out, out_dt,
                        static_cast<size_t>(ldo), width);
 #undef DN_STREAMS_HELD
   return dn_launch_status();
@@ -1859,8 +1923,14 @@ int dn_norm_pair_write(const float* z, long long ldz, int qw, int kw, const floa
   if (!float_kind(dt)) return DN_ERR_DTYPE;
   if (qw < 1 || kw != Hkv * dh || page_size < 1 || ldz < qw + kw || ldq < qw) return DN_ERR_SHAPE;
   if (T == 0) return 0;
-  hipLaunchKernelGGL(norm_pair_write_kernel, dim3(T), dim3(256), 0, stream, z, static_cast<size_t>(ldz), qw, kw, wq, wk, eps, q_out,
-                     static_cast<size_t>(ldq), slot_map, k_pool, v_pool, dh, page_size, dt, write, value_normed);
+#define DN_PAIR_WRITE(kernel)                                                                                            \
+  hipLaunchKernelGGL(kernel, dim3(T), dim3(256), 0, stream, z, static_cast<size_t>(ldz), qw, kw, wq, wk, eps, q_out, static_cast<size_t>(ldq), \
+                     slot_map, k_pool, v_pool, dh, page_size, dt, write, value_normed)
+  // (by the sizes alone, so that a row's sums do not depend on the step)
+  if (qw + kw <= 1024) DN_PAIR_WRITE(norm_pair_write_held_kernel<4>);
+  else if (qw + kw <= 3072) DN_PAIR_WRITE(norm_pair_write_held_kernel<12>);
+  else DN_PAIR_WRITE(norm_pair_write_kernel);
+#undef DN_PAIR_WRITE
   return dn_launch_status();
 }
 
@@ -1877,10 +1947,9 @@ int dn_norm_turn_write(const float* z, long long ldz, int H, int G, int dk, int 
   if (T == 0) return 0;
   const NormTurnArgs a{z, static_cast<size_t>(ldz), H, G, dk, dv, wq, wk, q_scale, eps, freq, dims, v_freq, v_dims, positions, q_out,
                        static_cast<size_t>(ldq), kept, slot_map, k_pool, v_pool, page_size, dt, write};
-  // (few rows: four vectors a workgroup, so that a step of decoded tokens is more than a handful of workgroups; many rows: one
-  // workgroup a row, whose angles are made once)
+  // (four vectors a workgroup: a wave that walks several waits for its loads and its sum once for each)
   const int groups = (H + 2 * G + 3) / 4;
-  hipLaunchKernelGGL(norm_turn_write_kernel, dim3(T, T <= 256 ? groups : 1), dim3(256), 0, stream, a);
+  hipLaunchKernelGGL(norm_turn_write_kernel, dim3(T, groups < 65535 ? groups : 65535), dim3(256), 0, stream, a);
   return dn_launch_status();
 }
 

@@ -95,8 +95,8 @@ def _declare(name, lib):
     P, I, F = c_void_p, c_int, c_float
     sigs = {
         "elementwise": {
-            "dn_embed": [P, P, P, P, P, I, I, I, I, I, F, P],
-            "dn_embed_sum": [P, P, P, P, I, P, I, I, I, P],
+            "dn_embed": [P, P, P, P, P, I, I, I, I, I, I, F, P],
+            "dn_embed_sum": [P, P, P, P, I, P, I, I, I, I, P],
             "dn_logits_post": [P, I, I, I, F, F, P],
             "dn_layernorm": [P, P, P, P, P, I, I, F, I, I, P],
             "dn_layernorm_join": [P, P, I, c_longlong, P, P, P, P, I, I, F, I, I, P],
@@ -147,7 +147,7 @@ def _declare(name, lib):
             "dn_step_sizes": [P, c_longlong, P, P, P, c_longlong, I, I, I, P, c_longlong, P, c_longlong, P],
             "dn_gate_scan": [P, c_longlong, P, c_longlong, P, c_longlong, P, P, P, c_longlong, P, P, I, I, I, P, I, c_longlong, P],
             "dn_streams_read": [P, c_longlong, I, P, P, F, P, I, c_longlong, P, I, I, P],
-            "dn_streams_write": [P, c_longlong, I, P, P, P, c_longlong, P, c_longlong, P, P, F, P, P, F, P, I, c_longlong, I, I, P],
+            "dn_streams_write": [P, c_longlong, I, P, P, P, c_longlong, P, c_longlong, P, P, F, P, I, P, P, F, P, I, c_longlong, I, I, P],
             "dn_norm_pair_write": [P, c_longlong, I, I, P, P, F, P, c_longlong, P, P, P, I, I, I, I, I, I, I, P],
             "dn_norm_turn_write": [P, c_longlong, I, I, I, I, P, P, P, F, P, I, P, I, P, P, c_longlong, I, P, P, P, I, I, I, I, P],
             "dn_turn_back_gate": [P, I, c_longlong, I, P, c_longlong, P, P, P, I, c_longlong, I, I, I, P],
@@ -242,21 +242,28 @@ _FLOATS = (torch.float32, torch.bfloat16)
 _I32 = (torch.int32,)
 
 
+def _copies(out, T, E, what):
+    _need(out.is_contiguous() and out.dim() in (2, 3) and tuple(out.shape[-2:]) == (T, E), lambda: f"{what}: rows {tuple(out.shape)}")
+    return out.shape[0] if out.dim() == 3 else 1
+
+
 def embed(tokens, positions, wte, wpe, out, token_scale=1.0):
-    """out[t,:] = wte[tokens[t],:] * token_scale + wpe[positions[t],:]; wpe may be None.  out is 32-bit."""
+    """out[t,:] = wte[tokens[t],:] * token_scale + wpe[positions[t],:]; wpe may be None.  out is 32-bit, [T, E], or
+    [copies, T, E]: the rows are stored that many times."""
     T = tokens.shape[0]
     _dev(tokens, "tokens", _I32, 1), _dev(positions, "positions", _I32, 1)
-    _dev(wte, "wte", _FLOATS, 2), _dev(out, "out", (torch.float32,), 2)
+    _dev(wte, "wte", _FLOATS, 2), _dev(out, "out", (torch.float32,))
     _need(tokens.is_contiguous() and positions.is_contiguous() and positions.shape[0] == T, "tokens/positions")
     E = wte.shape[1]
-    _need(wte.is_contiguous() and out.is_contiguous() and tuple(out.shape) == (T, E), "embed: shapes")
+    copies = _copies(out, T, E, "embed")
+    _need(wte.is_contiguous(), "embed: wte")
     n_pos = 0
     if wpe is not None:
         _dev(wpe, "wpe", (wte.dtype,), 2)
         _need(wpe.is_contiguous() and wpe.shape[1] == E, "embed: wpe shape")
         n_pos = wpe.shape[0]
     _ok(_lib("elementwise").dn_embed(tokens.data_ptr(), positions.data_ptr(), wte.data_ptr(), _ptr(wpe),
-                                     out.data_ptr(), T, E, wte.shape[0], n_pos, _CODE[wte.dtype], float(token_scale),
+                                     out.data_ptr(), T, E, copies, wte.shape[0], n_pos, _CODE[wte.dtype], float(token_scale),
                                      _stream()), "embed")
     return out
 
@@ -266,11 +273,12 @@ EMBED_TABLES_MAX = 4
 
 def embed_sum(parts, out):
     """out[t,:] = sum over parts, in their order, of table[index[t],:] * scale.  parts: up to four
-    (table [rows, E], index int32 [T], scale); all tables of one dtype; out is 32-bit [T, E]."""
+    (table [rows, E], index int32 [T], scale); all tables of one dtype; out is 32-bit [T, E], or [copies, T, E]:
+    the rows are stored that many times."""
     _need(1 <= len(parts) <= EMBED_TABLES_MAX, lambda: f"embed_sum: 1 to {EMBED_TABLES_MAX} tables, not {len(parts)}")
-    _dev(out, "out", (torch.float32,), 2)
-    T, E = out.shape
-    _need(out.is_contiguous(), "embed_sum: out")
+    _dev(out, "out", (torch.float32,))
+    T, E = out.shape[-2:]
+    copies = _copies(out, T, E, "embed_sum")
     dtype = parts[0][0].dtype
     n = len(parts)
     tables, indices = (c_void_p * n)(), (c_void_p * n)()
@@ -281,7 +289,7 @@ def embed_sum(parts, out):
         _need(table.is_contiguous() and table.shape[1] == E, lambda: f"embed_sum: table {i} is {tuple(table.shape)}, rows are {E} wide")
         _need(index.is_contiguous() and index.shape[0] == T, lambda: f"embed_sum: index {i}")
         tables[i], indices[i], rows[i], scales[i] = table.data_ptr(), index.data_ptr(), table.shape[0], float(scale)
-    _ok(_lib("elementwise").dn_embed_sum(tables, indices, rows, scales, n, out.data_ptr(), T, E, _CODE[dtype], _stream()),
+    _ok(_lib("elementwise").dn_embed_sum(tables, indices, rows, scales, n, out.data_ptr(), T, E, copies, _CODE[dtype], _stream()),
         "embed")
     return out
 
@@ -1423,14 +1431,20 @@ def streams_read(xs, w_in, weight, eps, out, rows=None):
     return out
 
 
-def streams_write(xs, y, mix, w_out, next_in=None, weight=None, eps=0.0, out=None, branches=None):
+def streams_write(xs, y, mix, w_out, next_in=None, weight=None, eps=0.0, out=None, branches=None, weigh=None):
     """Every copy anew from the old ones and a sublayer's result: xs[t] <- sum_s mix[s, t] xs[s] + w_out[t] * y, in place.
     next_in given: the same kernel then reads the new copies as streams_read(xs, next_in, weight, eps, out) does.
     branches = (y2, w1, w2, eps): the result is the mean of two branches, each normed over the width first with a weight of its
-    own: (y / rms(y) * w1 + y2 / rms(y2) * w2) / 2, as two calls of rmsnorm_add with mult 1/2 into zeros make it."""
+    own: (y / rms(y) * w1 + y2 / rms(y2) * w2) / 2, as two calls of rmsnorm_add with mult 1/2 into zeros make it.
+    weigh: 32-bit [T, top]: the result is sum_c weigh[t, c] * y[t * top + c], y [T * top, width], as moe_combine into zeros makes it."""
     n, T, width = _streams(xs, "streams_write")
     _dev(y, "y", (torch.float32,), 2)
-    _need(tuple(y.shape) == (T, width), "streams_write: y")
+    top = 0
+    if weigh is not None:
+        _dev(weigh, "weigh", (torch.float32,), 2)
+        top = weigh.shape[1]
+        _need(weigh.is_contiguous() and weigh.shape[0] == T and top >= 1 and branches is None, "streams_write: weigh")
+    _need(tuple(y.shape) == (T * max(top, 1), width), "streams_write: y")
     _f32vec(mix, "mix", n * n), _f32vec(w_out, "w_out", n), _f32vec(next_in, "next_in", n), _f32vec(weight, "weight", width)
     y2 = w1 = w2 = None
     beps = 0.0
@@ -1443,7 +1457,7 @@ def streams_write(xs, y, mix, w_out, next_in=None, weight=None, eps=0.0, out=Non
         _dev(out, "out", _FLOATS, 2)
         _need(tuple(out.shape) == (T, width), "streams_write: out")
     _ok(_lib("sequence").dn_streams_write(xs.data_ptr(), T * width, n, mix.data_ptr(), w_out.data_ptr(), y.data_ptr(), _rows(y, "y"),
-                                          _ptr(y2), _rows(y2, "y2") if y2 is not None else 0, _ptr(w1), _ptr(w2), float(beps),
+                                          _ptr(y2), _rows(y2, "y2") if y2 is not None else 0, _ptr(w1), _ptr(w2), float(beps), _ptr(weigh), top,
                                           _ptr(next_in), _ptr(weight), float(eps), _ptr(out) if next_in is not None else 0,
                                           _CODE[out.dtype] if next_in is not None else 0,
                                           _rows(out, "out") if next_in is not None else 0, T, width, _stream()), "streams_write")

@@ -266,14 +266,18 @@ class MultiStreamBlock:
         # (a mixer of two branches hands both results over: their norms and their mean happen in the write's kernel)
         pair = self.mixer.forward_pair(h, ctx, caches) if hasattr(self.mixer, "forward_pair") else None
         y, branches = pair if pair is not None else (SandwichBlock._result(self.mixer, xs[0], h, ctx, cache), None)
+        weigh = None
         nxt = getattr(runtime, "next_read", None)
         if self.has_ffn:
             h = self.hc1.write(xs, y, self.hc2, self.norm2, act, branches=branches)
-            y, branches = SandwichBlock._result(self.ffn, xs[0], h, ctx), None
+            # (experts' rows and weights are handed over as they are: the weighted sum happens in the write's kernel)
+            apart = self.ffn.forward_apart(h, ctx) if hasattr(self.ffn, "forward_apart") else None
+            y, weigh = apart if apart is not None else (SandwichBlock._result(self.ffn, xs[0], h, ctx), None)
+            branches = None
             last = self.hc2
         else:
             last = self.hc1
         if nxt is not None:
-            runtime.stream_rows = last.write(xs, y, nxt[0], nxt[1], act, branches=branches)
+            runtime.stream_rows = last.write(xs, y, nxt[0], nxt[1], act, branches=branches, weigh=weigh)
         else:
-            last.write(xs, y, branches=branches)
+            last.write(xs, y, branches=branches, weigh=weigh)

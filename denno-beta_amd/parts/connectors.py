@@ -37,13 +37,13 @@ class StreamMixer(Part):
         out = torch.empty(xs.shape[1:], dtype=out_dtype, device=xs.device)
         return ops.streams_read(xs, self.w_in, norm.weight, norm.eps, out)
 
-    def write(self, xs, y, then=None, norm=None, out_dtype=None, branches=None):
+    def write(self, xs, y, then=None, norm=None, out_dtype=None, branches=None, weigh=None):
         """The copies anew, in place.  then: the connector of the sublayer that reads the stream next; its read (with `norm`)
         then happens in the same kernel and its rows come back.  branches: y is the first of two results whose normed mean
-        is the sublayer's (ops.streams_write)."""
+        is the sublayer's; weigh: y is experts' rows, `weigh` their weights per row (ops.streams_write, both)."""
         if then is None:
-            ops.streams_write(xs, y, self.mix, self.w_out, branches=branches)
+            ops.streams_write(xs, y, self.mix, self.w_out, branches=branches, weigh=weigh)
             return None
         out = torch.empty(xs.shape[1:], dtype=out_dtype, device=xs.device)
         return ops.streams_write(xs, y, self.mix, self.w_out, next_in=then.w_in, weight=norm.weight, eps=norm.eps, out=out,
-                                 branches=branches)
+                                 branches=branches, weigh=weigh)

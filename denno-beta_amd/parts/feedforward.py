@@ -234,14 +234,20 @@ class RoutedExperts(Part):
                 self.down_dims = (E, self.width, self.inner)
         self.w_dtype = torch.bfloat16 if isinstance(self.w_up, ops.PackedMatrix) else self.w_up.dtype
 
-    def forward(self, h, ctx, accumulate_into):
+    def forward_apart(self, h, ctx):
+        """-> (the chosen experts' results [T * top, width], their weights [T, top]): for whoever adds the weighted sum up in a kernel
+        of its own (ops.streams_write's `weigh`); None where something else belongs to the result."""
+        if self.shared or self.weigh == "input":
+            return None
+        _, out, wts, _ = self._experts(h)
+        return out, wts
+
+    def _experts(self, h):
+        """-> (the router's result, the experts' results, the chosen ones' weights, h in the experts' precision)."""
         T, top, dev = h.shape[0], self.top, h.device
         wdt = self.w_dtype
         if h.dtype != wdt:        # (experts stored in 32-bit in a bfloat16 engine: their products run on widened rows)
             h = ops.cast(h.contiguous(), torch.empty(h.shape, dtype=wdt, device=dev))
-        returns = accumulate_into is None
-        if returns:
-            accumulate_into = torch.zeros((T, self.width), dtype=torch.float32, device=dev)
         z = self.router(h, out_dtype=torch.float32)
         ids = torch.empty((T, top), dtype=torch.int32, device=dev)
         wts = torch.empty((T, top), dtype=torch.float32, device=dev)
@@ -256,7 +262,15 @@ class RoutedExperts(Part):
                    kind=self.act, in_scale=wts if on_input else None)
         out = torch.empty((T * top, self.width), dtype=torch.float32, device=dev)
         ops.moe_down(y, order, offsets, self.w_down, out, dims=self.down_dims)
-        ops.moe_combine(out, None if on_input else wts, accumulate_into)
+        return z, out, wts, h
+
+    def forward(self, h, ctx, accumulate_into):
+        T, dev = h.shape[0], h.device
+        returns = accumulate_into is None
+        if returns:
+            accumulate_into = torch.zeros((T, self.width), dtype=torch.float32, device=dev)
+        z, out, wts, h = self._experts(h)
+        ops.moe_combine(out, None if self.weigh == "input" else wts, accumulate_into)
         if self.shared:
             n = self.shared["inner"]
             if not self.gated and not self.token_gate:

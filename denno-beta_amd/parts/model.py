@@ -274,8 +274,9 @@ class DecoderModel:
             x = kept[0]
         else:
             x = torch.empty((ctx.T, self.spec.width), dtype=torch.float32, device=rt.device)
+        rows = xs if xs is not None else x      # (every copy starts as the embedding stage's output)
         if not self.spec.extra_embeddings:
-            ops.embed(ctx.tokens, ctx.positions, self.embedding.weight, self.position.table(), x,
+            ops.embed(ctx.tokens, ctx.positions, self.embedding.weight, self.position.table(), rows,
                       token_scale=self.spec.embedding_scale)
         else:
             parts = [(self.embedding.weight, ctx.tokens, self.spec.embedding_scale)]
@@ -289,7 +290,7 @@ class DecoderModel:
                 else:
                     picked = getattr(ctx, t.index)
                 parts.append((self.extra_tables[t.name], picked, t.scale))
-            ops.embed_sum(parts, x)
+            ops.embed_sum(parts, rows)
         rt.stream_stats = rt.stream_deferred = rt.normed_rows = None      # nobody has left anything for a norm of these rows yet
         if self.embedding_norm is not None:
             x = self.embedding_norm.forward(x, torch.float32)
@@ -299,7 +300,6 @@ class DecoderModel:
                 kept[0].copy_(x)
             x = ops.depth_mix(kept, 1, self._one, kept[1])
         if xs is not None:
-            xs[1:].copy_(x)      # (every copy starts as the embedding stage's output)
             rt.stream_rows = None
         for i, call in enumerate(order):
             if xs is not None:

@@ -522,9 +522,11 @@ def streams_read(xs, w_in, weight, eps, out, rows=None):
     return out
 
 
-def streams_write(xs, y, mix, w_out, next_in=None, weight=None, eps=0.0, out=None, branches=None):
+def streams_write(xs, y, mix, w_out, next_in=None, weight=None, eps=0.0, out=None, branches=None, weigh=None):
     n = xs.shape[0]
     old = xs.double().clone()
+    if weigh is not None:
+        y = (y.double().view(xs.shape[1], weigh.shape[1], -1) * weigh.double()[:, :, None]).sum(dim=1)
     if branches is not None:
         y2, w1, w2, beps = branches
         unit = lambda v: v.double() / torch.sqrt((v.double() ** 2).mean(dim=-1, keepdim=True) + beps)      # noqa: E731

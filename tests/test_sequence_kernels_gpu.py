@@ -818,3 +818,35 @@ def test_a_normed_latent_kept_as_key_and_value(dtype):
     k, v = torch.zeros(5, 1, ps, dh, dtype=dtype, device=DEV), torch.zeros(5, 1, dh, ps, dtype=dtype, device=DEV)
     both("norm_pair_write", lambda: (z, qw, wq, wk, 1e-5, torch.zeros(T, qw, dtype=dtype, device=DEV), slot_map, k, v, True, True), [5, 7, 8], dtype)
     assert torch.equal(k[:, 0], v[:, 0].transpose(1, 2)) and float(k.float().abs().sum()) > 0
+
+
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("n,T,width,top", [(1, 3, 20, 1), (2, 9, 1000, 3), (4, 5, 1500, 2), (3, 4, 3000, 8), (6, 7, 260, 2), (4, 6, 4500, 2)])
+def test_experts_added_up_in_the_write_of_the_copies(dtype, n, T, width, top):
+    """Every width's kernel: against the reference, and the same bits as moe_combine into zeros followed by the write."""
+    xs, y = torch.randn(n, T, width, device=DEV), torch.randn(T * top, width, device=DEV)
+    weigh = torch.rand(T, top, device=DEV)
+    mix, w_out, w_in = torch.randn(n, n, device=DEV) / n, torch.randn(n, device=DEV), torch.randn(n, device=DEV)
+    g = torch.randn(width, device=DEV)
+    both("streams_write", lambda: (xs.clone(), y, mix, w_out, w_in, g, 1e-6, torch.empty(T, width, dtype=dtype, device=DEV), None, weigh), [0, 7], dtype)
+    a, b = xs.clone(), xs.clone()
+    one, two = (torch.empty(T, width, dtype=dtype, device=DEV) for _ in range(2))
+    ops.streams_write(a, y, mix, w_out, w_in, g, 1e-6, one, weigh=weigh)
+    summed = torch.zeros(T, width, device=DEV)
+    ops.moe_combine(y, weigh, summed)
+    ops.streams_write(b, summed, mix, w_out, w_in, g, 1e-6, two)
+    assert torch.equal(a, b) and torch.equal(one, two)
+
+
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("E", [7, 64])
+def test_rows_of_a_table_stored_as_several_copies(dtype, E):
+    T = 11
+    tables = [torch.randn(29, E, device=DEV).to(dtype) for _ in range(2)]
+    ids = [torch.randint(0, 29, (T,), dtype=torch.int32, device=DEV) for _ in range(2)]
+    for copies in (1, 3):
+        out = torch.zeros(copies, T, E, device=DEV)
+        ops.embed(ids[0], ids[1], tables[0], None, out, token_scale=2.0)
+        assert torch.equal(out, (tables[0][ids[0].long()].float() * 2.0).expand(copies, T, E))
+        ops.embed_sum([(tables[0], ids[0], 1.0), (tables[1], ids[1], 1.0)], out)
+        assert torch.equal(out, (tables[0][ids[0].long()].float() + tables[1][ids[1].long()].float()).expand(copies, T, E))
