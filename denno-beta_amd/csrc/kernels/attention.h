@@ -68,8 +68,8 @@ int dn_attention_flash_extras(const void* q, int ldq, void* out, int ldo, const 
                               int H, int Hkv, int dh, int page_size, float scale, int window, int chunk, const float* bias,
                               int span, int sink, const float* sink_at, int keep, hipStream_t stream);
 
-// bfloat16, one row per request (tile s = request s = row s); the context is cut into n_splits runs of
-// `chunks` chunks of waves * 64 keys; part: device memory for n_tiles * H * n_splits * (dh + 2) floats
+// bfloat16, one row per request (tile s = request s = row s); the tiles of 64 keys that a row reads are cut into n_splits runs
+// of `chunks` chunks of `waves` tiles; part: device memory for n_tiles * H * n_splits * (dh + 2) floats
 // of split results (not touched when n_splits == 1).  tile_row0 is not read: tile s is row s of q and
 // of out and row s of the block tables, whatever the table says (the kernels address them by the
 // workgroup's index, so that these loads do not wait for the table's); a caller whose tile s is

@@ -644,8 +644,8 @@ typedef __attribute__((__vector_size__(4 * sizeof(uint32_t)))) uint32_t u32x4;
 // POW2: the page size is a power of two (page_size = 1 << page_shift), so that a key's page and its place in
 // the page are a shift and a mask: a tile's keys need four such pairs a step, and a division by a number
 // known only at run time is some twenty-five vector instructions.
-// EXTRAS: chunks, a bias by distance, a sink and kept first keys (ScoreExtras).  A score is then the scaled product plus the bias, both
-// in units of log2(e), made before the maximum is taken (the largest product is no longer the largest score).
+// EXTRAS: chunks, a bias by distance, a sink and kept first keys (ScoreExtras).  With a bias a score is the scaled product
+// plus the bias, both in units of log2(e), made before the maximum is taken (the largest product is no longer the largest score).
 template <int DH16, int GROUPS, int TPS, bool POW2, bool EXTRAS = false>     // head size / 16; groups of 4 waves; tiles a wave takes per step
 __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH16 > 12 && GROUPS == 1 ? 1 : 2))) void kernel(
     const bf16_t* __restrict__ q, int ldq, bf16_t* __restrict__ out, int ldo, const bf16_t* __restrict__ k_pool,
@@ -699,6 +699,7 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
   const int keep = EXTRAS ? ex.keep : 0;
   const float NEG_INF = -INFINITY;
   const float scale2 = scale * 1.44269504088896340736f;    // log2(e)
+  const float per_score = EXTRAS && bias ? 1.0f : scale2;    // what is left to multiply a score with (a bias is added to scaled ones)
   const u32x4 zero4 = {0u, 0u, 0u, 0u};
 
   bf16x8 qf[DH16];
@@ -831,13 +832,12 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
         const int kw = kw0 + 32 * c;
         const bool edge = kw + 31 > pos0 + wrow0 || (kw < lo_last && kw + 31 >= keep);
         if (!act[c]) continue;
-        if constexpr (EXTRAS) {
+        if (EXTRAS && bias) {
 #pragma unroll
           for (int i = 0; i < 16; ++i) {
             const int key = kw + 8 * (i / 4) + 4 * g + (i % 4);
             const bool ok = reads_key(key, my_lo, my_pos, keep);
-            float sc = s[c][i] * scale2;
-            if (bias) sc = fmaf(bias[min(max(my_pos - key, 0), ex.span - 1)], 1.44269504088896340736f, sc);
+            const float sc = fmaf(bias[min(max(my_pos - key, 0), ex.span - 1)], 1.44269504088896340736f, s[c][i] * scale2);
             s[c][i] = (!edge || ok) ? sc : NEG_INF;
             tmax = fmaxf(tmax, s[c][i]);
           }
@@ -845,7 +845,7 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
 #pragma unroll
           for (int i = 0; i < 16; ++i) {
             int key = kw + 8 * (i / 4) + 4 * g + (i % 4);
-            bool ok = key >= my_lo && key <= my_pos;
+            const bool ok = reads_key(key, my_lo, my_pos, keep);
             s[c][i] = ok ? s[c][i] : NEG_INF;
             tmax = fmaxf(tmax, s[c][i]);
           }
@@ -854,7 +854,7 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
           for (int i = 0; i < 16; ++i) tmax = fmaxf(tmax, s[c][i]);
         }
       }
-      tmax = fmaxf(tmax, other_half(tmax)) * (EXTRAS ? 1.0f : scale2);      // (-inf stays -inf)
+      tmax = fmaxf(tmax, other_half(tmax)) * per_score;      // (-inf stays -inf)
       float p[TPS][16];
       float psum = 0.f, alpha = 1.f;
       if (tmax > NEG_INF) {
@@ -864,7 +864,7 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
         for (int c = 0; c < TPS; ++c)
 #pragma unroll
           for (int i = 0; i < 16; ++i) {
-            p[c][i] = __builtin_amdgcn_exp2f(EXTRAS ? s[c][i] - m_new : fmaf(s[c][i], scale2, -m_new));  // a masked score is -inf: 0
+            p[c][i] = __builtin_amdgcn_exp2f(fmaf(s[c][i], per_score, -m_new));  // a masked score is -inf: 0
             psum += p[c][i];
           }
         m = m_new;
@@ -1038,7 +1038,8 @@ extern "C" int dn_attention_flash_extras(const void* q, int ldq, void* out, int 
 // decode: one row per request, request s being tile s and row s of the step (tile_seq[s] < 0:
 // padding; tile_pos0[s]: its position).  A workgroup has 4, 8 or 16 waves, 64 keys each at a time
 // (its chunk: 256, 512 or 1024 keys), chosen so that a short context is one chunk: every load of
-// a wave is then issued at once, behind one lookup of its pages.  The context is cut into
+// a wave is then issued at once, behind one lookup of its pages.  The tiles of 64 keys that the row reads (all of its
+// context, or, in a window, those of the kept first keys and of the window: what lies between is not walked) are cut into
 // n_splits runs of `chunks` chunks; a workgroup walks its run chunk by chunk (each wave with a
 // running maximum, sum and weighted values, joined through LDS at the end) and, if there is
 // more than one split, a second kernel joins the splits' results in split order
@@ -1075,7 +1076,6 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
   constexpr int KPI = 64 / LPK;          // keys per load instruction
   constexpr int DPL = (DH + 63) / 64;    // dims per lane in the second product
   constexpr int GROUP = LPK < 8 ? LPK : 8;   // load instructions issued together
-  constexpr int CHUNK = WAVES * 64;          // keys that the workgroup's waves take at a time
   __shared__ float wm[WAVES], wl[WAVES];
   __shared__ float wacc[WAVES][DH];
   // In a step of single rows request s brings row s and is tile s: the block table and the query
@@ -1093,10 +1093,13 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
   const int lo = first_key(pos, window, EXTRAS ? ex.chunk : 0);
   const float* bias = EXTRAS && ex.bias ? ex.bias + static_cast<size_t>(h) * ex.span : nullptr;
   const int keep = EXTRAS ? ex.keep : 0;
-  const int key0 = split * chunks * CHUNK;
+  // the tiles of 64 keys that the row reads, counted from 0: those of the kept first keys, then those from `lo` on
+  const int kept_tiles = (keep + 63) / 64, rest = max(lo / 64, kept_tiles), last_tile = pos / 64;
+  const int n_tiles_read = kept_tiles > last_tile ? last_tile + 1 : kept_tiles + (last_tile - rest + 1);
+  const int first_tile = split * chunks * WAVES;
   const float NEG_INF = -INFINITY;
   float* mypart = part + ((static_cast<size_t>(tile) * H + h) * n_splits + split) * (DH + 2);
-  if (key0 > pos || (key0 + chunks * CHUNK <= lo && key0 >= keep)) {
+  if (first_tile >= n_tiles_read) {
     if (n_splits > 1 && threadIdx.x == 0) {
       mypart[0] = NEG_INF;     // the join skips it
       mypart[1] = 0.f;
@@ -1113,8 +1116,9 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
   for (int i = 0; i < DPL; ++i) acc[i] = 0.f;
 
   for (int c = 0; c < chunks; ++c) {
-    const int kbase = key0 + c * CHUNK + wave * 64;
-    if (kbase > pos || (kbase + 64 <= lo && kbase >= keep)) continue;     // the same for the whole wave; no barrier in this loop
+    const int tile_no = first_tile + c * WAVES + wave;
+    if (tile_no >= n_tiles_read) continue;     // the same for the whole wave; no barrier in this loop
+    const int kbase = 64 * (tile_no < kept_tiles ? tile_no : rest + (tile_no - kept_tiles));
     // values: lane = dim; 16 keys of one page at a time.  They are asked for first, before the keys
     // (whose use would otherwise stand between them and memory): keys and values then make one trip
     bf16x8 v0[4][DPL], v1[4][DPL];
@@ -1255,7 +1259,8 @@ __global__ void join_kernel(const float* __restrict__ part, bf16_t* __restrict__
 
 // part: 32-bit workspace of n_tiles * H * n_splits * (dh + 2) floats (unused when n_splits == 1);
 // waves: 4, 8 or 16 per workgroup (16 up to a head size of 64, 8 up to 128); the splits cover
-// n_splits * chunks * waves * 64 keys, which must reach the longest context.
+// n_splits * chunks * waves tiles of 64 keys, which must be as many as the longest context has, or, in a window, as hold the keys
+// that a row reads: (window + 62) / 64 + 1 and (keep + 63) / 64 more.
 // ldo == 0: out is a packed matrix of H * dh columns (a multiple of 32)
 extern "C" int dn_attention_decode(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                                    const int32_t* block_tables, int max_blocks, const int32_t* tile_seq,

@@ -1249,8 +1249,8 @@ __global__ __launch_bounds__(256) void norm_pair_write_held_kernel(const float* 
 // root; eps < 0: it is not) and weighed entry by entry (wq, wk: dk numbers shared by the heads), then its first `dims` entries are turned in
 // neighbouring pairs by position * freq; a value's first v_dims entries are turned by position * v_freq.  A query times
 // q_scale[head] goes to q_out (heads `kept` columns wide), keys and values to the cache's pools (heads `kept` wide, the row's
-// place from slot_map; a negative place: nothing is written); columns a vector does not have are zeros.  A wave a vector: a
-// lane holds the pairs lane and lane + 64, the squares are summed over the wave in one order.
+// place from slot_map; a negative place: nothing is written); columns a vector does not have are zeros.  LPV lanes (a wave, or half
+// of one) share a vector: a lane holds the pairs lane, lane + LPV, .. (J of them), the squares are summed over them in one order.
 struct NormTurnArgs {
   const float* z;
   size_t ldz;
@@ -1281,21 +1281,23 @@ __device__ __forceinline__ void store_pair(void* p, size_t i, int dt, float a, f
   }
 }
 
+template <int LPV, int J>
 __global__ __launch_bounds__(256) void norm_turn_write_kernel(NormTurnArgs a) {
   __shared__ float cs[256], sn[256];      // the row's angles: the keys' pairs, then the values' (at most 128 each)
   const size_t t = blockIdx.x;
-  const int lane = threadIdx.x & 63;
+  constexpr int AT_ONCE = 256 / LPV;      // vectors of a workgroup side by side
+  const int lane = threadIdx.x % LPV;
   const int half = a.dims / 2, v_half = a.v_dims / 2, n_vec = a.H + 2 * a.G;
   const float p = static_cast<float>(a.positions[t]);
   if (threadIdx.x < half + v_half) {
     const float ang = p * (threadIdx.x < half ? a.freq[threadIdx.x] : a.v_freq[threadIdx.x - half]);
-    cs[threadIdx.x] = cosf(ang), sn[threadIdx.x] = sinf(ang);
+    sincosf(ang, &sn[threadIdx.x], &cs[threadIdx.x]);
   }
   __syncthreads();
   const int slot = a.slot_map[t];
   const bool writes = a.write && slot >= 0;
   const int page = writes ? slot / a.page_size : 0, off = writes ? slot % a.page_size : 0;
-  for (int vec = blockIdx.y * 4 + (threadIdx.x >> 6); vec < n_vec; vec += gridDim.y * 4) {      // (the whole wave)
+  for (int vec = blockIdx.y * AT_ONCE + threadIdx.x / LPV; vec < n_vec; vec += gridDim.y * AT_ONCE) {      // (all lanes of a vector)
     const bool is_q = vec < a.H, is_v = vec >= a.H + a.G;
     if (!is_q && !writes) continue;
     const int n = is_q ? vec : (is_v ? vec - a.H - a.G : vec - a.H);      // the head's number among its kind
@@ -1303,20 +1305,20 @@ __global__ __launch_bounds__(256) void norm_turn_write_kernel(NormTurnArgs a) {
     const float* src = a.z + t * a.ldz + (is_v ? static_cast<size_t>(a.H + a.G) * a.dk + static_cast<size_t>(n) * a.dv
                                                : static_cast<size_t>(vec) * a.dk);
     const float* w = is_q ? a.wq : (is_v ? nullptr : a.wk);
-    float lo[2], hi[2], ss = 0.f;
+    float lo[J], hi[J], ss = 0.f;
 #pragma unroll
-    for (int j = 0; j < 2; ++j) {
-      const int e = 2 * (lane + 64 * j);
+    for (int j = 0; j < J; ++j) {
+      const int e = 2 * (lane + LPV * j);
       lo[j] = e < width ? src[e] : 0.f;
       hi[j] = e + 1 < width ? src[e + 1] : 0.f;
       ss = fmaf(lo[j], lo[j], ss);
       ss = fmaf(hi[j], hi[j], ss);
     }
-    const float inv = is_v || a.eps < 0.f ? 1.0f : 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(width) + a.eps);
+    const float inv = is_v || a.eps < 0.f ? 1.0f : 1.0f / sqrtf(group_reduce<LPV>(ss, SumOp()) / static_cast<float>(width) + a.eps);
     const float times = is_q && a.q_scale ? a.q_scale[n] : 1.0f;
 #pragma unroll
-    for (int j = 0; j < 2; ++j) {
-      const int i = lane + 64 * j, e = 2 * i;
+    for (int j = 0; j < J; ++j) {
+      const int i = lane + LPV * j, e = 2 * i;
       if (e >= a.kept) continue;
       float x = lo[j], y = hi[j];
       if (!is_v) {
@@ -1359,7 +1361,7 @@ __global__ __launch_bounds__(256) void turn_back_gate_kernel(const void* o, int 
   if (freq) {
     if (threadIdx.x < per) {
       const float ang = static_cast<float>(positions[t]) * freq[threadIdx.x];
-      cs[threadIdx.x] = cosf(ang), sn[threadIdx.x] = sinf(ang);
+      sincosf(ang, &sn[threadIdx.x], &cs[threadIdx.x]);
     }
     __syncthreads();
   }
@@ -1465,6 +1467,50 @@ __global__ __launch_bounds__(256) void streams_read_kernel(const float* xs, size
       if (s < n) u = fmaf(wi[s], xs[s * plane + src + c], u);
     u *= inv;
     store_as(out, static_cast<size_t>(r) * ldo + c, out_dt, g ? u * g[c] : u);
+  }
+}
+
+// streams_read_kernel for rows of up to 256 NC columns and up to NS copies: a thread's share of the row is asked for at once and
+// stays in registers between the sum and the store.  The same sums in the same order: the same bits.
+template <int NS, int NC>
+__global__ __launch_bounds__(256) void streams_read_held_kernel(const float* xs, size_t plane, int n, const float* w_in, const float* g,
+                                                                float eps, void* out, int out_dt, size_t ldo, const int* rows, int width) {
+  __shared__ float sh[4];
+  const int r = blockIdx.x;
+  const size_t src = static_cast<size_t>(rows ? rows[r] : r) * width;
+  float x[NS][NC], gv[NC], u[NC];
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = threadIdx.x + 256 * k;
+    const bool ok = c < width;
+#pragma unroll
+    for (int s = 0; s < NS; ++s) x[s][k] = ok && s < n ? xs[s * plane + src + c] : 0.f;
+    gv[k] = g && ok ? g[c] : 1.0f;
+  }
+  float wi[NS];
+#pragma unroll
+  for (int s = 0; s < NS; ++s) wi[s] = s < n ? (w_in ? w_in[s] : 1.0f) : 0.f;
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    u[k] = 0.f;
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+      if (s < n) u[k] = fmaf(wi[s], x[s][k], u[k]);
+    ss = fmaf(u[k], u[k], ss);
+  }
+  float inv = 1.0f;
+  if (eps >= 0.f) {
+    ss = block_sum_256(ss, sh);
+    inv = 1.0f / sqrtf(ss / static_cast<float>(width) + eps);
+  }
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = threadIdx.x + 256 * k;
+    if (c < width) {
+      const float v = u[k] * inv;
+      store_as(out, static_cast<size_t>(r) * ldo + c, out_dt, g ? v * gv[k] : v);
+    }
   }
 }
 
@@ -1886,8 +1932,13 @@ int dn_streams_read(const float* xs, long long plane, int n, const float* w_in, 
   if (!float_kind(out_dt)) return DN_ERR_DTYPE;
   if (n < 1 || n > STREAMS_MAX || width < 1) return DN_ERR_SHAPE;
   if (R == 0) return 0;
-  hipLaunchKernelGGL(streams_read_kernel, dim3(R), dim3(256), 0, stream, xs, static_cast<size_t>(plane), n, w_in, g, eps, out, out_dt,
-                     static_cast<size_t>(ldo), rows, width);
+#define DN_STREAMS_READ(kernel)                                                                                               \
+  hipLaunchKernelGGL((kernel), dim3(R), dim3(256), 0, stream, xs, static_cast<size_t>(plane), n, w_in, g, eps, out, out_dt,    \
+                     static_cast<size_t>(ldo), rows, width)
+  if (n <= 4 && width <= 1024) DN_STREAMS_READ((streams_read_held_kernel<4, 4>));
+  else if (n <= 4 && width <= 2048) DN_STREAMS_READ((streams_read_held_kernel<4, 8>));
+  else DN_STREAMS_READ(streams_read_kernel);
+#undef DN_STREAMS_READ
   return dn_launch_status();
 }
 
@@ -1947,9 +1998,13 @@ int dn_norm_turn_write(const float* z, long long ldz, int H, int G, int dk, int 
   if (T == 0) return 0;
   const NormTurnArgs a{z, static_cast<size_t>(ldz), H, G, dk, dv, wq, wk, q_scale, eps, freq, dims, v_freq, v_dims, positions, q_out,
                        static_cast<size_t>(ldq), kept, slot_map, k_pool, v_pool, page_size, dt, write};
-  // (four vectors a workgroup: a wave that walks several waits for its loads and its sum once for each)
-  const int groups = (H + 2 * G + 3) / 4;
-  hipLaunchKernelGGL(norm_turn_write_kernel, dim3(T, groups < 65535 ? groups : 65535), dim3(256), 0, stream, a);
+  // (few rows: the vectors of a row spread over workgroups, so that a step of decoded tokens is more than a handful of them; many
+  // rows: one workgroup a row, whose angles are made once.  By the sizes alone a vector has 32 or 64 lanes: the same bits either way)
+  const int at_once = kept <= 64 ? 8 : 4, groups = T <= 256 ? (H + 2 * G + at_once - 1) / at_once : 1;
+  const dim3 grid(T, groups < 65535 ? groups : 65535);
+  if (kept <= 64) hipLaunchKernelGGL((norm_turn_write_kernel<32, 1>), grid, dim3(256), 0, stream, a);
+  else if (kept <= 128) hipLaunchKernelGGL((norm_turn_write_kernel<64, 1>), grid, dim3(256), 0, stream, a);
+  else hipLaunchKernelGGL((norm_turn_write_kernel<64, 2>), grid, dim3(256), 0, stream, a);
   return dn_launch_status();
 }
 

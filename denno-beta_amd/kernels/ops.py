@@ -697,11 +697,15 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
         # (where the batch alone gives two workgroups or more per CU the chip is busy anyway, and
         # the smallest workgroups were measured fastest)
         groups = n_tiles * n_heads
+        # (in a window or a chunk the kernel walks the tiles of 64 keys that hold what a row reads, wherever they lie)
+        reach = max_context
+        for span_keys in ([window] if window > 0 else []) + ([chunk] if chunk > 0 else []):
+            reach = min(reach, 64 * ((span_keys + 62) // 64 + 1 + -(-keep_first // 64)))
         # (a head size that is no power of two leaves lanes empty and needs more registers: from a thousand
         # workgroups on its smallest ones are up to a third faster, where the others' sizes are level)
         many = 8 if dh & (dh - 1) == 0 else 4
-        waves = (4 if max_context <= 256 else many if groups >= 1024 else 4 if groups >= 512 else
-                 8 if groups >= 300 or max_context <= 512 else 16)
+        waves = (4 if reach <= 256 else many if groups >= 1024 else 4 if groups >= 512 else
+                 8 if groups >= 300 or reach <= 512 else 16)
         waves = min(waves, 16 if dh <= 64 else 8 if dh <= 128 else 4)
         if decode_waves is not None:       # (for measurements and tests: 4, 8 or 16 as far as the head size allows)
             _need(decode_waves in (4, 8, 16) and decode_waves <= (16 if dh <= 64 else 8 if dh <= 128 else 4),
@@ -709,7 +713,7 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
             waves = decode_waves
         # the context is split over workgroups only where the batch alone does not give about one
         # workgroup per CU: a second kernel has to join the splits
-        total_chunks = -(-max_context // (waves * 64))
+        total_chunks = -(-reach // (waves * 64))
         n_splits = max(1, min(total_chunks, 256 // max(1, n_tiles * n_heads)))
         chunks = -(-total_chunks // n_splits)
         n_splits = -(-total_chunks // chunks)
