@@ -268,11 +268,10 @@ ALONE = {
 }
 
 
-@pytest.mark.parametrize("streams", [0, 1, 2, 4, 7])
-@pytest.mark.parametrize("what", sorted(ALONE))
+# (every number of copies with three of the mechanisms, two with all)
+@pytest.mark.parametrize("what,streams", [(w, n) for w in sorted(ALONE) for n in (0, 2)]
+                         + [(w, n) for w in ("attention_first_kept", "experts", "dense") for n in (1, 4, 7)])
 def test_each_mechanism_alone(backend, folders, what, streams):
-    if streams in (1, 4, 7) and what not in ("attention_first_kept", "experts", "dense"):
-        pytest.skip("every number of copies with three of the mechanisms only")
     cfg = config(ALONE[what], width=24, vocab=53, streams=streams)
     folder = folders(f"alone_{what}_{streams}", "float32", cfg, 5)
     seq = seqs_for(cfg, [29])[0]
