@@ -1388,7 +1388,7 @@ __global__ __launch_bounds__(256) void turn_back_gate_kernel(const void* o, int 
 }
 
 // ---- a polynomial of normed powers ----------------------------------------------------------------------------------
-// out = a N(z) + b N(z^2) + c N(z^3) + e with (a, b, c, e) the four numbers, powers entry by entry, N the division of a row by its
+// out = s_1 n(z) + s_2 n(z^2) + s_3 n(z^3) + s_0, numbers = (s_1, s_2, s_3, s_0), with entrywise powers and n the division of a row by its
 // root mean square (eps inside the root).  One workgroup a row; up to 256 NC columns a thread holds its share of the row (NC 0:
 // it reads it twice); a thread sums its own columns in ascending order, waves are joined in order.
 template <int NC>

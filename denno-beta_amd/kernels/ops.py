@@ -1535,7 +1535,7 @@ def turn_back_gate(o, n_heads, dv, out, positions=None, freq=None, gate=None, he
 
 
 def poly_norm(z, numbers, eps, out):
-    """out = a N(z) + b N(z^2) + c N(z^3) + e with (a, b, c, e) = numbers (32-bit), powers entry by entry, N(v) = v / sqrt(mean(v^2) + eps)
+    """out = s_1 n(z) + s_2 n(z^2) + s_3 n(z^3) + s_0, numbers = (s_1, s_2, s_3, s_0), 32-bit; powers are entrywise and n(v) = v / sqrt(mean(v^2) + eps)
     over the row; z 32-bit."""
     _dev(z, "z", (torch.float32,), 2), _dev(out, "out", _FLOATS, 2)
     T, n = z.shape

@@ -22,8 +22,8 @@ class DenseMLP(Part):
 
     activation "xielu": z > 0: softplus(p) z^2 + z / 2; else (1/2 + softplus(q)) (e^z - 1 - z) + z / 2, with (p, q) the two
     numbers of the tensor `activation_params`; it runs as a kernel of its own on the first product's 32-bit result.
-    activation "poly_norm": a N(z) + b N(z^2) + c N(z^3) + e over the row of `inner` values, (a, b, c, e) the tensor's four numbers,
-    powers entry by entry, N(v) = v / sqrt(mean(v^2) + eps); likewise a kernel of its own."""
+    activation "poly_norm": s_1 n(z) + s_2 n(z^2) + s_3 n(z^3) + s_0 over the row of `inner` values, with s_1, s_2, s_3, s_0 the tensor's four
+    numbers in this order, entrywise powers and n(v) = v / sqrt(mean(v^2) + eps); likewise a kernel of its own."""
     graph_safe = True
     returns_rows = True
 

@@ -123,9 +123,9 @@ def latent_attention(h, p, m, eps):
 # ----------------------------------------------------------------------------
 
 def poly_norm(z, numbers, eps):
-    """a N(z) + b N(z^2) + c N(z^3) + e, N the division by the root mean square over the last dimension."""
-    a, b, c, e = numbers
-    return a * rms_norm(z, None, eps) + b * rms_norm(z ** 2, None, eps) + c * rms_norm(z ** 3, None, eps) + e
+    """The first three numbers weigh z and its (entrywise) square and cube, each divided by its own root mean square over the
+    last dimension; the fourth is added to every entry."""
+    return sum(numbers[k - 1] * rms_norm(z ** k, None, eps) for k in (1, 2, 3)) + numbers[3]
 
 
 def dense_ff(h, p, eps):
