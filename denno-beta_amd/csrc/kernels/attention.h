@@ -14,7 +14,8 @@
 // What a layer may add to the scores of any of the kernels below.  chunk > 0: the row at position p reads only keys from
 // p / chunk * chunk on; bias: 32-bit [H, span], bias[h][p - key] is added to the scaled score (distances from span on take
 // the last entry), or null; sink: a key without a value that every row sees, with score sink_at[h] (null: 0), which nothing
-// scales; keep: with a window, the first `keep` keys are read by every row as well.
+// scales; keep: with a window, the first `keep` keys are read by every row as well; cap > 0: a scaled score s becomes
+// cap * tanh(s / cap), before the bias.
 struct ScoreExtras {
   int chunk;
   const float* bias;
@@ -22,6 +23,7 @@ struct ScoreExtras {
   int sink;
   const float* sink_at;
   int keep;
+  float cap;
 };
 
 extern "C" {
@@ -35,16 +37,16 @@ int dn_attention(const void* q, int ldq, void* out, int ldo, const void* k_pool,
                  const int32_t* tile_nrows, const int32_t* tile_pos0, int n_tiles, int H, int Hkv, int dh,
                  int page_size, float scale, int window, int dtype, hipStream_t stream);
 
-// dn_attention with chunks, a bias by distance, a sink and kept first keys (ScoreExtras)
+// dn_attention with chunks, a bias by distance, a sink, kept first keys and a soft cap (ScoreExtras)
 int dn_attention_extras(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                         const int32_t* block_tables, int max_blocks, const int32_t* tile_seq, const int32_t* tile_row0,
                         const int32_t* tile_nrows, const int32_t* tile_pos0, int n_tiles, int H, int Hkv, int dh,
                         int page_size, float scale, int window, int chunk, const float* bias, int span, int sink,
-                        const float* sink_at, int keep, int dtype, hipStream_t stream);
+                        const float* sink_at, int keep, float cap, int dtype, hipStream_t stream);
 int dn_attention_rows_extras(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                              const int32_t* block_tables, int max_blocks, const int32_t* tile_seq, const int32_t* tile_pos0,
                              int n_tiles, float* part, int max_context, int H, int Hkv, int dh, int page_size, float scale,
-                             int window, int chunk, const float* bias, int span, int sink, const float* sink_at, int keep,
+                             int window, int chunk, const float* bias, int span, int sink, const float* sink_at, int keep, float cap,
                              int dtype, hipStream_t stream);
 
 // the same kernels' arithmetic for a step of single rows (tile s = request s = row s), every tile of keys a
@@ -61,12 +63,12 @@ int dn_attention_flash(const void* q, int ldq, void* out, int ldo, const void* k
                        const int32_t* tile_row0, const int32_t* tile_nrows, const int32_t* tile_pos0, int n_tiles,
                        int H, int Hkv, int dh, int page_size, float scale, int window, hipStream_t stream);
 
-// dn_attention_flash with chunks, a bias by distance, a sink and kept first keys (ScoreExtras); with any of them, pages of a power of two
+// dn_attention_flash with chunks, a bias by distance, a sink, kept first keys and a soft cap (ScoreExtras); with any of them, pages of a power of two
 int dn_attention_flash_extras(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                               const int32_t* block_tables, int max_blocks, const int32_t* tile_seq,
                               const int32_t* tile_row0, const int32_t* tile_nrows, const int32_t* tile_pos0, int n_tiles,
                               int H, int Hkv, int dh, int page_size, float scale, int window, int chunk, const float* bias,
-                              int span, int sink, const float* sink_at, int keep, hipStream_t stream);
+                              int span, int sink, const float* sink_at, int keep, float cap, hipStream_t stream);
 
 // bfloat16, one row per request (tile s = request s = row s); the tiles of 64 keys that a row reads are cut into n_splits runs
 // of `chunks` chunks of `waves` tiles; part: device memory for n_tiles * H * n_splits * (dh + 2) floats
@@ -80,12 +82,12 @@ int dn_attention_decode(const void* q, int ldq, void* out, int ldo, const void* 
                         int chunks, int waves, int H, int Hkv, int dh, int page_size, float scale, int window,
                         hipStream_t stream);
 
-// dn_attention_decode with chunks, a bias by distance, a sink and kept first keys (ScoreExtras); with any of them, pages of a power of two
+// dn_attention_decode with chunks, a bias by distance, a sink, kept first keys and a soft cap (ScoreExtras); with any of them, pages of a power of two
 int dn_attention_decode_extras(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                                const int32_t* block_tables, int max_blocks, const int32_t* tile_seq,
                                const int32_t* tile_row0, const int32_t* tile_pos0, int n_tiles, float* part, int n_splits,
                                int chunks, int waves, int H, int Hkv, int dh, int page_size, float scale, int window,
-                               int chunk, const float* bias, int span, int sink, const float* sink_at, int keep,
+                               int chunk, const float* bias, int span, int sink, const float* sink_at, int keep, float cap,
                                hipStream_t stream);
 
 // dn_attention_decode for callers that cannot allocate device memory (code under HIP graph capture,

@@ -11,8 +11,9 @@
 // What a layer may add to this (ScoreExtras): chunks (a row reads only the keys of its own run of `chunk` positions, runs
 // counted from the request's position 0), a bias by distance (bias[h][pos - key] is added to the scaled score; distances
 // from `span` on take the last entry), a sink (a key that every row sees, with a score per head, or 0, and no value: one more
-// summand, exp(score), under the softmax) and, with a window, the request's first `keep` keys, which every row reads as well
-// (their pages stay; those between them and the window are given back, and the kernels step over the gap).
+// summand, exp(score), under the softmax), with a window, the request's first `keep` keys, which every row reads as well
+// (their pages stay; those between them and the window are given back, and the kernels step over the gap), and a soft cap:
+// a scaled score s becomes cap * tanh(s / cap), before a bias is added.
 //
 // The key pool is [n_pages, Hkv, page_size, dh], the value pool [n_pages, Hkv, dh, page_size];
 // query head h reads key head h / (H / Hkv).
@@ -35,6 +36,13 @@ __device__ __forceinline__ bool reads_key(int key, int lo, int pos, int keep) { 
 
 // the score of the sink that head h sees (ex.sink set)
 __device__ __forceinline__ float sink_score(const ScoreExtras& ex, int h) { return ex.sink_at ? ex.sink_at[h] : 0.f; }
+
+// a scaled score as the soft cap leaves it (cap 0: none)
+__device__ __forceinline__ float soft_cap(float s, float cap) { return cap > 0.f ? cap * tanhf(s / cap) : s; }
+
+// 1 - 2 / (2^x + 1) = tanh(x / (2 log2(e))), by the hardware's exponential and reciprocal: what is lost is some 1e-7 of 1, which
+// times a cap is far below the rounding of a product of bfloat16 queries and keys
+__device__ __forceinline__ float tanh_of_exp2(float x) { return fmaf(-2.0f, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(x) + 1.0f), 1.0f); }
 
 // Keys are walked in tiles of `tile` from multiples of `tile`: those that hold the first `keep` keys, then those from the
 // window's first key `lo` on.  The walk starts at first(), goes from kt to next(kt), and ends where the caller's last key is
@@ -86,9 +94,15 @@ __device__ __forceinline__ float dim_sum(const float* ps, const float* vs, int d
   return a;
 }
 
+// a key's score from its product with the query
+__device__ __forceinline__ float score_of(float dot, float scale, float cap, const float* bias, int distance, int span) {
+  if (cap > 0.f) return soft_cap(dot * scale, cap) + (bias ? bias[min(distance, span - 1)] : 0.f);
+  return bias ? fmaf(dot, scale, bias[min(distance, span - 1)]) : dot * scale;
+}
+
 // the scores of one row against the tile in Ks: p[j] to Ps (this row's BK entries), -> m_T, l_T
 __device__ __forceinline__ void tile_scores(const float* qr, const float* Ks, float* ps, int g, int nc, int dh, int kt,
-                                            int lo, int pos, int keep, bool row_ok, float scale, const float* bias, int span,
+                                            int lo, int pos, int keep, bool row_ok, float scale, float cap, const float* bias, int span,
                                             float& m_t, float& l_t) {
   const float NEG_INF = -INFINITY;
   float s[4];
@@ -101,7 +115,7 @@ __device__ __forceinline__ void tile_scores(const float* qr, const float* Ks, fl
       const int key = kt + j;
       const float dot = key_dot(qr, Ks + j * (dh + 1), dh);
       const bool ok = row_ok && reads_key(key, lo, pos, keep);
-      s[c] = ok ? (bias ? fmaf(dot, scale, bias[min(pos - key, span - 1)]) : dot * scale) : NEG_INF;
+      s[c] = ok ? score_of(dot, scale, cap, bias, pos - key, span) : NEG_INF;
       tmax = fmaxf(tmax, s[c]);
     }
   }
@@ -265,7 +279,7 @@ __global__ __launch_bounds__(THREADS) void attention_kernel(
     __syncthreads();
     load_tile(Ks, Vs, Kb, Vb, k_pool, v_pool, bt, kt, last_pos, BK, dh, page_size, Hkv, hk, dhp + 1);
     float m_t, l_t, a_t[16];
-    tile_scores(Qs + qi * dhp, Ks, Ps + qi * BK, g, nc, dhp, kt, my_lo, my_pos, ex.keep, row_ok, scale, bias, ex.span, m_t,
+    tile_scores(Qs + qi * dhp, Ks, Ps + qi * BK, g, nc, dhp, kt, my_lo, my_pos, ex.keep, row_ok, scale, ex.cap, bias, ex.span, m_t,
                 l_t);
     __syncthreads();
     if (m_t > NEG_INF) {                // the same for the 16 threads of a row
@@ -325,7 +339,7 @@ __global__ __launch_bounds__(THREADS) void row_tiles_kernel(
     if (t < BK) {
       const int key = kt + t;
       const float dot = key_dot(Qs, Ks + t * (dh + 1), dh);
-      s = reads_key(key, lo, pos, ex.keep) ? (bias ? fmaf(dot, scale, bias[min(pos - key, ex.span - 1)]) : dot * scale) : NEG_INF;
+      s = reads_key(key, lo, pos, ex.keep) ? score_of(dot, scale, ex.cap, bias, pos - key, ex.span) : NEG_INF;
     }
     const float tmax = wave_max(s);
     if (t < BK) Ps[t] = s > NEG_INF ? expf(s - tmax) : 0.f;
@@ -428,7 +442,7 @@ __global__ __launch_bounds__(64) void row_tile64_kernel(
     dot = fmaf(a.w, b.w, dot);
   }
   const int key = kt + lane;
-  const float sc = reads_key(key, lo, pos, ex.keep) ? (bias ? fmaf(dot, scale, bias[min(pos - key, ex.span - 1)]) : dot * scale) : NEG_INF;
+  const float sc = reads_key(key, lo, pos, ex.keep) ? score_of(dot, scale, ex.cap, bias, pos - key, ex.span) : NEG_INF;
   const float tmax = wave_max(sc);
   Ps[lane] = sc > NEG_INF ? expf(sc - tmax) : 0.f;
   __syncthreads();
@@ -507,18 +521,18 @@ extern "C" int dn_attention(const void* q, int ldq, void* out, int ldo, const vo
                             int n_tiles, int H, int Hkv, int dh, int page_size, float scale, int window, int dtype,
                             hipStream_t stream) {
   return dn_attention_extras(q, ldq, out, ldo, k_pool, v_pool, block_tables, max_blocks, tile_seq, tile_row0, tile_nrows, tile_pos0,
-                             n_tiles, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, nullptr, 0, dtype, stream);
+                             n_tiles, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, nullptr, 0, 0.f, dtype, stream);
 }
 
 extern "C" int dn_attention_extras(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                                    const int32_t* block_tables, int max_blocks, const int32_t* tile_seq,
                                    const int32_t* tile_row0, const int32_t* tile_nrows, const int32_t* tile_pos0,
                                    int n_tiles, int H, int Hkv, int dh, int page_size, float scale, int window, int chunk,
-                                   const float* bias, int span, int sink, const float* sink_at, int keep, int dtype,
+                                   const float* bias, int span, int sink, const float* sink_at, int keep, float cap, int dtype,
                                    hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  if (chunk < 0 || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
-  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep};
+  if (chunk < 0 || !(cap >= 0.f) || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
+  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep, cap};
   // (any head size up to 256: one that is no multiple of 16 is padded to the next inside the kernel)
   if (dh < 1 || dh > 256 || Hkv < 1 || H % Hkv != 0 || page_size < 1 || max_blocks < 1) return DN_ERR_SHAPE;
   const int dhp = (dh + 15) / 16 * 16;
@@ -551,17 +565,17 @@ extern "C" int dn_attention_rows(const void* q, int ldq, void* out, int ldo, con
                                  const int32_t* tile_pos0, int n_tiles, float* part, int max_context, int H, int Hkv,
                                  int dh, int page_size, float scale, int window, int dtype, hipStream_t stream) {
   return dn_attention_rows_extras(q, ldq, out, ldo, k_pool, v_pool, block_tables, max_blocks, tile_seq, tile_pos0, n_tiles, part,
-                                  max_context, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, nullptr, 0, dtype, stream);
+                                  max_context, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, nullptr, 0, 0.f, dtype, stream);
 }
 
 extern "C" int dn_attention_rows_extras(const void* q, int ldq, void* out, int ldo, const void* k_pool, const void* v_pool,
                                         const int32_t* block_tables, int max_blocks, const int32_t* tile_seq,
                                         const int32_t* tile_pos0, int n_tiles, float* part, int max_context, int H, int Hkv,
                                         int dh, int page_size, float scale, int window, int chunk, const float* bias, int span,
-                                        int sink, const float* sink_at, int keep, int dtype, hipStream_t stream) {
+                                        int sink, const float* sink_at, int keep, float cap, int dtype, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  if (chunk < 0 || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
-  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep};
+  if (chunk < 0 || !(cap >= 0.f) || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
+  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep, cap};
   if (dh < 16 || dh > 256 || dh % 16 != 0 || Hkv < 1 || H % Hkv != 0 || page_size < 1 || max_blocks < 1 ||
       max_context < 1 || !part || n_tiles > 65535 || H > 65535)
     return DN_ERR_SHAPE;
@@ -644,8 +658,8 @@ typedef __attribute__((__vector_size__(4 * sizeof(uint32_t)))) uint32_t u32x4;
 // POW2: the page size is a power of two (page_size = 1 << page_shift), so that a key's page and its place in
 // the page are a shift and a mask: a tile's keys need four such pairs a step, and a division by a number
 // known only at run time is some twenty-five vector instructions.
-// EXTRAS: chunks, a bias by distance, a sink and kept first keys (ScoreExtras).  With a bias a score is the scaled product
-// plus the bias, both in units of log2(e), made before the maximum is taken (the largest product is no longer the largest score).
+// EXTRAS: chunks, a bias by distance, a sink, kept first keys and a soft cap (ScoreExtras).  With a bias or a cap a score is made
+// whole, in units of log2(e), before the maximum is taken (the largest product is no longer the largest score, or not its multiple).
 template <int DH16, int GROUPS, int TPS, bool POW2, bool EXTRAS = false>     // head size / 16; groups of 4 waves; tiles a wave takes per step
 __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH16 > 12 && GROUPS == 1 ? 1 : 2))) void kernel(
     const bf16_t* __restrict__ q, int ldq, bf16_t* __restrict__ out, int ldo, const bf16_t* __restrict__ k_pool,
@@ -699,7 +713,10 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
   const int keep = EXTRAS ? ex.keep : 0;
   const float NEG_INF = -INFINITY;
   const float scale2 = scale * 1.44269504088896340736f;    // log2(e)
-  const float per_score = EXTRAS && bias ? 1.0f : scale2;    // what is left to multiply a score with (a bias is added to scaled ones)
+  const bool made = EXTRAS && (bias || ex.cap > 0.f);         // (scores are made whole before the maximum)
+  const float cap2 = EXTRAS ? ex.cap * 1.44269504088896340736f : 0.f;
+  const float to_tanh = EXTRAS && ex.cap > 0.f ? 2.0f * scale2 / ex.cap : 0.f;
+  const float per_score = made ? 1.0f : scale2;    // what is left to multiply a score with
   const u32x4 zero4 = {0u, 0u, 0u, 0u};
 
   bf16x8 qf[DH16];
@@ -832,12 +849,13 @@ __global__ __launch_bounds__(256 * GROUPS) __attribute__((amdgpu_waves_per_eu(DH
         const int kw = kw0 + 32 * c;
         const bool edge = kw + 31 > pos0 + wrow0 || (kw < lo_last && kw + 31 >= keep);
         if (!act[c]) continue;
-        if (EXTRAS && bias) {
+        if (EXTRAS && made) {
 #pragma unroll
           for (int i = 0; i < 16; ++i) {
             const int key = kw + 8 * (i / 4) + 4 * g + (i % 4);
             const bool ok = reads_key(key, my_lo, my_pos, keep);
-            const float sc = fmaf(bias[min(max(my_pos - key, 0), ex.span - 1)], 1.44269504088896340736f, s[c][i] * scale2);
+            float sc = cap2 > 0.f ? cap2 * tanh_of_exp2(s[c][i] * to_tanh) : s[c][i] * scale2;
+            if (bias) sc = fmaf(bias[min(max(my_pos - key, 0), ex.span - 1)], 1.44269504088896340736f, sc);
             s[c][i] = (!edge || ok) ? sc : NEG_INF;
             tmax = fmaxf(tmax, s[c][i]);
           }
@@ -964,7 +982,7 @@ extern "C" int dn_attention_flash(const void* q, int ldq, void* out, int ldo, co
                                   int n_tiles, int H, int Hkv, int dh, int page_size, float scale, int window,
                                   hipStream_t stream) {
   return dn_attention_flash_extras(q, ldq, out, ldo, k_pool, v_pool, block_tables, max_blocks, tile_seq, tile_row0, tile_nrows,
-                                   tile_pos0, n_tiles, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, nullptr, 0, stream);
+                                   tile_pos0, n_tiles, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0, nullptr, 0, 0.f, stream);
 }
 
 // With any of ScoreExtras: pages of a power of two only.
@@ -972,11 +990,11 @@ extern "C" int dn_attention_flash_extras(const void* q, int ldq, void* out, int 
                                          const int32_t* block_tables, int max_blocks, const int32_t* tile_seq,
                                          const int32_t* tile_row0, const int32_t* tile_nrows, const int32_t* tile_pos0,
                                          int n_tiles, int H, int Hkv, int dh, int page_size, float scale, int window, int chunk,
-                                         const float* bias, int span, int sink, const float* sink_at, int keep, hipStream_t stream) {
+                                         const float* bias, int span, int sink, const float* sink_at, int keep, float cap, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  const bool extras = chunk > 0 || bias != nullptr || sink != 0 || keep > 0;
-  if (chunk < 0 || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
-  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep};
+  const bool extras = chunk > 0 || bias != nullptr || sink != 0 || keep > 0 || cap > 0.f;
+  if (chunk < 0 || !(cap >= 0.f) || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
+  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep, cap};
   // ldo == 0: out is a packed matrix of H * dh columns (a multiple of 32); the kernel takes the largest score
   // for the largest product of a query and a key, so the scale is positive
   if (!(scale > 0.f)) return DN_ERR_SHAPE;
@@ -1093,6 +1111,7 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
   const int lo = first_key(pos, window, EXTRAS ? ex.chunk : 0);
   const float* bias = EXTRAS && ex.bias ? ex.bias + static_cast<size_t>(h) * ex.span : nullptr;
   const int keep = EXTRAS ? ex.keep : 0;
+  const float to_tanh = EXTRAS && ex.cap > 0.f ? 2.0f * 1.44269504088896340736f / ex.cap : 0.f;
   // the tiles of 64 keys that the row reads, counted from 0: those of the kept first keys, then those from `lo` on
   const int kept_tiles = (keep + 63) / 64, rest = max(lo / 64, kept_tiles), last_tile = pos / 64;
   const int n_tiles_read = kept_tiles > last_tile ? last_tile + 1 : kept_tiles + (last_tile - rest + 1);
@@ -1161,6 +1180,7 @@ __global__ __launch_bounds__(WAVES * 64) void partial_kernel(const bf16_t* __res
 #pragma unroll
         for (int i = 0; i < 8; ++i) dot = fmaf(qr[i], static_cast<float>(kv[u][i]), dot);
         dot = group_reduce<LPK>(dot, SumOp());
+        if (EXTRAS && ex.cap > 0.f) dot = ex.cap * tanh_of_exp2(dot * to_tanh);
         if (EXTRAS && bias) dot += bias[min(max(pos - key, 0), ex.span - 1)];
         sc[it0 + u] = reads_key(key, lo, pos, keep) ? dot : NEG_INF;
       }
@@ -1269,7 +1289,7 @@ extern "C" int dn_attention_decode(const void* q, int ldq, void* out, int ldo, c
                                    float scale, int window, hipStream_t stream) {
   return dn_attention_decode_extras(q, ldq, out, ldo, k_pool, v_pool, block_tables, max_blocks, tile_seq, tile_row0, tile_pos0,
                                     n_tiles, part, n_splits, chunks, waves, H, Hkv, dh, page_size, scale, window, 0, nullptr, 0, 0,
-                                    nullptr, 0, stream);
+                                    nullptr, 0, 0.f, stream);
 }
 
 // With any of ScoreExtras: pages of a power of two only.
@@ -1278,11 +1298,11 @@ extern "C" int dn_attention_decode_extras(const void* q, int ldq, void* out, int
                                           const int32_t* tile_row0, const int32_t* tile_pos0, int n_tiles, float* part,
                                           int n_splits, int chunks, int waves, int H, int Hkv, int dh, int page_size,
                                           float scale, int window, int chunk, const float* bias, int span, int sink,
-                                          const float* sink_at, int keep, hipStream_t stream) {
+                                          const float* sink_at, int keep, float cap, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  const bool extras = chunk > 0 || bias != nullptr || sink != 0 || keep > 0;
-  if (chunk < 0 || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
-  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep};
+  const bool extras = chunk > 0 || bias != nullptr || sink != 0 || keep > 0 || cap > 0.f;
+  if (chunk < 0 || !(cap >= 0.f) || (bias && span < 1) || !keep_ok(keep, window, chunk)) return DN_ERR_SHAPE;
+  const ScoreExtras ex{chunk, bias, span, sink, sink_at, keep, cap};
   if (Hkv < 1 || H % Hkv != 0 || page_size % 16 != 0 || max_blocks < 1 || n_splits < 1 || chunks < 1 ||
       ldq % 8 != 0 || ldo < 0 || (ldo == 0 && (H * dh) % 32 != 0) || reinterpret_cast<uintptr_t>(q) % 16 != 0 || reinterpret_cast<uintptr_t>(k_pool) % 16 != 0 ||
       reinterpret_cast<uintptr_t>(v_pool) % 16 != 0)

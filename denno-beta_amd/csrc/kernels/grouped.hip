@@ -128,10 +128,10 @@ __global__ __launch_bounds__(64) void route_kernel(const float* z, size_t ldz, c
 // The same choice with a wave a row (up to 8,192 experts, `top` up to 64): lane l has the experts l, l + 64, ...; the
 // largest score is found over the lanes, the lowest index among equals wins, and lane c keeps the c-th choice.
 // groups > 1: the experts are `groups` equal runs of neighbours; a group's score is the sum of its two largest
-// s + correction (of its one, if it has one expert), and only the experts of the `keep` best groups (the lower index wins a
-// tie) can be chosen.  scale multiplies the weights.
+// s + correction (of its one, if it has one expert), or (by_best) its largest alone, and only the experts of the `keep` best
+// groups (the lower index wins a tie) can be chosen.  scale multiplies the weights.
 __global__ __launch_bounds__(64) void route_wave_kernel(const float* z, size_t ldz, const float* correction, int E, int top, int sigmoid,
-                                                        int renorm, int* ids, float* wts, int groups, int keep, float scale) {
+                                                        int renorm, int* ids, float* wts, int groups, int keep, int by_best, float scale) {
   const int t = blockIdx.x, lane = threadIdx.x;
   const float* row = z + static_cast<size_t>(t) * ldz;
   const float none = -__builtin_huge_valf();
@@ -154,7 +154,7 @@ __global__ __launch_bounds__(64) void route_wave_kernel(const float* z, size_t l
         if (v > first) second = first, first = v;
         else if (v > second) second = v;
       }
-      group_score[g] = per > 1 ? first + second : first;
+      group_score[g] = per > 1 && !by_best ? first + second : first;
       open_group[g] = 0;
     }
     __syncthreads();
@@ -203,7 +203,8 @@ __global__ __launch_bounds__(64) void route_wave_kernel(const float* z, size_t l
 
 // ---- the plan ------------------------------------------------------------------------------------------------
 // The n pairs (row, choice), pair i = row * top + choice, sorted by expert and inside an expert by i:
-// offsets[e] .. offsets[e + 1] - 1 are expert e's places in `order`.  One workgroup.
+// offsets[e] .. offsets[e + 1] - 1 are expert e's places in `order`.  A choice of E or more is none of the experts': its pair has
+// no place (`order` is then filled up to offsets[E] only).  One workgroup.
 __global__ __launch_bounds__(256) void plan_kernel(const int* ids, int n, int E, int* offsets, int* order) {
   extern __shared__ int shm[];
   int* base = shm;         // [E]
@@ -211,7 +212,8 @@ __global__ __launch_bounds__(256) void plan_kernel(const int* ids, int n, int E,
   const int tid = threadIdx.x;
   for (int e = tid; e < E; e += 256) base[e] = 0;
   __syncthreads();
-  for (int i = tid; i < n; i += 256) atomicAdd(&base[ids[i]], 1);
+  for (int i = tid; i < n; i += 256)
+    if (ids[i] < E) atomicAdd(&base[ids[i]], 1);
   __syncthreads();
   if (tid == 0) {
     int run = 0;
@@ -226,7 +228,7 @@ __global__ __launch_bounds__(256) void plan_kernel(const int* ids, int n, int E,
   __syncthreads();
   for (int c0 = 0; c0 < n; c0 += 256) {
     const int i = c0 + tid;
-    const int e = i < n ? ids[i] : -1;
+    const int id = i < n ? ids[i] : -1, e = id < E ? id : -1;
     cid[tid] = e;
     __syncthreads();
     if (e >= 0) {
@@ -250,7 +252,8 @@ __global__ __launch_bounds__(256) void plan_runs_kernel(const int* ids, int n, i
   const int L = (n + R - 1) / R, lo = min(tid * L, n), hi = min(lo + L, n);
   if (tid < R)
     for (int e = 0; e < E; ++e) cnt[tid * E + e] = 0;
-  for (int i = lo; i < hi; ++i) cnt[tid * E + ids[i]] += 1;
+  for (int i = lo; i < hi; ++i)
+    if (ids[i] < E) cnt[tid * E + ids[i]] += 1;
   __syncthreads();
   __shared__ int total[49];
   if (tid < E) {
@@ -275,6 +278,7 @@ __global__ __launch_bounds__(256) void plan_runs_kernel(const int* ids, int n, i
   __syncthreads();
   for (int i = lo; i < hi; ++i) {
     const int e = ids[i];
+    if (e >= E) continue;
     order[total[e] + cnt[tid * E + e]++] = i;
   }
 }
@@ -372,16 +376,18 @@ __global__ __launch_bounds__(256) void expert_down_kernel(const void* y, int y_d
 }
 
 // x[t, :] += sum_c wts[t, c] * out[t * top + c, :], the choices in their order (wts none: every weight is 1)
-// (logits: a weight is sigmoid of what wts holds; the weights of a row are then ldw numbers apart)
+// (logits: a weight is sigmoid of what wts holds; the weights of a row are then ldw numbers apart; ids: a choice of n_experts or
+// more gives h[t, :], the row that the experts read, in place of a row of `out`)
 __global__ __launch_bounds__(256) void combine_kernel(const float* out, const float* wts, size_t ldw, int logits, int top, int width,
-                                                      float* x, size_t ldx) {
+                                                      float* x, size_t ldx, const int* ids, int n_experts, const void* h, int h_dt, size_t ldh) {
   const int t = blockIdx.x;
   for (int c = threadIdx.x; c < width; c += 256) {
     float acc = 0.f;
     for (int q = 0; q < top; ++q) {
       float wq = wts ? wts[t * ldw + q] : 1.0f;
       if (logits) wq = 1.0f / (1.0f + expf(-wq));
-      acc = fmaf(wq, out[(static_cast<size_t>(t) * top + q) * width + c], acc);
+      const bool same = ids && ids[t * top + q] >= n_experts;
+      acc = fmaf(wq, same ? load_as(h, t * ldh + c, h_dt) : out[(static_cast<size_t>(t) * top + q) * width + c], acc);
     }
     x[t * ldx + c] += acc;
   }
@@ -731,13 +737,13 @@ int dn_heads_linear(const void* a, int a_dt, long long lda, int a_off, int a_str
 }
 
 int dn_moe_route(const float* z, long long ldz, const float* correction, int T, int E, int top, int sigmoid, int renorm, int* ids,
-                 float* wts, int groups, int keep, float scale, hipStream_t stream) {
+                 float* wts, int groups, int keep, int by_best, float scale, hipStream_t stream) {
   if (E < 1 || top < 1 || top > E || ldz < E) return DN_ERR_SHAPE;
   if (groups < 1 || E % groups != 0 || keep < 1 || keep > groups || top > keep * (E / groups)) return DN_ERR_SHAPE;
   if (T == 0) return 0;
   if (E <= 8192 && top <= 64) {
     hipLaunchKernelGGL(route_wave_kernel, dim3(T), dim3(64), 0, stream, z, static_cast<size_t>(ldz), correction, E, top, sigmoid, renorm,
-                       ids, wts, keep < groups ? groups : 1, keep, scale);
+                       ids, wts, keep < groups ? groups : 1, keep, by_best, scale);
     return dn_launch_status();
   }
   if (keep < groups || scale != 1.0f) return DN_ERR_SHAPE;      // (the kernel of a thread a row knows neither)
@@ -835,10 +841,11 @@ int dn_moe_down(const void* y, int y_dt, const int* order, const int* offsets, i
 }
 
 int dn_moe_combine(const float* out, const float* wts, long long ldw, int logits, int T, int top, int width, float* x, long long ldx,
-                   hipStream_t stream) {
+                   const int* ids, int n_experts, const void* h, int h_dt, long long ldh, hipStream_t stream) {
+  if (ids && (!h || !float_kind(h_dt))) return DN_ERR_DTYPE;
   if (T == 0) return 0;
   hipLaunchKernelGGL(combine_kernel, dim3(T), dim3(256), 0, stream, out, wts, static_cast<size_t>(ldw), logits, top, width, x,
-                     static_cast<size_t>(ldx));
+                     static_cast<size_t>(ldx), ids, n_experts, h, h_dt, static_cast<size_t>(ldh));
   return dn_launch_status();
 }
 

@@ -163,14 +163,40 @@ __global__ __launch_bounds__(256) void conv_rows_kernel(const float* h, size_t l
   }
 }
 
+// channel c of the convolution at a request's row i of this step (rows: its first; past: its history [taps - 1][width]).  Four
+// taps are asked for before the first is used; the sum runs over the taps in ascending order.
+__device__ __forceinline__ float conv_channel(const float* rows, size_t ldh, const float* past, int width, const float* w, int taps, int i, int c) {
+  float acc = 0.f;
+  for (int q0 = 0; q0 < taps; q0 += 4) {
+    float v[4], wq[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int q = min(q0 + u, taps - 1), src = i - taps + 1 + q;
+      v[u] = *(src >= 0 ? rows + static_cast<size_t>(src) * ldh + c : past + static_cast<size_t>(i + q) * width + c);
+      wq[u] = w[q];
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+      if (q0 + u < taps) acc = fmaf(wq[u], v[u], acc);
+  }
+  return acc;
+}
+
+// channel c of a history takes in one more row: the oldest goes
+__device__ __forceinline__ void history_move_on(float* past, int width, int taps, int c, float row) {
+  for (int m = 0; m + 1 < taps; ++m)
+    past[static_cast<size_t>(m) * width + c] = m + 2 < taps ? past[static_cast<size_t>(m + 1) * width + c] : row;
+}
+
 // The same convolution (without the row itself, then silu) over channels that are heads' vectors, a wave a vector, and for
 // the vectors of the first `n_unit` heads (of `unit_dim` channels each; the others have `rest_dim`) the vector is then
 // divided by sqrt(sum of its squares + eps) and multiplied by the head's scale: scale_a for the first n_a of them, scale_b
-// for the others.  Queries, keys and values of a recurrence leave one kernel as the recurrence reads them.
-__global__ __launch_bounds__(64) void conv_heads_kernel(const float* h, size_t ldh, const float* w, const float* hist, const int* row_start,
+// for the others.  Queries, keys and values of a recurrence leave one kernel as the recurrence reads them.  move_on (steps
+// in which every request has one row): the channel's history takes the row in, as history_update_kernel would do it next.
+__global__ __launch_bounds__(64) void conv_heads_kernel(const float* h, size_t ldh, const float* w, float* hist, const int* row_start,
                                                         const int* slots, int S, int width, int taps, int n_unit, int unit_dim, int n_a,
                                                         float scale_a, float scale_b, float eps, int rest_dim, float* out, size_t ldo,
-                                                        size_t hist_stride) {
+                                                        size_t hist_stride, int move_on) {
   const int t = blockIdx.x, vec = blockIdx.y, lane = threadIdx.x;
   const bool unit = vec < n_unit;
   const int dim = unit ? unit_dim : rest_dim;
@@ -182,17 +208,13 @@ __global__ __launch_bounds__(64) void conv_heads_kernel(const float* h, size_t l
     for (int j = lane; j < dim; j += 64) dst[j] = 0.f;
     return;
   }
-  const int i = t - row_start[s];
-  const float* past = hist + static_cast<size_t>(slot) * hist_stride;
+  const int row0 = row_start[s], i = t - row0;
+  float* past = hist + static_cast<size_t>(slot) * hist_stride;
   float ss = 0.f;
   for (int j = lane; j < dim; j += 64) {
     const int c = c0 + j;
-    float acc = 0.f;
-    for (int q = 0; q < taps; ++q) {
-      const int src = i - taps + 1 + q;
-      const float v = src >= 0 ? h[static_cast<size_t>(row_start[s] + src) * ldh + c] : past[static_cast<size_t>(i + q) * width + c];
-      acc = fmaf(w[c * taps + q], v, acc);
-    }
+    float acc = conv_channel(h + static_cast<size_t>(row0) * ldh, ldh, past, width, w + static_cast<size_t>(c) * taps, taps, i, c);
+    if (move_on) history_move_on(past, width, taps, c, h[static_cast<size_t>(t) * ldh + c]);
     acc = acc / (1.0f + expf(-acc));
     ss = fmaf(acc, acc, ss);
     dst[j] = acc;
@@ -246,11 +268,11 @@ __global__ __launch_bounds__(256) void shift_mix_kernel(const void* h, int h_dt,
 // ---- pairs of dimensions turned by the position ------------------------------------------------------------
 // Vector n of row t starts at src_off + n * src_stride; its entries 2i and 2i + 1 (i < dims / 2) are turned by the
 // angle position * freq[i] (cos and sin times `mag`: a scaled encoding's factor, 1 otherwise), the other `width - dims`
-// entries pass; the result goes to dst_off + n * dst_stride.
+// entries pass; the result goes to dst_off + n * dst_stride.  halves: the pairs are entries i and i + dims / 2 instead.
 __global__ __launch_bounds__(256) void rotary_kernel(const void* src, int src_dt, size_t ld_src, int src_off, int src_stride,
                                                      void* dst, int dst_dt, size_t ld_dst, int dst_off, int dst_stride,
                                                      const int* positions, const float* freq, int n_vec, int dims, int width,
-                                                     float mag) {
+                                                     float mag, int halves) {
   const int t = blockIdx.x;
   const float p = static_cast<float>(positions[t]);
   const int half = dims / 2, rest = width - dims;
@@ -262,9 +284,10 @@ __global__ __launch_bounds__(256) void rotary_kernel(const void* src, int src_dt
     if (i < half) {
       const float ang = p * freq[i];
       const float c = cosf(ang) * mag, sn = sinf(ang) * mag;
-      const float u = load_as(src, a + 2 * i, src_dt), v = load_as(src, a + 2 * i + 1, src_dt);
-      store_as(dst, b + 2 * i, dst_dt, u * c - v * sn);
-      store_as(dst, b + 2 * i + 1, dst_dt, v * c + u * sn);
+      const int lo = halves ? i : 2 * i, hi = halves ? i + half : 2 * i + 1;
+      const float u = load_as(src, a + lo, src_dt), v = load_as(src, a + hi, src_dt);
+      store_as(dst, b + lo, dst_dt, u * c - v * sn);
+      store_as(dst, b + hi, dst_dt, v * c + u * sn);
     } else {
       const int k = dims + (i - half);
       store_as(dst, b + k, dst_dt, load_as(src, a + k, src_dt));
@@ -548,6 +571,29 @@ __global__ __launch_bounds__(256) void gated_kernel(const void* x, int x_dt, siz
     store_as(out, t * ldo + c, out_dt, load_as(x, t * ldx + c, x_dt) * activation(kind, g[t * ldg + c], 0.f));
 }
 
+// out[t, c] = g sigmoid(alpha g) (u + 1) with g = min(z[t, c], limit) and u = z[t, n + c] between -limit and limit: both halves of
+// a row of one product.  VEC: four columns a thread (rows at multiples of 16 bytes, n a multiple of 4).
+__device__ __forceinline__ float clamped_gate(float g, float u, float limit, float alpha) {
+  g = fminf(g, limit), u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+}
+
+template <bool VEC>
+__global__ __launch_bounds__(256) void clamped_glu_kernel(const float* z, size_t ldz, float limit, float alpha, void* out, int out_dt,
+                                                          size_t ldo, int n) {
+  const size_t t = blockIdx.x;
+  if constexpr (VEC) {
+    for (int c = (blockIdx.y * 256 + threadIdx.x) * 4; c < n; c += gridDim.y * 1024) {
+      const f32x4 g = *reinterpret_cast<const f32x4*>(z + t * ldz + c), u = *reinterpret_cast<const f32x4*>(z + t * ldz + n + c);
+#pragma unroll
+      for (int k = 0; k < 4; ++k) store_as(out, t * ldo + c + k, out_dt, clamped_gate(g[k], u[k], limit, alpha));
+    }
+  } else {
+    for (int c = blockIdx.y * 256 + threadIdx.x; c < n; c += gridDim.y * 256)
+      store_as(out, t * ldo + c, out_dt, clamped_gate(z[t * ldz + c], z[t * ldz + n + c], limit, alpha));
+  }
+}
+
 // ---- the scan ----------------------------------------------------------------------------------------------
 // Per request, head and 16 (or 4) value columns one wave keeps the head's state S [dk][those columns] in registers and
 // walks the request's rows of this step in order:
@@ -556,7 +602,8 @@ __global__ __launch_bounds__(256) void gated_kernel(const void* x, int x_dt, siz
 //   delta:        S_i <- w_i S_i ;  e_j = beta (v_j - sum_i a_i S_i) ;  S_i <- S_i + a_i e_j ;  o_j = sum_i r_i S_i
 //   else:         o_j = sum_i r_i (S_i + u_i a_i v_j) ;  S_i <- w_i S_i + a_i v_j
 // w is a number per row, head and key channel, or (w_rows) one per row and head for all the head's channels, or (w_head) one
-// per head for all rows and channels.  r and k may have
+// per head for all rows and channels.  The delta rule with w_rows is a mode of its own: the row's decay stays a single number,
+// and may be given as z, the decay being exp(-w_rate[h] log(1 + e^(z + w_bias[h]))).  r and k may have
 // fewer heads than v: head h reads r and k of head h / (H / G).
 // A column's key channels are shared out among KG lanes that lie side by side (4 lanes for heads of up to 32 key
 // channels, 16 beyond), so a wave has 64 / KG columns and a column's parts are joined inside a row of 16 lanes,
@@ -565,10 +612,10 @@ __global__ __launch_bounds__(256) void gated_kernel(const void* x, int x_dt, siz
 // A row's r, k and w reach the lanes through LDS, some rows at a time (16, or 2 in a step of single rows); the next are asked for before the
 // current ones are worked on.  Places beyond a request's last row hold r = 0, a = 0, w = 1, which change nothing, so the
 // rows of a fetch are worked on without a branch between them.
-enum { SCAN_BEFORE = 0, SCAN_AFTER = 1, SCAN_DELTA = 2 };
+enum { SCAN_BEFORE = 0, SCAN_AFTER = 1, SCAN_DELTA = 2, SCAN_DELTA_ROWS = 3 };
 
 struct ScanArgs {
-  const float *r, *k, *v, *w, *u, *beta, *w_head;
+  const float *r, *k, *v, *w, *u, *beta, *w_head, *w_rate, *w_bias;
   size_t ldr, ldk, ldv, ldw, ldb;
   int G;
   float* state;
@@ -581,17 +628,19 @@ struct ScanArgs {
 
 template <int DK, int KG, int MODE, bool VEC, int TB>
 __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
-  constexpr bool AFTER = MODE == SCAN_AFTER, DELTA = MODE == SCAN_DELTA;
+  constexpr bool AFTER = MODE == SCAN_AFTER, DELTA = MODE == SCAN_DELTA || MODE == SCAN_DELTA_ROWS;
+  constexpr bool ROWS = MODE == SCAN_DELTA_ROWS;      // (a row's decay is one number: it takes no place beside r and k)
+  constexpr int PARTS = ROWS ? 2 : 3;
   constexpr int KQ = DK / KG;
   constexpr int CW = 64 / KG;      // value columns of a wave
   constexpr int NL = DK >= 64 ? DK / 64 : 1;
   // TB: rows asked for at a time (a trip to memory is paid once per TB rows, not per row; all TB places are worked on,
   // so steps of single rows take a small TB).  A row's sums are the same for every TB.
   constexpr int N4 = TB * DK / 4, NV = N4 >= 64 ? N4 / 64 : 1;      // VEC: groups of four numbers per array, per lane
-  __shared__ __attribute__((aligned(16))) float sh[TB][3 * DK];
+  __shared__ __attribute__((aligned(16))) float sh[TB][PARTS * DK];
   __shared__ __attribute__((aligned(16))) float shv[TB][CW];
   __shared__ __attribute__((aligned(16))) float shu[DK];
-  __shared__ float shb[TB];
+  __shared__ float shb[TB], shw[TB];
   const int s = blockIdx.z, h = blockIdx.y, lane = threadIdx.x;
   const int hq = h / (a.H / a.G);                     // the head of r and k that this head reads
   const float wh = a.w_head ? a.w_head[h] : 1.0f;     // one decay for the head, where w is none
@@ -611,9 +660,10 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
   // what a fetch brings: (not VEC) a lane's own numbers row by row; (VEC: every size a multiple of 4 and every row at a
   // multiple of 16 bytes) 16 bytes a lane and load, eight rows of r, k or w in DK / 32 loads: a row then costs a wave
   // 7 / 8 of a vector load where it cost four, and those loads, not the arithmetic, were what a row waited for
-  float nr[VEC ? 1 : TB][NL], nk[VEC ? 1 : TB][NL], nw[VEC ? 1 : TB][NL], nv[VEC ? 1 : TB], nb[VEC ? 1 : TB];
+  float nr[VEC ? 1 : TB][NL], nk[VEC ? 1 : TB][NL], nw[VEC ? 1 : TB][NL], nv[VEC ? 1 : TB], nb[VEC ? 1 : TB], nd[VEC ? 1 : TB];
   f32x4 r4[VEC ? NV : 1], k4[VEC ? NV : 1], w4[VEC ? NV : 1], v4;
   auto beta_of = [&](float z) { return a.beta_logits ? 1.0f / (1.0f + expf(-z)) : z; };      // (beta given as it is, or as sigmoid's argument)
+  auto decay_of = [&](float z) { return a.w_rate ? expf(-a.w_rate[h] * softplus_f(z + (a.w_bias ? a.w_bias[h] : 0.f))) : z; };
   auto fetch = [&](int t0) {
     if constexpr (VEC) {
       const f32x4 zero = {0.f, 0.f, 0.f, 0.f}, one = {1.f, 1.f, 1.f, 1.f};
@@ -623,9 +673,10 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
         const bool ok = idx < N4 && t < row1 && i < dk;
         r4[it] = ok ? *reinterpret_cast<const f32x4*>(a.r + t * a.ldr + hq * dk + i) : zero;
         k4[it] = (ok && !a.key_from_decay) ? *reinterpret_cast<const f32x4*>(a.k + t * a.ldk + hq * dk + i) : zero;
-        w4[it] = !ok ? one : a.w_head ? one * wh : a.w_rows ? one * a.w[t * a.ldw + h] : *reinterpret_cast<const f32x4*>(a.w + t * a.ldw + h * dk + i);
+        if constexpr (!ROWS) w4[it] = !ok ? one : a.w_head ? one * wh : a.w_rows ? one * a.w[t * a.ldw + h] : *reinterpret_cast<const f32x4*>(a.w + t * a.ldw + h * dk + i);
       }
       if constexpr (DELTA) nb[0] = (lane < TB && t0 + lane < row1) ? beta_of(a.beta[(t0 + lane) * a.ldb + h]) : 0.f;
+      if constexpr (ROWS) nd[0] = (lane < TB && t0 + lane < row1) ? decay_of(a.w[(t0 + lane) * a.ldw + h]) : 1.f;
       const int bq = lane / (CW / 4), col = j0 + (lane % (CW / 4)) * 4, t = t0 + bq;
       v4 = (lane < TB * CW / 4 && t < row1 && col < dv) ? *reinterpret_cast<const f32x4*>(a.v + t * a.ldv + h * dv + col) : zero;
     } else {
@@ -639,19 +690,23 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
           const bool ok = row && i < dk;
           nr[bq][q] = ok ? a.r[t * a.ldr + hq * dk + i] : 0.f;
           nk[bq][q] = (ok && !a.key_from_decay) ? a.k[t * a.ldk + hq * dk + i] : 0.f;
-          nw[bq][q] = !ok ? 1.f : a.w_head ? wh : a.w_rows ? a.w[t * a.ldw + h] : a.w[t * a.ldw + h * dk + i];
+          if constexpr (!ROWS) nw[bq][q] = !ok ? 1.f : a.w_head ? wh : a.w_rows ? a.w[t * a.ldw + h] : a.w[t * a.ldw + h * dk + i];
         }
         if constexpr (DELTA) nb[bq] = row ? beta_of(a.beta[t * a.ldb + h]) : 0.f;
+        if constexpr (ROWS) nd[bq] = row ? decay_of(a.w[t * a.ldw + h]) : 1.f;
         nv[bq] = (row && live) ? a.v[t * a.ldv + h * dv + j] : 0.f;
       }
     }
   };
   fetch(row0);
   for (int t0 = row0; t0 < row1; t0 += TB) {
-    float vj[TB], bj[TB];
+    float vj[TB], bj[TB], dj[TB];
     if constexpr (VEC) {
       if constexpr (DELTA) {
         if (lane < TB) shb[lane] = nb[0];
+      }
+      if constexpr (ROWS) {
+        if (lane < TB) shw[lane] = nd[0];
       }
 #pragma unroll
       for (int it = 0; it < NV; ++it) {
@@ -659,8 +714,8 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
         if (idx < N4) {
           const f32x4 one = {1.f, 1.f, 1.f, 1.f};
           *reinterpret_cast<f32x4*>(&sh[bq][i]) = r4[it];
-          *reinterpret_cast<f32x4*>(&sh[bq][DK + i]) = a.key_from_decay ? one - w4[it] : k4[it];
-          *reinterpret_cast<f32x4*>(&sh[bq][2 * DK + i]) = w4[it];
+          *reinterpret_cast<f32x4*>(&sh[bq][DK + i]) = !ROWS && a.key_from_decay ? one - w4[it] : k4[it];
+          if constexpr (!ROWS) *reinterpret_cast<f32x4*>(&sh[bq][2 * DK + i]) = w4[it];
         }
       }
       if (lane < TB * CW / 4) *reinterpret_cast<f32x4*>(&shv[lane / (CW / 4)][(lane % (CW / 4)) * 4]) = v4;
@@ -672,12 +727,13 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
           const int i = lane + 64 * q;
           if (i < DK) {
             sh[bq][i] = nr[bq][q];
-            sh[bq][DK + i] = a.key_from_decay ? 1.0f - nw[bq][q] : nk[bq][q];
-            sh[bq][2 * DK + i] = nw[bq][q];
+            sh[bq][DK + i] = !ROWS && a.key_from_decay ? 1.0f - nw[bq][q] : nk[bq][q];
+            if constexpr (!ROWS) sh[bq][2 * DK + i] = nw[bq][q];
           }
         }
         vj[bq] = nv[bq];
         if constexpr (DELTA) bj[bq] = nb[bq];
+        if constexpr (ROWS) dj[bq] = nd[bq];
       }
     }
     __syncthreads();
@@ -686,6 +742,7 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
       for (int bq = 0; bq < TB; ++bq) {
         vj[bq] = shv[bq][lane / KG];
         if constexpr (DELTA) bj[bq] = shb[bq];
+        if constexpr (ROWS) dj[bq] = shw[bq];
       }
     }
     if (t0 + TB < row1) fetch(t0 + TB);
@@ -703,7 +760,7 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
         float ans = 0.f;
 #pragma unroll
         for (int q = 0; q < KQ; ++q) {
-          S[q] *= mw[q];
+          S[q] *= ROWS ? dj[bq] : mw[q];
           ans = fmaf(mk[q], S[q], ans);
         }
         ans = group_reduce<KG>(ans, SumOp());
@@ -1248,7 +1305,7 @@ __global__ __launch_bounds__(256) void norm_pair_write_held_kernel(const float* 
 // A row of z is [q: H x dk | k: G x dk | v: G x dv].  Each query and key is divided by its root mean square (eps inside the
 // root; eps < 0: it is not) and weighed entry by entry (wq, wk: dk numbers shared by the heads), then its first `dims` entries are turned in
 // neighbouring pairs by position * freq; a value's first v_dims entries are turned by position * v_freq.  A query times
-// q_scale[head] goes to q_out (heads `kept` columns wide), keys and values to the cache's pools (heads `kept` wide, the row's
+// q_scale[head] and times 1 + pos_coef ln(floor((position + 1) / pos_every) + 1) goes to q_out (heads `kept` columns wide), keys and values to the cache's pools (heads `kept` wide, the row's
 // place from slot_map; a negative place: nothing is written); columns a vector does not have are zeros.  LPV lanes (a wave, or half
 // of one) share a vector: a lane holds the pairs lane, lane + LPV, .. (J of them), the squares are summed over them in one order.
 struct NormTurnArgs {
@@ -1256,6 +1313,8 @@ struct NormTurnArgs {
   size_t ldz;
   int H, G, dk, dv;
   const float *wq, *wk, *q_scale;      // (each may be none)
+  float pos_coef;      // (0: no temperature by position)
+  double pos_every;
   float eps;
   const float* freq;
   int dims;
@@ -1289,6 +1348,9 @@ __global__ __launch_bounds__(256) void norm_turn_write_kernel(NormTurnArgs a) {
   const int lane = threadIdx.x % LPV;
   const int half = a.dims / 2, v_half = a.v_dims / 2, n_vec = a.H + 2 * a.G;
   const float p = static_cast<float>(a.positions[t]);
+  // (the quotient in 64-bit: an exact multiple gives its whole number, and nothing below one reaches it)
+  const float warm = a.pos_coef == 0.f ? 1.0f
+                                       : fmaf(a.pos_coef, logf(static_cast<float>(floor((a.positions[t] + 1.0) / a.pos_every)) + 1.0f), 1.0f);
   if (threadIdx.x < half + v_half) {
     const float ang = p * (threadIdx.x < half ? a.freq[threadIdx.x] : a.v_freq[threadIdx.x - half]);
     sincosf(ang, &sn[threadIdx.x], &cs[threadIdx.x]);
@@ -1315,7 +1377,7 @@ __global__ __launch_bounds__(256) void norm_turn_write_kernel(NormTurnArgs a) {
       ss = fmaf(hi[j], hi[j], ss);
     }
     const float inv = is_v || a.eps < 0.f ? 1.0f : 1.0f / sqrtf(group_reduce<LPV>(ss, SumOp()) / static_cast<float>(width) + a.eps);
-    const float times = is_q && a.q_scale ? a.q_scale[n] : 1.0f;
+    const float times = is_q ? (a.q_scale ? a.q_scale[n] : 1.0f) * warm : 1.0f;
 #pragma unroll
     for (int j = 0; j < J; ++j) {
       const int i = lane + LPV * j, e = 2 * i;
@@ -1344,6 +1406,100 @@ __global__ __launch_bounds__(256) void norm_turn_write_kernel(NormTurnArgs a) {
         } else {
           store_pair(a.k_pool, head + static_cast<size_t>(off) * a.kept + e, a.dt, x, y);
         }
+      }
+    }
+  }
+}
+
+// ---- the same behind a short convolution, with norms over all heads at once -------------------------------------------
+// A row of z is [q: H x dk | k: G x dk | v: G x dv].  Every channel passes a short causal convolution over time (no activation; w
+// [channels][taps], the last tap the row's own; rows before the step's from the history); q and k are each divided by their
+// root mean square as one vector over all heads and weighed entry by entry (wq: H x dk numbers, wk: G x dk); the first `dims`
+// entries of every head's q and k are turned by position * freq in pairs (i, i + dims / 2); then to their places as
+// norm_turn_write_kernel puts them.  move_on as in conv_heads_kernel.  One workgroup a row, the row in LDS; how many threads it
+// has follows from the sizes alone, so a row's sums do not depend on the step.
+struct ConvTurnArgs {
+  const float* z;
+  size_t ldz;
+  int H, G, dk, dv, taps;
+  const float* w;
+  float* hist;
+  size_t hist_stride;
+  const int *row_start, *slots;
+  int S;
+  const float *wq, *wk;
+  float eps;
+  const float* freq;
+  int dims;
+  const int* positions;
+  void* q_out;
+  size_t ldq;
+  int kept;
+  const int* slot_map;
+  void *k_pool, *v_pool;
+  int page_size, dt, write, move_on;
+};
+
+template <int THREADS>
+__global__ __launch_bounds__(THREADS) void conv_turn_write_kernel(ConvTurnArgs a) {
+  extern __shared__ float vals[];      // [channels]
+  __shared__ float cs[128], sn[128], sums[2][THREADS / 64];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const int qw = a.H * a.dk, kw = a.G * a.dk, C = qw + kw + a.G * a.dv, half = a.dims / 2, pairs = a.kept / 2;
+  const int s = request_of(a.row_start, a.S, t);
+  const int slot = a.slots[s], row0 = a.row_start[s];
+  if (slot < 0 || t >= a.row_start[a.S]) {      // a padding row: zeros, so that what follows works on numbers
+    for (int i = tid; i < a.H * pairs; i += THREADS) store_pair(a.q_out, t * a.ldq + 2 * i, a.dt, 0.f, 0.f);
+    return;
+  }
+  const int place = a.slot_map[t];
+  if (tid < half) {
+    const float ang = static_cast<float>(a.positions[t]) * a.freq[tid];
+    sincosf(ang, &sn[tid], &cs[tid]);
+  }
+  float* past = a.hist + static_cast<size_t>(slot) * a.hist_stride;
+  float sq = 0.f, sk = 0.f;
+  for (int c = tid; c < C; c += THREADS) {
+    const float v = conv_channel(a.z + static_cast<size_t>(row0) * a.ldz, a.ldz, past, C, a.w + static_cast<size_t>(c) * a.taps, a.taps, t - row0, c);
+    if (a.move_on) history_move_on(past, C, a.taps, c, a.z[static_cast<size_t>(t) * a.ldz + c]);
+    if (c < qw) sq = fmaf(v, v, sq);
+    else if (c < qw + kw) sk = fmaf(v, v, sk);
+    vals[c] = v;
+  }
+  sq = wave_sum(sq), sk = wave_sum(sk);
+  if ((tid & 63) == 0) sums[0][tid >> 6] = sq, sums[1][tid >> 6] = sk;
+  __syncthreads();
+  sq = sk = 0.f;
+#pragma unroll
+  for (int u = 0; u < THREADS / 64; ++u) sq += sums[0][u], sk += sums[1][u];
+  const float iq = 1.0f / sqrtf(sq / static_cast<float>(qw) + a.eps), ik = 1.0f / sqrtf(sk / static_cast<float>(kw) + a.eps);
+  for (int c = tid; c < qw + kw; c += THREADS) vals[c] *= c < qw ? iq * a.wq[c] : ik * a.wk[c - qw];      // (the thread's own)
+  __syncthreads();
+  const bool writes = a.write && place >= 0;
+  const int page = writes ? place / a.page_size : 0, off = writes ? place % a.page_size : 0;
+  const int n = (writes ? a.H + 2 * a.G : a.H) * pairs;
+  for (int i = tid; i < n; i += THREADS) {
+    const int vec = i / pairs, e = 2 * (i % pairs);
+    const bool is_v = vec >= a.H + a.G;
+    const int width = is_v ? a.dv : a.dk;
+    const float* x = vals + (is_v ? qw + kw + (vec - a.H - a.G) * a.dv : vec * a.dk);
+    float out[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const int d = e + u;
+      float y = d < width ? x[d] : 0.f;
+      if (!is_v && d < 2 * half) y = d < half ? y * cs[d] - x[d + half] * sn[d] : y * cs[d - half] + x[d - half] * sn[d - half];
+      out[u] = y;
+    }
+    if (vec < a.H) {
+      store_pair(a.q_out, t * a.ldq + static_cast<size_t>(vec) * a.kept + e, a.dt, out[0], out[1]);
+    } else {
+      const size_t head = (static_cast<size_t>(page) * a.G + (vec - a.H) % a.G) * a.page_size * a.kept;
+      if (is_v) {
+        store_as(a.v_pool, head + static_cast<size_t>(e) * a.page_size + off, a.dt, out[0]);
+        store_as(a.v_pool, head + static_cast<size_t>(e + 1) * a.page_size + off, a.dt, out[1]);
+      } else {
+        store_pair(a.k_pool, head + static_cast<size_t>(off) * a.kept + e, a.dt, out[0], out[1]);
       }
     }
   }
@@ -1671,6 +1827,162 @@ __global__ __launch_bounds__(256) void streams_write_held_kernel(float* xs, size
   }
 }
 
+// ---- a norm behind the sum of the stream and a sublayer's result -------------------------------------------------------
+// x[t] <- (u - mean(u)) / sqrt(mean((u - mean(u))^2) + eps) * g + b with u = alpha x[t] + r, r being the sublayer's result:
+//   y[t];
+//   y2 given: the mean of two branches, each divided by its root mean square over the width and weighed first, (y / rms(y) * by +
+//     y2 / rms(y2) * by2) / 2;
+//   top > 0: a weighted sum of the choices of a router, sum_c weigh[t, c] * (ids[t, c] < n_rows ? y[t * top + c] : x[t]), c
+//     ascending: a choice beyond the experts gives the row that they read back (its row of y is not read).
+// out: the same rows for whoever reads the stream next, in its own precision (or none).  One workgroup a row; the sums as in
+// rmsnorm_kernel.  Up to 256 NC columns a thread holds its share of the row; NC 0: the row goes to x and comes back.
+struct PostNormArgs {
+  float* x;
+  size_t ldx;
+  float alpha;
+  const float* y;
+  size_t ldy;
+  const float* y2;
+  size_t ldy2;
+  const float *by, *by2;
+  float beps;
+  const float* weigh;
+  const int* ids;
+  int top, n_rows;
+  const float *g, *b;
+  float eps;
+  void* out;
+  int out_dt;
+  size_t ldo;
+  int width;
+};
+
+template <int NC>
+__global__ __launch_bounds__(256) void post_norm_kernel(PostNormArgs a) {
+  __shared__ float sh[2][4];
+  const size_t row = blockIdx.x;
+  const int tid = threadIdx.x, wave = tid >> 6;
+  float x[NC], y[NC], g[NC], b[NC];
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = min(tid + 256 * k, a.width - 1);
+    x[k] = a.x[row * a.ldx + c];
+    g[k] = a.g[c];
+    b[k] = a.b ? a.b[c] : 0.f;
+    y[k] = a.top > 0 ? 0.f : a.y[row * a.ldy + c];
+  }
+  if (a.top > 0) {
+    for (int q0 = 0; q0 < a.top; q0 += 4) {
+      // (four choices' rows are asked for before the first is added)
+      float v[4][NC], wq[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int q = min(q0 + u, a.top - 1);
+        const size_t at = row * a.top + q;
+        const bool expert = a.ids[at] < a.n_rows;
+        const float* src = expert ? a.y + at * a.ldy : a.x + row * a.ldx;
+        wq[u] = q0 + u < a.top ? a.weigh[at] : 0.f;
+#pragma unroll
+        for (int k = 0; k < NC; ++k) v[u][k] = src[min(tid + 256 * k, a.width - 1)];
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+        if (q0 + u < a.top) {
+#pragma unroll
+          for (int k = 0; k < NC; ++k) y[k] = fmaf(wq[u], v[u][k], y[k]);
+        }
+    }
+  }
+  if (a.y2) {
+    float y2[NC], s1 = 0.f, s2 = 0.f;
+#pragma unroll
+    for (int k = 0; k < NC; ++k) y2[k] = a.y2[row * a.ldy2 + min(tid + 256 * k, a.width - 1)];
+#pragma unroll
+    for (int k = 0; k < NC; ++k)
+      if (tid + 256 * k < a.width) s1 = fmaf(y[k], y[k], s1), s2 = fmaf(y2[k], y2[k], s2);
+    s1 = wave_sum(s1), s2 = wave_sum(s2);
+    if ((tid & 63) == 0) sh[0][wave] = s1, sh[1][wave] = s2;
+    __syncthreads();
+    s1 = (sh[0][0] + sh[0][1]) + (sh[0][2] + sh[0][3]), s2 = (sh[1][0] + sh[1][1]) + (sh[1][2] + sh[1][3]);
+    const float i1 = 0.5f / sqrtf(s1 / static_cast<float>(a.width) + a.beps), i2 = 0.5f / sqrtf(s2 / static_cast<float>(a.width) + a.beps);
+#pragma unroll
+    for (int k = 0; k < NC; ++k) {
+      const int c = min(tid + 256 * k, a.width - 1);
+      y[k] = fmaf(y2[k] * i2, a.by2[c], y[k] * i1 * a.by[c]);
+    }
+  }
+  float s = 0.f;
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    x[k] = fmaf(a.alpha, x[k], y[k]);
+    if (tid + 256 * k < a.width) s += x[k];
+  }
+  const float mean = block_sum_256(s, sh[0]) / static_cast<float>(a.width);
+  s = 0.f;
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    x[k] -= mean;
+    if (tid + 256 * k < a.width) s = fmaf(x[k], x[k], s);
+  }
+  const float inv = 1.0f / sqrtf(block_sum_256(s, sh[0]) / static_cast<float>(a.width) + a.eps);
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = tid + 256 * k;
+    if (c < a.width) {
+      const float v = fmaf(x[k] * inv, g[k], b[k]);
+      a.x[row * a.ldx + c] = v;
+      if (a.out) store_as(a.out, row * a.ldo + c, a.out_dt, v);
+    }
+  }
+}
+
+// (rows of any width: what the thread owns goes to x and comes back)
+template <>
+__global__ __launch_bounds__(256) void post_norm_kernel<0>(PostNormArgs a) {
+  __shared__ float sh[4];
+  const size_t row = blockIdx.x;
+  float* xr = a.x + row * a.ldx;
+  float i1 = 0.f, i2 = 0.f;
+  if (a.y2) {
+    float s1 = 0.f, s2 = 0.f;
+    for (int c = threadIdx.x; c < a.width; c += 256) {
+      const float u = a.y[row * a.ldy + c], v = a.y2[row * a.ldy2 + c];
+      s1 = fmaf(u, u, s1), s2 = fmaf(v, v, s2);
+    }
+    i1 = 0.5f / sqrtf(block_sum_256(s1, sh) / static_cast<float>(a.width) + a.beps);
+    i2 = 0.5f / sqrtf(block_sum_256(s2, sh) / static_cast<float>(a.width) + a.beps);
+  }
+  float s = 0.f;
+  for (int c = threadIdx.x; c < a.width; c += 256) {
+    const float old = xr[c];
+    float y = 0.f;
+    if (a.top > 0) {
+      for (int q = 0; q < a.top; ++q) {
+        const size_t at = row * a.top + q;
+        y = fmaf(a.weigh[at], a.ids[at] < a.n_rows ? a.y[at * a.ldy + c] : old, y);
+      }
+    } else {
+      y = a.y[row * a.ldy + c];
+      if (a.y2) y = fmaf(a.y2[row * a.ldy2 + c] * i2, a.by2[c], y * i1 * a.by[c]);
+    }
+    const float u = fmaf(a.alpha, old, y);
+    xr[c] = u;
+    s += u;
+  }
+  const float mean = block_sum_256(s, sh) / static_cast<float>(a.width);
+  s = 0.f;
+  for (int c = threadIdx.x; c < a.width; c += 256) {
+    const float d = xr[c] - mean;
+    s = fmaf(d, d, s);
+  }
+  const float inv = 1.0f / sqrtf(block_sum_256(s, sh) / static_cast<float>(a.width) + a.eps);
+  for (int c = threadIdx.x; c < a.width; c += 256) {
+    const float v = fmaf((xr[c] - mean) * inv, a.g[c], a.b ? a.b[c] : 0.f);
+    xr[c] = v;
+    if (a.out) store_as(a.out, row * a.ldo + c, a.out_dt, v);
+  }
+}
+
 bool float_kind(int dt) { return dt == DN_F32 || dt == DN_BF16; }
 
 }  // namespace
@@ -1739,16 +2051,17 @@ int dn_conv_rows(const float* h, long long ldh, const float* w, const float* bia
   return dn_launch_status();
 }
 
-int dn_conv_heads(const float* h, long long ldh, const float* w, const float* hist, const int* row_start, const int* slots, int S, int T,
+int dn_conv_heads(const float* h, long long ldh, const float* w, float* hist, const int* row_start, const int* slots, int S, int T,
                   int taps, int n_unit, int unit_dim, int n_a, float scale_a, float scale_b, float eps, int n_rest, int rest_dim,
-                  float* out, long long ldo, long long hist_stride, hipStream_t stream) {
+                  float* out, long long ldo, long long hist_stride, int move_on, hipStream_t stream) {
   const long long width = static_cast<long long>(n_unit) * unit_dim + static_cast<long long>(n_rest) * rest_dim;
-  if (taps < 1 || S < 1 || n_unit < 0 || n_rest < 0 || n_unit + n_rest < 1 || ldh < width || ldo < width || n_a < 0 || n_a > n_unit)
+  if (taps < 1 || S < 1 || n_unit < 0 || n_rest < 0 || n_unit + n_rest < 1 || ldh < width || ldo < width || n_a < 0 || n_a > n_unit ||
+      (move_on && T != S))
     return DN_ERR_SHAPE;
   if (T == 0) return 0;
   hipLaunchKernelGGL(conv_heads_kernel, dim3(T, n_unit + n_rest), dim3(64), 0, stream, h, static_cast<size_t>(ldh), w, hist, row_start,
                      slots, S, static_cast<int>(width), taps, n_unit, unit_dim, n_a, scale_a, scale_b, eps, rest_dim, out,
-                     static_cast<size_t>(ldo), static_cast<size_t>(hist_stride));
+                     static_cast<size_t>(ldo), static_cast<size_t>(hist_stride), move_on && taps > 1);
   return dn_launch_status();
 }
 
@@ -1802,12 +2115,12 @@ int dn_shift_mix(const void* h, int h_dt, const float* hist, const float* mu, in
 
 int dn_rotary(const void* src, int src_dt, long long ld_src, int src_off, int src_stride, void* dst, int dst_dt, long long ld_dst,
               int dst_off, int dst_stride, const int* positions, const float* freq, int T, int n_vec, int dims, int width, float mag,
-              hipStream_t stream) {
+              int halves, hipStream_t stream) {
   if (!float_kind(src_dt) || !float_kind(dst_dt)) return DN_ERR_DTYPE;
   if (dims % 2 != 0 || dims > width || dims < 0) return DN_ERR_SHAPE;
   if (T == 0 || n_vec == 0) return 0;
   hipLaunchKernelGGL(rotary_kernel, dim3(T), dim3(256), 0, stream, src, src_dt, static_cast<size_t>(ld_src), src_off, src_stride, dst,
-                     dst_dt, static_cast<size_t>(ld_dst), dst_off, dst_stride, positions, freq, n_vec, dims, width, mag);
+                     dst_dt, static_cast<size_t>(ld_dst), dst_off, dst_stride, positions, freq, n_vec, dims, width, mag, halves);
   return dn_launch_status();
 }
 
@@ -1834,14 +2147,16 @@ int dn_gated(const void* x, int x_dt, long long ldx, const float* g, long long l
 int dn_state_scan(const float* r, long long ldr, const float* k, long long ldk, const float* v, long long ldv, const float* w,
                   long long ldw, const float* u, const float* beta, long long ldb, const float* w_head, int G, float* state,
                   long long slot_stride, const int* row_start, const int* slots, int S, int T, int H, int dk, int dv, int mode,
-                  int key_from_decay, int beta_logits, int w_rows, float* out, long long ldo, hipStream_t stream) {
+                  int key_from_decay, int beta_logits, int w_rows, const float* w_rate, const float* w_bias, float* out, long long ldo,
+                  hipStream_t stream) {
   if (dk < 1 || dk > 256 || dv < 1 || H < 1 || G < 1 || H % G != 0) return DN_ERR_SHAPE;
   if ((!key_from_decay && k == nullptr) || (w_rows && (w == nullptr || key_from_decay))) return DN_ERR_SHAPE;
   if (mode < SCAN_BEFORE || mode > SCAN_DELTA || (mode == SCAN_DELTA && beta == nullptr) || (w == nullptr) == (w_head == nullptr))
     return DN_ERR_SHAPE;
+  if (w_rate && !(mode == SCAN_DELTA && w_rows)) return DN_ERR_SHAPE;
   if (S == 0) return 0;
   const int read_after = mode;
-  ScanArgs a{r, k, v, w, u, beta, w_head, static_cast<size_t>(ldr), static_cast<size_t>(ldk), static_cast<size_t>(ldv),
+  ScanArgs a{r, k, v, w, u, beta, w_head, w_rate, w_bias, static_cast<size_t>(ldr), static_cast<size_t>(ldk), static_cast<size_t>(ldv),
              static_cast<size_t>(ldw), static_cast<size_t>(ldb), G, state, static_cast<size_t>(slot_stride), row_start, slots, H, dk, dv, read_after, key_from_decay, beta_logits, w_rows, out,
              static_cast<size_t>(ldo)};
   // (the parts of a column's sum by the head's size alone, never by the step: a row's bits are the same in every step)
@@ -1862,7 +2177,8 @@ int dn_state_scan(const float* r, long long ldr, const float* k, long long ldk, 
   } while (0)
 #define DN_SCAN(DK, KG, GRID)                                     \
   do {                                                            \
-    if (mode == SCAN_DELTA) DN_SCAN2(DK, KG, GRID, SCAN_DELTA);   \
+    if (mode == SCAN_DELTA && w_rows) DN_SCAN2(DK, KG, GRID, SCAN_DELTA_ROWS); \
+    else if (mode == SCAN_DELTA) DN_SCAN2(DK, KG, GRID, SCAN_DELTA);   \
     else if (mode == SCAN_AFTER) DN_SCAN2(DK, KG, GRID, SCAN_AFTER); \
     else DN_SCAN2(DK, KG, GRID, SCAN_BEFORE);                     \
   } while (0)
@@ -1986,7 +2302,7 @@ int dn_norm_pair_write(const float* z, long long ldz, int qw, int kw, const floa
 }
 
 int dn_norm_turn_write(const float* z, long long ldz, int H, int G, int dk, int dv, const float* wq, const float* wk, const float* q_scale,
-                       float eps, const float* freq, int dims, const float* v_freq, int v_dims, const int* positions, void* q_out,
+                       float pos_coef, double pos_every, float eps, const float* freq, int dims, const float* v_freq, int v_dims, const int* positions, void* q_out,
                        long long ldq, int kept, const int* slot_map, void* k_pool, void* v_pool, int T, int page_size, int dt, int write,
                        hipStream_t stream) {
   if (!float_kind(dt)) return DN_ERR_DTYPE;
@@ -1996,7 +2312,8 @@ int dn_norm_turn_write(const float* z, long long ldz, int H, int G, int dk, int 
       reinterpret_cast<uintptr_t>(q_out) % 8 != 0 || reinterpret_cast<uintptr_t>(k_pool) % 8 != 0)
     return DN_ERR_SHAPE;
   if (T == 0) return 0;
-  const NormTurnArgs a{z, static_cast<size_t>(ldz), H, G, dk, dv, wq, wk, q_scale, eps, freq, dims, v_freq, v_dims, positions, q_out,
+  if (pos_coef != 0.f && !(pos_every > 0.0)) return DN_ERR_SHAPE;
+  const NormTurnArgs a{z, static_cast<size_t>(ldz), H, G, dk, dv, wq, wk, q_scale, pos_coef, pos_every, eps, freq, dims, v_freq, v_dims, positions, q_out,
                        static_cast<size_t>(ldq), kept, slot_map, k_pool, v_pool, page_size, dt, write};
   // (few rows: the vectors of a row spread over workgroups, so that a step of decoded tokens is more than a handful of them; many
   // rows: one workgroup a row, whose angles are made once.  By the sizes alone a vector has 32 or 64 lanes: the same bits either way)
@@ -2005,6 +2322,60 @@ int dn_norm_turn_write(const float* z, long long ldz, int H, int G, int dk, int 
   if (kept <= 64) hipLaunchKernelGGL((norm_turn_write_kernel<32, 1>), grid, dim3(256), 0, stream, a);
   else if (kept <= 128) hipLaunchKernelGGL((norm_turn_write_kernel<64, 1>), grid, dim3(256), 0, stream, a);
   else hipLaunchKernelGGL((norm_turn_write_kernel<64, 2>), grid, dim3(256), 0, stream, a);
+  return dn_launch_status();
+}
+
+int dn_conv_turn_write(const float* z, long long ldz, int H, int G, int dk, int dv, const float* w, int taps, float* hist,
+                       long long hist_stride, const int* row_start, const int* slots, int S, const float* wq, const float* wk, float eps,
+                       const float* freq, int dims, const int* positions, void* q_out, long long ldq, int kept, const int* slot_map,
+                       void* k_pool, void* v_pool, int T, int page_size, int dt, int write, int move_on, hipStream_t stream) {
+  if (!float_kind(dt)) return DN_ERR_DTYPE;
+  const long long C = static_cast<long long>(H + G) * dk + static_cast<long long>(G) * dv;
+  if (H < 1 || G < 1 || dk < 1 || dv < 1 || taps < 1 || (taps > 1 && !hist) || kept > 256 || kept % 2 != 0 || dk > kept || dv > kept || dims < 0 ||
+      dims % 2 != 0 || dims > dk || (dims > 0 && !freq) || !wq || !wk || page_size < 1 || S < 1 || ldz < C || C > 15000 ||
+      ldq < static_cast<long long>(H) * kept || ldq % 2 != 0 || (move_on && T != S) || reinterpret_cast<uintptr_t>(q_out) % 8 != 0 ||
+      reinterpret_cast<uintptr_t>(k_pool) % 8 != 0)
+    return DN_ERR_SHAPE;
+  if (T == 0) return 0;
+  const ConvTurnArgs a{z, static_cast<size_t>(ldz), H, G, dk, dv, taps, w, hist, static_cast<size_t>(hist_stride), row_start, slots, S, wq, wk,
+                       eps, freq, dims, positions, q_out, static_cast<size_t>(ldq), kept, slot_map, k_pool, v_pool, page_size, dt, write,
+                       move_on && taps > 1};
+  const size_t lds = static_cast<size_t>(C) * sizeof(float);
+  if (C <= 1024) hipLaunchKernelGGL(conv_turn_write_kernel<256>, dim3(T), dim3(256), lds, stream, a);
+  else hipLaunchKernelGGL(conv_turn_write_kernel<1024>, dim3(T), dim3(1024), lds, stream, a);
+  return dn_launch_status();
+}
+
+int dn_clamped_glu(const float* z, long long ldz, float limit, float alpha, void* out, int out_dt, long long ldo, int T, int n,
+                   hipStream_t stream) {
+  if (!float_kind(out_dt)) return DN_ERR_DTYPE;
+  if (n < 1 || ldz < 2LL * n || ldo < n) return DN_ERR_SHAPE;
+  if (T == 0) return 0;
+  const bool vec = n % 4 == 0 && ldz % 4 == 0 && reinterpret_cast<uintptr_t>(z) % 16 == 0;
+  const dim3 grid(T, T <= 256 ? (n + 1023) / 1024 : 1);
+  if (vec) hipLaunchKernelGGL(clamped_glu_kernel<true>, grid, dim3(256), 0, stream, z, static_cast<size_t>(ldz), limit, alpha, out, out_dt,
+                              static_cast<size_t>(ldo), n);
+  else hipLaunchKernelGGL(clamped_glu_kernel<false>, grid, dim3(256), 0, stream, z, static_cast<size_t>(ldz), limit, alpha, out, out_dt,
+                          static_cast<size_t>(ldo), n);
+  return dn_launch_status();
+}
+
+int dn_post_norm(float* x, long long ldx, float alpha, const float* y, long long ldy, const float* y2, long long ldy2, const float* by,
+                 const float* by2, float beps, const float* weigh, const int* ids, int top, int n_rows, const float* g, const float* b,
+                 float eps, void* out, int out_dt, long long ldo, int T, int width, hipStream_t stream) {
+  if (out && !float_kind(out_dt)) return DN_ERR_DTYPE;
+  if (width < 1 || ldx < width || ldy < width || !g || (y2 && (!by || !by2 || ldy2 < width)) || top < 0 ||
+      (top > 0 && (!weigh || !ids || y2 || n_rows < 0)) || (out && ldo < width))
+    return DN_ERR_SHAPE;
+  if (T == 0) return 0;
+  const PostNormArgs a{x, static_cast<size_t>(ldx), alpha, y, static_cast<size_t>(ldy), y2, static_cast<size_t>(ldy2), by, by2, beps, weigh,
+                       ids, top, n_rows, g, b, eps, out, out_dt, static_cast<size_t>(ldo), width};
+  // (by the width alone, so that a row's sums do not depend on the step)
+  if (width <= 512) hipLaunchKernelGGL(post_norm_kernel<2>, dim3(T), dim3(256), 0, stream, a);
+  else if (width <= 1024) hipLaunchKernelGGL(post_norm_kernel<4>, dim3(T), dim3(256), 0, stream, a);
+  else if (width <= 2048) hipLaunchKernelGGL(post_norm_kernel<8>, dim3(T), dim3(256), 0, stream, a);
+  else if (width <= 4096) hipLaunchKernelGGL(post_norm_kernel<16>, dim3(T), dim3(256), 0, stream, a);
+  else hipLaunchKernelGGL(post_norm_kernel<0>, dim3(T), dim3(256), 0, stream, a);
   return dn_launch_status();
 }
 

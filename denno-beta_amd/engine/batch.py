@@ -54,6 +54,7 @@ class StepContext:
     host_first_pos: List[int] = field(default_factory=list)
     host_slots: List[int] = field(default_factory=list)
     rids: List[int] = field(default_factory=list)
+    single_rows: bool = False      # every request brings one row (a pure decode step)
 
 
 class BatchError(ValueError):
@@ -161,4 +162,4 @@ def build_context(entries: Sequence[StepEntry], cache, vocab: int, max_positions
     return StepContext(
         T=T, S=S, R=R, tokens=view("tokens"), positions=view("positions"), logit_rows=view("logit_rows"),
         state_slots=view("state_slots"), row_start=view("row_start"), groups=groups,
-        host_row_start=row_start, host_first_pos=starts, host_slots=slots, rids=[e.rid for e in entries])
+        host_row_start=row_start, host_first_pos=starts, host_slots=slots, rids=[e.rid for e in entries], single_rows=single)

@@ -69,7 +69,7 @@ class DecodeGraph:
         self.ctx = StepContext(T=B, S=B, R=B, tokens=v("tokens"), positions=v("positions"),
                                logit_rows=v("logit_rows"), state_slots=v("state_slots"), row_start=v("row_start"),
                                groups=groups, host_row_start=list(range(B + 1)), host_first_pos=[0] * B,
-                               host_slots=[-1] * B, rids=[-1] * B)
+                               host_slots=[-1] * B, rids=[-1] * B, single_rows=True)
         none = np.empty(0, dtype=np.int32)
         self._fill(self.host[0].numpy(), np.empty(0, dtype=np.int64), none, none, none)
         self.dev.copy_(self.host[0])

@@ -7,7 +7,7 @@ implementation behind these names: without a GPU or without the built library th
 from __future__ import annotations
 
 import ctypes
-from ctypes import c_float, c_int, c_longlong, c_void_p
+from ctypes import c_double, c_float, c_int, c_longlong, c_void_p
 
 import torch
 
@@ -120,10 +120,10 @@ def _declare(name, lib):
             "dn_attention": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P],
             "dn_attention_rows": [P, I, P, I, P, P, P, I, P, P, I, P, I, I, I, I, I, F, I, I, P],
             "dn_attention_rows_tile": [I],
-            "dn_attention_extras": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P, I, I, P, I, I, P],
-            "dn_attention_rows_extras": [P, I, P, I, P, P, P, I, P, P, I, P, I, I, I, I, I, F, I, I, P, I, I, P, I, I, P],
-            "dn_attention_flash_extras": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P, I, I, P, I, P],
-            "dn_attention_decode_extras": [P, I, P, I, P, P, P, I, P, P, P, I, P, I, I, I, I, I, I, I, F, I, I, P, I, I, P, I, P],
+            "dn_attention_extras": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P, I, I, P, I, F, I, P],
+            "dn_attention_rows_extras": [P, I, P, I, P, P, P, I, P, P, I, P, I, I, I, I, I, F, I, I, P, I, I, P, I, F, I, P],
+            "dn_attention_flash_extras": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P, I, I, P, I, F, P],
+            "dn_attention_decode_extras": [P, I, P, I, P, P, P, I, P, P, P, I, P, I, I, I, I, I, I, I, F, I, I, P, I, I, P, I, F, P],
             "dn_attention_flash": [P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, P],
             "dn_attention_decode": [P, I, P, I, P, P, P, I, P, P, P, I, P, I, I, I, I, I, I, I, F, I, P],
         },
@@ -135,21 +135,24 @@ def _declare(name, lib):
             "dn_unit_heads": [P, c_longlong, P, c_longlong, I, I, I, F, F, P],
             "dn_conv_rows": [P, c_longlong, P, P, P, P, P, I, I, I, I, I, I, P, I, c_longlong, c_longlong, P],
             "dn_history_update": [P, I, c_longlong, P, P, P, I, I, I, c_longlong, P],
-            "dn_conv_heads": [P, c_longlong, P, P, P, P, I, I, I, I, I, I, F, F, F, I, I, P, c_longlong, c_longlong, P],
+            "dn_conv_heads": [P, c_longlong, P, P, P, P, I, I, I, I, I, I, F, F, F, I, I, P, c_longlong, c_longlong, I, P],
             "dn_rotary_runs": [P, I, c_longlong, P, I, P, P, I, F, c_longlong, F, P],
             "dn_shift_mix": [P, I, P, P, I, P, P, I, I, I, P, I, c_longlong, P],
-            "dn_rotary": [P, I, c_longlong, I, I, P, I, c_longlong, I, I, P, P, I, I, I, I, F, P],
+            "dn_rotary": [P, I, c_longlong, I, I, P, I, c_longlong, I, I, P, P, I, I, I, I, F, I, P],
             "dn_activate": [P, c_longlong, P, P, I, P, I, c_longlong, I, I, P],
             "dn_gated": [P, I, c_longlong, P, c_longlong, I, P, I, c_longlong, I, I, P],
             "dn_state_scan": [P, c_longlong, P, c_longlong, P, c_longlong, P, c_longlong, P, P, c_longlong, P, I, P, c_longlong, P, P,
-                              I, I, I, I, I, I, I, I, I, P, c_longlong, P],
+                              I, I, I, I, I, I, I, I, I, P, P, P, c_longlong, P],
             "dn_head_norm": [P, c_longlong, P, I, F, P, c_longlong, I, I, P, c_longlong, P, I, P, I, c_longlong, I, I, I, P],
             "dn_step_sizes": [P, c_longlong, P, P, P, c_longlong, I, I, I, P, c_longlong, P, c_longlong, P],
             "dn_gate_scan": [P, c_longlong, P, c_longlong, P, c_longlong, P, P, P, c_longlong, P, P, I, I, I, P, I, c_longlong, P],
             "dn_streams_read": [P, c_longlong, I, P, P, F, P, I, c_longlong, P, I, I, P],
             "dn_streams_write": [P, c_longlong, I, P, P, P, c_longlong, P, c_longlong, P, P, F, P, I, P, P, F, P, I, c_longlong, I, I, P],
             "dn_norm_pair_write": [P, c_longlong, I, I, P, P, F, P, c_longlong, P, P, P, I, I, I, I, I, I, I, P],
-            "dn_norm_turn_write": [P, c_longlong, I, I, I, I, P, P, P, F, P, I, P, I, P, P, c_longlong, I, P, P, P, I, I, I, I, P],
+            "dn_norm_turn_write": [P, c_longlong, I, I, I, I, P, P, P, F, c_double, F, P, I, P, I, P, P, c_longlong, I, P, P, P, I, I, I, I, P],
+            "dn_conv_turn_write": [P, c_longlong, I, I, I, I, P, I, P, c_longlong, P, P, I, P, P, F, P, I, P, P, c_longlong, I, P, P, P, I, I, I, I, I, P],
+            "dn_clamped_glu": [P, c_longlong, F, F, P, I, c_longlong, I, I, P],
+            "dn_post_norm": [P, c_longlong, F, P, c_longlong, P, c_longlong, P, P, F, P, P, I, I, P, P, F, P, I, c_longlong, I, I, P],
             "dn_turn_back_gate": [P, I, c_longlong, I, P, c_longlong, P, P, P, I, c_longlong, I, I, I, P],
             "dn_poly_norm": [P, c_longlong, P, F, P, I, c_longlong, I, I, P],
             "dn_head_gate": [P, I, c_longlong, I, P, c_longlong, P, I, c_longlong, I, I, I, P],
@@ -160,11 +163,11 @@ def _declare(name, lib):
         },
         "grouped": {
             "dn_heads_linear": [P, I, c_longlong, I, I, P, I, P, I, c_longlong, I, I, I, I, I, I, P],
-            "dn_moe_route": [P, c_longlong, P, I, I, I, I, I, P, P, I, I, F, P],
+            "dn_moe_route": [P, c_longlong, P, I, I, I, I, I, P, P, I, I, I, F, P],
             "dn_moe_plan": [P, I, I, P, P, P],
             "dn_moe_up": [P, I, c_longlong, P, P, I, I, I, P, P, I, I, I, F, F, I, P, P, I, I, P],
             "dn_moe_down": [P, I, P, P, I, I, P, I, I, I, P, I, P],
-            "dn_moe_combine": [P, P, c_longlong, I, I, I, I, P, c_longlong, P],
+            "dn_moe_combine": [P, P, c_longlong, I, I, I, I, P, c_longlong, P, I, P, I, c_longlong, P],
         },
         "sampling": {
             "dn_sample": [P, I, I, I, P, P, P, P],
@@ -630,7 +633,7 @@ def attention_writes_packed(dtype, page_size, head_dim, single_rows, max_context
 
 
 def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, window=0, tiles_wide=None,
-              single_rows=False, max_context=0, decode_waves=None, chunk=0, bias=None, sink=False, keep_first=0):
+              single_rows=False, max_context=0, decode_waves=None, chunk=0, bias=None, sink=False, keep_first=0, softcap=0.0):
     """Causal attention of the batch's rows over the paged cache.
 
     q: [T, >= H*dh] rows contiguous, head h at columns h*dh..; out: [T, H*dh];
@@ -645,7 +648,7 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
     the request's first); bias: 32-bit [H, span], bias[h, p - key] is added to the scaled score (distances from span on
     take the last entry); sink: True: one more summand exp(0) under the softmax (a key with score 0 and no value), or 32-bit [H]:
     head h's summand is exp(sink[h]), which nothing scales; keep_first: with a window, the request's first so many keys are
-    read by every row as well.
+    read by every row as well; softcap > 0: a scaled score s becomes softcap * tanh(s / softcap), before the bias.
 
     Three kernels: 32-bit takes the plain one; bfloat16 takes the MFMA kernel over tiles_wide, or,
     for a pure decode step, the split kernel (with both, out may be packed rows); a head size that
@@ -673,7 +676,8 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
     _f32vec(sink_at, "sink", n_heads)
     keep_first = int(keep_first) if window > 0 else 0      # (without a window every key is read anyway)
     _need(keep_first >= 0 and not (keep_first and chunk), "attention: kept first keys go with a window and not with chunks")
-    extras = chunk > 0 or bias is not None or sink or keep_first > 0
+    _need(softcap >= 0, "attention: softcap")
+    extras = chunk > 0 or bias is not None or sink or keep_first > 0 or softcap > 0
     span = 0
     if bias is not None:
         _dev(bias, "bias", (torch.float32,), 2)
@@ -682,7 +686,7 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
     _need(chunk >= 0, "attention: chunk")
     lib = _lib("attention")
     # (the kernel for portions takes the largest score for the largest product: a scale that is not positive goes the plain way)
-    # (with chunks, a bias, a sink or kept first keys the two bfloat16 kernels take pages of a power of two)
+    # (with chunks, a bias, a sink, kept first keys or a soft cap the two bfloat16 kernels take pages of a power of two)
     fast = (q.dtype == torch.bfloat16 and ps % 16 == 0 and ldq % 8 == 0 and q.data_ptr() % 16 == 0 and scale > 0
             and (not extras or ps & (ps - 1) == 0))
     decode = fast and decode_attention_applies(q.dtype, ps, dh, single_rows, max_context)
@@ -725,7 +729,7 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
             q.data_ptr(), ldq, out.data_ptr(), ldo, k_pool.data_ptr(), v_pool.data_ptr(), block_tables.data_ptr(),
             block_tables.shape[1], base, base + 4 * n_tiles, base + 12 * n_tiles, n_tiles, part.data_ptr(), n_splits,
             chunks, waves, n_heads, Hkv, dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(sink),
-            _ptr(sink_at), keep_first, _stream()), "attention (decode)")
+            _ptr(sink_at), keep_first, float(softcap), _stream()), "attention (decode)")
         return out
     if fast and tiles_wide is not None and dh in FLASH_HEAD_DIMS:
         _dev(tiles_wide, "tiles_wide", _I32, 2)
@@ -736,7 +740,7 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
             q.data_ptr(), ldq, out.data_ptr(), ldo, k_pool.data_ptr(), v_pool.data_ptr(), block_tables.data_ptr(),
             block_tables.shape[1], base, base + 4 * n_tiles, base + 8 * n_tiles, base + 12 * n_tiles, n_tiles,
             n_heads, Hkv, dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(sink), _ptr(sink_at),
-            keep_first, _stream()), "attention (flash)")
+            keep_first, float(softcap), _stream()), "attention (flash)")
         return out
     n_tiles = tiles.shape[1]
     base = tiles.data_ptr()
@@ -750,14 +754,14 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
         _ok(lib.dn_attention_rows_extras(
             q.data_ptr(), ldq, out.data_ptr(), ldo, k_pool.data_ptr(), v_pool.data_ptr(), block_tables.data_ptr(),
             block_tables.shape[1], base, base + 12 * n_tiles, n_tiles, part.data_ptr(), int(max_context), n_heads, Hkv,
-            dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(sink), _ptr(sink_at), keep_first, _CODE[q.dtype],
-            _stream()), "attention (single rows)")
+            dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(sink), _ptr(sink_at), keep_first, float(softcap),
+            _CODE[q.dtype], _stream()), "attention (single rows)")
         return out
     _ok(lib.dn_attention_extras(
         q.data_ptr(), ldq, out.data_ptr(), ldo, k_pool.data_ptr(), v_pool.data_ptr(), block_tables.data_ptr(),
         block_tables.shape[1], base, base + 4 * n_tiles, base + 8 * n_tiles, base + 12 * n_tiles, n_tiles,
         n_heads, Hkv, dh, ps, float(scale), int(window), int(chunk), _ptr(bias), span, int(sink), _ptr(sink_at), keep_first,
-        _CODE[q.dtype], _stream()), "attention")
+        float(softcap), _CODE[q.dtype], _stream()), "attention")
     return out
 
 
@@ -1122,21 +1126,22 @@ def history_update(h, hist, row_start, slots):
                                            slots.data_ptr(), S, width, keep, stride, _stream()), "history_update")
 
 
-def conv_heads(h, w, hist, row_start, slots, out, n_unit, unit_dim, n_first, scale_first, scale_rest, eps, n_rest, rest_dim):
+def conv_heads(h, w, hist, row_start, slots, out, n_unit, unit_dim, n_first, scale_first, scale_rest, eps, n_rest, rest_dim,
+               move_on=False):
     """conv_rows(identity=False, act="silu") over channels that are heads' vectors, and the first n_unit vectors (unit_dim
     channels each; n_rest more of rest_dim follow) made unit vectors on the way out: x / sqrt(sum(x^2) + eps), times
     scale_first for the first n_first of them and scale_rest for the others.  h: 32-bit rows whose first columns are the
-    channels; out: 32-bit [T, channels]."""
+    channels; out: 32-bit [T, channels].  move_on: history_update in the same launch, for steps in which every request has one row."""
     _dev(h, "h", (torch.float32,), 2), _dev(w, "w", (torch.float32,), 2), _dev(out, "out", (torch.float32,), 2)
     T = h.shape[0]
     width, taps = w.shape
     S = _request_tables(row_start, slots, "conv_heads")
     _need(width == n_unit * unit_dim + n_rest * rest_dim and h.shape[1] >= width and w.is_contiguous() and tuple(out.shape) == (T, width)
-          and 0 <= n_first <= n_unit and n_unit + n_rest >= 1 and n_unit + n_rest <= 65535, "conv_heads: shapes")
+          and 0 <= n_first <= n_unit and n_unit + n_rest >= 1 and n_unit + n_rest <= 65535 and not (move_on and T != S), "conv_heads: shapes")
     stride = _history(hist, (taps - 1) * width, "conv_heads") if taps > 1 else 0
     _ok(_lib("sequence").dn_conv_heads(h.data_ptr(), _rows(h, "h"), w.data_ptr(), _ptr(hist) if taps > 1 else 0, row_start.data_ptr(),
                                        slots.data_ptr(), S, T, taps, n_unit, unit_dim, n_first, float(scale_first), float(scale_rest),
-                                       float(eps), n_rest, rest_dim, out.data_ptr(), _rows(out, "out"), stride, _stream()), "conv_heads")
+                                       float(eps), n_rest, rest_dim, out.data_ptr(), _rows(out, "out"), stride, int(bool(move_on)), _stream()), "conv_heads")
     return out
 
 
@@ -1184,10 +1189,11 @@ def shift_mix(h, hist, mu, row_start, slots, out):
     return out
 
 
-def rotary(src, dst, positions, freq, n_vec, dims, width, src_off=0, src_stride=None, dst_off=0, dst_stride=None, mag=1.0):
+def rotary(src, dst, positions, freq, n_vec, dims, width, src_off=0, src_stride=None, dst_off=0, dst_stride=None, mag=1.0,
+           halves=False):
     """Vector n (n < n_vec) of row t, `width` wide, starts at column src_off + n * src_stride of src; of its first `dims`
     entries, 2i and 2i + 1 are turned by positions[t] * freq[i] (32-bit angles; cos and sin times `mag`), the rest pass; it
-    goes to column dst_off + n * dst_stride of dst (which may be src)."""
+    goes to column dst_off + n * dst_stride of dst (which may be src).  halves: the pairs are entries i and i + dims / 2."""
     _dev(src, "src", _FLOATS, 2), _dev(dst, "dst", _FLOATS, 2), _dev(positions, "positions", _I32, 1)
     T = src.shape[0]
     src_stride = width if src_stride is None else src_stride
@@ -1200,7 +1206,7 @@ def rotary(src, dst, positions, freq, n_vec, dims, width, src_off=0, src_stride=
               and dst_off >= 0 and dst_off + (n_vec - 1) * dst_stride + width <= dst.shape[1], "rotary: vectors outside their rows")
     _ok(_lib("sequence").dn_rotary(src.data_ptr(), _CODE[src.dtype], _rows(src, "src"), src_off, src_stride, dst.data_ptr(),
                                    _CODE[dst.dtype], _rows(dst, "dst"), dst_off, dst_stride, positions.data_ptr(), freq.data_ptr(),
-                                   T, n_vec, dims, width, float(mag), _stream()), "rotary")
+                                   T, n_vec, dims, width, float(mag), int(bool(halves)), _stream()), "rotary")
     return dst
 
 
@@ -1230,7 +1236,7 @@ def gated(x, g, kind, out):
 
 
 def state_scan(r, k, v, w, u, state, row_start, slots, n_heads, dk, dv, out, read_after=False, key_from_decay=False, beta=None,
-               w_head=None, qk_heads=None, beta_logits=False, w_rows=False):
+               w_head=None, qk_heads=None, beta_logits=False, w_rows=False, w_rate=None, w_bias=None):
     """The recurrence of a matrix state per head, S [dk, dv], over each request's rows of this step in order:
       a = 1 - w if key_from_decay else k
       read_after:  S <- diag(w) S + a v^T ;  o = S^T r
@@ -1239,6 +1245,7 @@ def state_scan(r, k, v, w, u, state, row_start, slots, n_heads, dk, dv, out, rea
     r, k: 32-bit [T, qk_heads * dk] (qk_heads None: n_heads; fewer: head h reads head h // (n_heads // qk_heads));
     w: 32-bit [T, heads * dk], or (w_rows) [T, heads], one decay per row and head for all the head's channels, or None with
     w_head: 32-bit [heads], one decay per head for every row and channel;
+    w_rate (and w_bias): 32-bit [heads], with w_rows in the delta rule: w holds z and the decay is exp(-w_rate log(1 + e^(z + w_bias)));
     v, out: 32-bit [T, heads * dv]; beta: 32-bit [T, heads] (beta_logits: it holds z, and beta is 1 / (1 + e^-z)); state: 32-bit [slots, heads * dv * dk] (a head's state
     held [value column][key channel]), read and written at the requests' slots."""
     G = n_heads if qk_heads is None else qk_heads
@@ -1256,7 +1263,8 @@ def state_scan(r, k, v, w, u, state, row_start, slots, n_heads, dk, dv, out, rea
     _need(all(t.shape[0] == T for t, _, _ in given), "state_scan: rows")
     _need(1 <= dk <= 256, lambda: f"state_scan: {dk} key channels a head; the kernel keeps up to 256 in registers")
     _need(beta is None or (not read_after and u is None), "state_scan: the delta rule reads after its write and has no bonus")
-    _f32vec(u, "u", n_heads * dk), _f32vec(w_head, "w_head", n_heads)
+    _need(w_rate is None or (w_rows and beta is not None), "state_scan: decays made from their arguments are the delta rule's, one per row and head")
+    _f32vec(u, "u", n_heads * dk), _f32vec(w_head, "w_head", n_heads), _f32vec(w_rate, "w_rate", n_heads), _f32vec(w_bias, "w_bias", n_heads)
     stride = _history(state, n_heads * dk * dv, "state_scan")
     mode = 2 if beta is not None else int(bool(read_after))
     _ok(_lib("sequence").dn_state_scan(r.data_ptr(), _rows(r, "r"), 0 if key_from_decay else k.data_ptr(),
@@ -1264,7 +1272,8 @@ def state_scan(r, k, v, w, u, state, row_start, slots, n_heads, dk, dv, out, rea
                                        _rows(w, "w") if w is not None else 0, _ptr(u), _ptr(beta),
                                        _rows(beta, "beta") if beta is not None else 0, _ptr(w_head), G, state.data_ptr(), stride,
                                        row_start.data_ptr(), slots.data_ptr(), S, T, n_heads, dk, dv, mode, int(key_from_decay),
-                                       int(bool(beta_logits)), int(bool(w_rows)), out.data_ptr(), _rows(out, "out"), _stream()),
+                                       int(bool(beta_logits)), int(bool(w_rows)), _ptr(w_rate), _ptr(w_bias), out.data_ptr(),
+                                       _rows(out, "out"), _stream()),
         "state_scan" if beta is None else "state_scan (delta rule)")
     return out
 
@@ -1489,12 +1498,13 @@ def norm_pair_write(z, q_width, wq, wk, eps, q_out, slot_map, k_pool, v_pool, wr
 
 
 def norm_turn_write(z, n_heads, n_kv, dk, dv, positions, q_out, slot_map, k_pool, v_pool, wq=None, wk=None, eps=None, q_scale=None,
-                    freq=None, v_freq=None, write=True):
+                    freq=None, v_freq=None, write=True, q_by_position=None):
     """A row of z (32-bit) begins with [q: n_heads x dk | k: n_kv x dk | v: n_kv x dv].  Every query and key is x / sqrt(mean(x^2) + eps)
     (eps None: x) times wq or wk (dk numbers shared by the heads, or None), then its first 2 len(freq) entries are turned in pairs (2i, 2i + 1) by
     positions[t] * freq[i]; a value's first 2 len(v_freq) entries likewise.  Queries times q_scale[head] go to q_out (heads side by
     side, as wide as the pools' keys), keys to k_pool [pages, n_kv, page, width], values to v_pool [pages, n_kv, width, page];
-    the columns a vector does not have are zeros.  slot_map as in norm_pair_write.  One launch."""
+    the columns a vector does not have are zeros.  slot_map as in norm_pair_write.  q_by_position = (coef, every): queries are also multiplied
+    by 1 + coef * ln(floor((positions[t] + 1) / every) + 1).  One launch."""
     _dev(z, "z", (torch.float32,), 2), _dev(q_out, "q_out", _FLOATS, 2), _dev(slot_map, "slot_map", _I32, 1), _dev(positions, "positions", _I32, 1)
     _dev(k_pool, "k_pool", (q_out.dtype,), 4), _dev(v_pool, "v_pool", (q_out.dtype,), 4)
     T = z.shape[0]
@@ -1506,11 +1516,89 @@ def norm_turn_write(z, n_heads, n_kv, dk, dv, positions, q_out, slot_map, k_pool
     _f32vec(wq, "wq", dk), _f32vec(wk, "wk", dk), _f32vec(q_scale, "q_scale", n_heads), _f32vec(freq, "freq"), _f32vec(v_freq, "v_freq")
     dims, v_dims = (0 if f is None else 2 * f.numel() for f in (freq, v_freq))
     _need(dims <= dk and v_dims <= dv, "norm_turn_write: more turned entries than a vector has")
+    coef, every = (0.0, 1.0) if q_by_position is None else (float(q_by_position[0]), float(q_by_position[1]))
+    _need(every > 0, "norm_turn_write: q_by_position")
     _ok(_lib("sequence").dn_norm_turn_write(z.data_ptr(), _rows(z, "z"), n_heads, n_kv, dk, dv, _ptr(wq), _ptr(wk), _ptr(q_scale),
-                                            -1.0 if eps is None else float(eps), _ptr(freq), dims, _ptr(v_freq), v_dims, positions.data_ptr(), q_out.data_ptr(),
+                                            coef, every, -1.0 if eps is None else float(eps), _ptr(freq), dims, _ptr(v_freq), v_dims, positions.data_ptr(), q_out.data_ptr(),
                                             _rows(q_out, "q_out"), kept, slot_map.data_ptr(), k_pool.data_ptr(), v_pool.data_ptr(), T, ps,
                                             _CODE[q_out.dtype], int(bool(write)), _stream()), "norm_turn_write")
     return q_out
+
+
+CONV_TURN_CHANNELS_MAX = 15000     # conv_turn_write keeps a row in LDS
+
+
+def conv_turn_write(z, n_heads, n_kv, dk, dv, w, hist, row_start, slots, positions, q_out, slot_map, k_pool, v_pool, wq, wk, eps, freq=None,
+                    write=True, move_on=False):
+    """A row of z (32-bit) begins with [q: n_heads x dk | k: n_kv x dk | v: n_kv x dv].  Every channel passes the short causal
+    convolution of conv_rows (identity=False, no activation; w [channels, taps], hist [slots, (taps - 1) * channels]); q and k are
+    each x / sqrt(mean(x^2) + eps) times a weight per entry as one vector over all heads; the first 2 len(freq) entries of every
+    head's q and k are turned in pairs (i, i + len(freq)) by positions[t] * freq[i]; then to q_out and the pools as norm_turn_write
+    puts them.  move_on: history_update in the same launch, for steps in which every request has one row."""
+    _dev(z, "z", (torch.float32,), 2), _dev(w, "w", (torch.float32,), 2), _dev(q_out, "q_out", _FLOATS, 2)
+    _dev(slot_map, "slot_map", _I32, 1), _dev(positions, "positions", _I32, 1)
+    _dev(k_pool, "k_pool", (q_out.dtype,), 4), _dev(v_pool, "v_pool", (q_out.dtype,), 4)
+    T = z.shape[0]
+    C, taps = w.shape
+    S = _request_tables(row_start, slots, "conv_turn_write")
+    n_pages, Hkv, ps, kept = k_pool.shape
+    _need(C == (n_heads + n_kv) * dk + n_kv * dv and w.is_contiguous() and z.shape[1] >= C and Hkv == n_kv and tuple(q_out.shape) == (T, n_heads * kept)
+          and max(dk, dv) <= kept <= 256 and kept % 2 == 0 and not (move_on and T != S), "conv_turn_write: shapes")
+    _need(C <= CONV_TURN_CHANNELS_MAX, lambda: f"conv_turn_write: {C} channels; a row in LDS has up to {CONV_TURN_CHANNELS_MAX}")
+    _need(slot_map.is_contiguous() and slot_map.shape[0] == T and positions.is_contiguous() and positions.shape[0] == T, "conv_turn_write: rows")
+    _need(k_pool.is_contiguous() and v_pool.is_contiguous() and tuple(v_pool.shape) == (n_pages, Hkv, kept, ps), "conv_turn_write: pools")
+    stride = _history(hist, (taps - 1) * C, "conv_turn_write") if taps > 1 else 0
+    _f32vec(wq, "wq", n_heads * dk), _f32vec(wk, "wk", n_kv * dk), _f32vec(freq, "freq")
+    dims = 0 if freq is None else 2 * freq.numel()
+    _need(dims <= dk, "conv_turn_write: more turned entries than a head has")
+    _ok(_lib("sequence").dn_conv_turn_write(z.data_ptr(), _rows(z, "z"), n_heads, n_kv, dk, dv, w.data_ptr(), taps, _ptr(hist) if taps > 1 else 0,
+                                            stride, row_start.data_ptr(), slots.data_ptr(), S, wq.data_ptr(), wk.data_ptr(), float(eps),
+                                            _ptr(freq) if dims else 0, dims, positions.data_ptr(), q_out.data_ptr(), _rows(q_out, "q_out"), kept,
+                                            slot_map.data_ptr(), k_pool.data_ptr(), v_pool.data_ptr(), T, ps, _CODE[q_out.dtype],
+                                            int(bool(write)), int(bool(move_on)), _stream()), "conv_turn_write")
+    return q_out
+
+
+def clamped_glu(z, limit, alpha, out):
+    """out = g * sigmoid(alpha g) * (u + 1) with g = min(z[:, :n], limit) and u = z[:, n:] clamped to +-limit; z: 32-bit [T, 2 n]."""
+    _dev(z, "z", (torch.float32,), 2), _dev(out, "out", _FLOATS, 2)
+    T, n = out.shape
+    _need(tuple(z.shape) == (T, 2 * n), "clamped_glu: shapes")
+    _ok(_lib("sequence").dn_clamped_glu(z.data_ptr(), _rows(z, "z"), float(limit), float(alpha), out.data_ptr(), _CODE[out.dtype],
+                                        _rows(out, "out"), T, n, _stream()), "clamped_glu")
+    return out
+
+
+def post_norm(x, y, alpha, weight, bias, eps, out=None, branches=None, chosen=None):
+    """x <- (u - mean(u)) / sqrt(var(u) + eps) * weight + bias with u = alpha * x + r, in place on 32-bit rows x [T, width]; out: the same
+    rows in its own dtype as well.  r is y; or, branches = (y2, w1, w2, beps), (y / rms(y) * w1 + y2 / rms(y2) * w2) / 2 with
+    rms(v) = sqrt(mean(v^2) + beps); or, chosen = (weights [T, top], ids int32 [T, top], n), sum_c weights[t, c] * y[t * top + c] over y
+    [T * top, width], where a choice ids[t, c] >= n gives the row x[t] itself (its row of y is not read)."""
+    _dev(x, "x", (torch.float32,), 2), _dev(y, "y", (torch.float32,), 2)
+    T, width = x.shape
+    _f32vec(weight, "weight", width), _f32vec(bias, "bias", width)
+    _need(weight is not None and not (branches is not None and chosen is not None), "post_norm: weight, or two kinds of results")
+    y2 = w1 = w2 = wts = ids = None
+    beps, top, n_rows = 0.0, 0, 0
+    if branches is not None:
+        y2, w1, w2, beps = branches
+        _dev(y2, "y2", (torch.float32,), 2)
+        _need(tuple(y2.shape) == (T, width), "post_norm: the second branch")
+        _f32vec(w1, "w1", width), _f32vec(w2, "w2", width)
+    if chosen is not None:
+        wts, ids, n_rows = chosen
+        _dev(wts, "weights", (torch.float32,), 2), _dev(ids, "ids", _I32, 2)
+        top = wts.shape[1]
+        _need(wts.is_contiguous() and ids.is_contiguous() and wts.shape[0] == T and ids.shape == wts.shape and top >= 1, "post_norm: choices")
+    _need(tuple(y.shape) == (T * max(top, 1), width), "post_norm: y")
+    if out is not None:
+        _dev(out, "out", _FLOATS, 2)
+        _need(tuple(out.shape) == (T, width), "post_norm: out")
+    _ok(_lib("sequence").dn_post_norm(x.data_ptr(), _rows(x, "x"), float(alpha), y.data_ptr(), _rows(y, "y"), _ptr(y2),
+                                      _rows(y2, "y2") if y2 is not None else 0, _ptr(w1), _ptr(w2), float(beps), _ptr(wts), _ptr(ids), top,
+                                      int(n_rows), weight.data_ptr(), _ptr(bias), float(eps), _ptr(out), _CODE[out.dtype] if out is not None else 0,
+                                      _rows(out, "out") if out is not None else 0, T, width, _stream()), "post_norm")
+    return x
 
 
 def turn_back_gate(o, n_heads, dv, out, positions=None, freq=None, gate=None, head_stride=None):
@@ -1563,28 +1651,30 @@ def heads_linear(a, w, out, a_off=0, a_stride=None, o_off=0, o_stride=None):
     return out
 
 
-def moe_route(z, correction, top, ids, wts, score="softmax", renorm=True, n_experts=None, groups=1, keep=1, scale=1.0):
+def moe_route(z, correction, top, ids, wts, score="softmax", renorm=True, n_experts=None, groups=1, keep=1, scale=1.0, group_by="two"):
     """Per row: s = softmax(z) over the experts, or (score "sigmoid") each expert's own 1 / (1 + e^-z); the `top` experts with
     the largest s + correction (the lower index wins a tie) go to ids [T, top]; wts [T, top] gets their s divided by the sum
     of the chosen s (+ 1e-20), or (renorm False) their s as it is, times `scale`.  n_experts: the first columns of z that are
     experts (None: all of them).  groups > 1: the experts are that many equal runs of neighbours, a group's score is the sum
-    of its two largest s + correction, and only experts of the `keep` best groups can be chosen."""
+    of its two largest s + correction (group_by "best": its largest), and only experts of the `keep` best groups can be chosen."""
     _dev(z, "z", (torch.float32,), 2), _dev(ids, "ids", _I32, 2), _dev(wts, "wts", (torch.float32,), 2)
     T = z.shape[0]
     E = z.shape[1] if n_experts is None else n_experts
     _need(ids.is_contiguous() and wts.is_contiguous() and tuple(ids.shape) == (T, top) and E <= z.shape[1]
-          and tuple(wts.shape) == (T, top) and 1 <= top <= E and score in ("softmax", "sigmoid"), "moe_route: shapes")
+          and tuple(wts.shape) == (T, top) and 1 <= top <= E and score in ("softmax", "sigmoid")
+          and group_by in ("two", "best"), "moe_route: shapes")
     _need(groups >= 1 and E % groups == 0 and 1 <= keep <= groups and top <= keep * (E // groups),
           lambda: f"moe_route: {E} experts in {groups} groups of which {keep} are kept, for {top} choices")
     _f32vec(correction, "correction", E)
     _ok(_lib("grouped").dn_moe_route(z.data_ptr(), _rows(z, "z"), _ptr(correction), T, E, top, int(score == "sigmoid"),
-                                     int(bool(renorm)), ids.data_ptr(), wts.data_ptr(), int(groups), int(keep), float(scale),
+                                     int(bool(renorm)), ids.data_ptr(), wts.data_ptr(), int(groups), int(keep), int(group_by == "best"), float(scale),
                                      _stream()), "moe_route")
 
 
 def moe_plan(ids, n_experts, offsets, order):
     """The pairs (row, choice), pair i = row * top + choice, sorted by expert and then by i: order [T * top]; expert e has
-    the places offsets[e] .. offsets[e + 1] - 1 (offsets [experts + 1])."""
+    the places offsets[e] .. offsets[e + 1] - 1 (offsets [experts + 1]).  A choice of n_experts or more is none of the experts':
+    its pair has no place, and the last entries of `order` are not written."""
     _dev(ids, "ids", _I32, 2), _dev(offsets, "offsets", _I32, 1), _dev(order, "order", _I32, 1)
     n = ids.numel()
     _need(ids.is_contiguous() and offsets.shape[0] == n_experts + 1 and order.shape[0] == n and offsets.is_contiguous()
@@ -1653,9 +1743,10 @@ def moe_down(y, order, offsets, w_down, out, dims=None):
                                     _CODE[wdt], width, ff, out.data_ptr(), int(dims is not None), _stream()), "moe_down")
 
 
-def moe_combine(out, wts, x, logits=False):
+def moe_combine(out, wts, x, logits=False, ids=None, n_experts=0, h=None):
     """x[t, :] += sum_c wts[t, c] * out[t * top + c, :], the choices in their order (wts None: every weight is 1; logits: a
-    weight is 1 / (1 + e^-z) of what wts holds; wts may be columns of wider rows)."""
+    weight is 1 / (1 + e^-z) of what wts holds; wts may be columns of wider rows).  ids (int32 [T, top]), h [T, width]: a choice
+    of n_experts or more gives h[t, :] in place of its row of `out`."""
     _dev(out, "out", (torch.float32,), 2), _dev(x, "x", (torch.float32,), 2)
     T, width = x.shape
     top = out.shape[0] // max(T, 1) if wts is None else wts.shape[1]
@@ -1663,6 +1754,10 @@ def moe_combine(out, wts, x, logits=False):
         _dev(wts, "wts", (torch.float32,), 2)
         _need(wts.shape[0] == T and not (logits and wts is None), "moe_combine: weights")
     _need(out.is_contiguous() and tuple(out.shape) == (T * top, width), "moe_combine: shapes")
+    if ids is not None:
+        _dev(ids, "ids", _I32, 2), _dev(h, "h", _FLOATS, 2)
+        _need(ids.is_contiguous() and tuple(ids.shape) == (T, top) and tuple(h.shape) == (T, width), "moe_combine: ids or h")
     _ok(_lib("grouped").dn_moe_combine(out.data_ptr(), _ptr(wts), _rows(wts, "wts") if wts is not None else 0, int(bool(logits)), T, top,
-                                       width, x.data_ptr(), _rows(x, "x"), _stream()),
+                                       width, x.data_ptr(), _rows(x, "x"), _ptr(ids), int(n_experts), _ptr(h),
+                                       _CODE[h.dtype] if h is not None else 0, _rows(h, "h") if h is not None else 0, _stream()),
         "moe_combine")

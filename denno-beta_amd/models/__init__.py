@@ -1,2 +1,2 @@
 """Architectures the framework ships.  Importing a module registers it."""
-from . import dogalorn, fikupel, gpt2, nigilorn, pafivik, ridopel   # noqa: F401
+from . import dogalorn, fikupel, gpt2, nigilorn, pafivik, pepapel, ridopel   # noqa: F401

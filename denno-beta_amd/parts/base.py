@@ -88,6 +88,9 @@ class Runtime:
     # rows that the kernel which last changed the stream has normed already for the norm that reads it next: (norm, rows), or
     # None; whoever changes the stream otherwise clears it (the model does at a step's start and end)
     normed_rows: Optional[tuple] = None
+    # the stream's rows in the activation dtype as the kernel that last changed the stream left them beside it (the "post_norm"
+    # arrangement, whose sublayers read the stream itself), or None; the model clears it where the stream changes in any other way
+    stream_cast: Optional[torch.Tensor] = None
     # the model's further tables by name (DecoderSpec.tables), for parts that pick rows of them (set by the model)
     tables: Dict[str, torch.Tensor] = field(default_factory=dict)
 

@@ -144,6 +144,46 @@ class PlainPreNormBlock:
             self.ffn.forward(self.norm2.forward(x, runtime.act_dtype), ctx, accumulate_into=x)
 
 
+@ARRANGEMENTS.register("post_norm")
+class PostNormBlock:
+    """A norm behind the sum: x <- norm1(alpha x + mixer(x)); x <- norm2(alpha x + ffn(x)).  The sublayers read the stream
+    itself; the norms are of a kind that takes a result into the stream (`replace(x, y, ..)`, parts.norms.SumLayerNorm: alpha is
+    theirs) and leaves the new rows in the activation dtype for the next reader (across blocks: `runtime.stream_cast`).  Two
+    branches of a mixer, and experts' rows with their weights, are handed to that kernel as they are.  The mixer may be several
+    side by side (its `cache_parts`).  A block whose feed-forward is "none" ends after the mixer."""
+
+    SLOTS = {"mixer": "mixer", "norm1": "norm", "ffn": "feed_forward", "norm2": "norm"}
+    keeps_cast = True
+
+    def __init__(self, mixer, norm1, ffn, norm2):
+        self.mixer, self.norm1, self.ffn, self.norm2 = mixer, norm1, ffn, norm2
+        self.has_ffn = not getattr(ffn, "absent", False)
+        for n in (norm1, norm2):
+            if not hasattr(n, "replace"):
+                raise TypeError(f"post_norm: the norm behind a sum must take a result into the stream; {type(n).__name__} does not")
+
+    def parts(self):
+        return [self.mixer, self.norm1] + ([self.ffn, self.norm2] if self.has_ffn else [])
+
+    def mixers(self):
+        return self.mixer.cache_parts()
+
+    def forward(self, x, ctx, caches, runtime):
+        act = runtime.act_dtype
+        runtime.stream_stats = None
+        h, runtime.stream_cast = runtime.stream_cast, None
+        if h is None:
+            h = x if act == x.dtype else ops.cast(x, torch.empty(x.shape, dtype=act, device=x.device))
+        pair = self.mixer.forward_pair(h, ctx, caches) if hasattr(self.mixer, "forward_pair") else None
+        y, branches = pair if pair is not None else (SandwichBlock._result(self.mixer, x, h, ctx, caches if len(caches) != 1 else caches[0]), None)
+        h = self.norm1.replace(x, y, act, branches=branches)
+        if self.has_ffn:
+            apart = self.ffn.forward_chosen(h, ctx) if hasattr(self.ffn, "forward_chosen") else None
+            y, chosen = apart if apart is not None else (SandwichBlock._result(self.ffn, x, h, ctx), None)
+            h = self.norm2.replace(x, y, act, chosen=chosen)
+        runtime.stream_cast = h
+
+
 @ARRANGEMENTS.register("sandwich")
 class SandwichBlock:
     """A norm before and a norm behind each sublayer: x += post1(mixer(norm1(x))); x += post2(ffn(norm2(x))).  The norms

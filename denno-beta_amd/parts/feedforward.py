@@ -91,19 +91,25 @@ class DenseMLP(Part):
 
 @FEED_FORWARDS.register("gated_mlp")
 class GatedMLP(Part):
-    """W_down (act(W_gate h) * (W_up h)), act "silu"; no biases.  Gate and up are one product whose 32-bit result the
-    activation reads."""
+    """W_down (act(W_gate h) * (W_up h)), act "silu"; without biases, or with one for each of the three matrices (gate_bias,
+    up_bias, down_bias).  Gate and up are one product whose 32-bit result the activation reads.
+    activation "clamped": with g = min(W_gate h, limit) and u = W_up h between -limit and limit, W_down (g sigmoid(alpha g) (u + 1))."""
     graph_safe = True
     returns_rows = True
     libraries = ("sequence",)
 
-    def __init__(self, width: int, inner: int, gate_weight: str, up_weight: str, down_weight: str, activation: str = "silu"):
-        if activation != "silu":
-            raise ValueError(f"gated_mlp: activation {activation!r}; known: ['silu']")
+    def __init__(self, width: int, inner: int, gate_weight: str, up_weight: str, down_weight: str, activation: str = "silu",
+                 gate_bias=None, up_bias=None, down_bias=None, limit: float = 0.0, alpha: float = 1.0):
+        if activation not in ("silu", "clamped"):
+            raise ValueError(f"gated_mlp: activation {activation!r}; known: ['clamped', 'silu']")
+        if (gate_bias is None) != (up_bias is None):
+            raise ValueError("gated_mlp: gate and up are one product: both have a bias, or neither")
         self.width, self.inner, self.activation = width, inner, activation
-        self.up = Linear(width, 2 * inner, gate_weight + "+up", None, init_std=width ** -0.5,
-                         weight_sources=((gate_weight, inner), (up_weight, inner)))
-        self.down = Linear(inner, width, down_weight, None, init_std=inner ** -0.5)
+        self.limit, self.alpha = float(limit), float(alpha)
+        self.up = Linear(width, 2 * inner, gate_weight + "+up", gate_bias + "+up" if gate_bias else None, init_std=width ** -0.5,
+                         weight_sources=((gate_weight, inner), (up_weight, inner)),
+                         bias_sources=((gate_bias, inner), (up_bias, inner)) if gate_bias else None)
+        self.down = Linear(inner, width, down_weight, down_bias, init_std=inner ** -0.5)
 
     def param_specs(self):
         return self.up.param_specs() + self.down.param_specs()
@@ -115,7 +121,11 @@ class GatedMLP(Part):
     def forward(self, h, ctx, accumulate_into):
         n = self.inner
         gu = self.up(h, out_dtype=F32)
-        f = ops.gated(gu[:, n:], gu[:, :n], self.activation, torch.empty((h.shape[0], n), dtype=self.runtime.act_dtype, device=h.device))
+        f = torch.empty((h.shape[0], n), dtype=self.runtime.act_dtype, device=h.device)
+        if self.activation == "clamped":
+            ops.clamped_glu(gu, self.limit, self.alpha, f)
+        else:
+            ops.gated(gu[:, n:], gu[:, :n], self.activation, f)
         if accumulate_into is None:
             return self.down(f, out_dtype=F32)
         self.down(f, residual=accumulate_into)
@@ -149,27 +159,36 @@ class RoutedExperts(Part):
     shared: an expert of the same form that every token uses, dict(inner, gate, up, down, token_gate): its result is
     added, times sigmoid(w . h) with w the vector `token_gate` (a name, or None: as it is); groups and keep: the experts are
     `groups` equal runs of neighbours, a group's score is the sum of its two largest s + correction, and only the experts
-    of the `keep` best groups can be chosen; route_scale multiplies the weights; router_bias: a vector's name, added to W_router h
-    (score "softmax" with renorm: the weights are then the softmax over the chosen logits alone)."""
+    of the `keep` best groups can be chosen (group_by "best": a group's score is its largest s + correction); route_scale multiplies
+    the weights; router_bias: a vector's name, added to W_router h (score "softmax" with renorm: the weights are then the softmax over
+    the chosen logits alone); identity: the router has that many outputs behind the experts' (scores, correction and groups run over
+    all of them), and one of those, chosen, returns the row that the experts read, times its weight."""
     graph_safe = True
     returns_rows = True
     libraries = ("grouped", "sequence")
 
     def __init__(self, width: int, inner: int, n_experts: int, top: int, router: str, correction, gate: str, up: str, down: str,
                  limit: float = 0.0, alpha: float = 1.0, score: str = "softmax", renorm: bool = True, weigh: str = "output",
-                 act: str = "clamped", shared=None, groups: int = 1, keep: int = 1, route_scale: float = 1.0, router_bias=None):
+                 act: str = "clamped", shared=None, groups: int = 1, keep: int = 1, route_scale: float = 1.0, router_bias=None,
+                 identity: int = 0, group_by: str = "two"):
         """gate, up, down: tensor names with {e} for the expert's number; correction: a name or None."""
-        if not 1 <= top <= n_experts:
-            raise ValueError(f"routed_experts: {top} of {n_experts} experts")
+        outputs = n_experts + identity      # (of the router)
+        if identity < 0 or not 1 <= top <= outputs:
+            raise ValueError(f"routed_experts: {top} of {n_experts} experts and {identity} that return their input")
+        if identity and (shared or weigh != "output"):
+            raise ValueError("routed_experts: outputs that return their input beside a shared expert or weights on the input are not built")
         if score not in ("softmax", "sigmoid") or weigh not in ("output", "input") or act not in ("clamped", "silu", "relu2"):
             raise ValueError(f"routed_experts: score {score!r}, weigh {weigh!r}, act {act!r}")
         if weigh == "input" and act != "silu":
             raise ValueError("routed_experts: a weight on what the expert reads goes with act 'silu'")
         if (act == "relu2") != (gate is None):
             raise ValueError("routed_experts: act 'relu2' is an expert without a gate matrix, and only that one")
-        if groups < 1 or n_experts % groups != 0 or not 1 <= keep <= groups or top > keep * (n_experts // groups):
-            raise ValueError(f"routed_experts: {n_experts} experts in {groups} groups of which {keep} are kept, for {top} choices")
+        if group_by not in ("two", "best"):
+            raise ValueError(f"routed_experts: group_by {group_by!r}")
+        if groups < 1 or outputs % groups != 0 or not 1 <= keep <= groups or top > keep * (outputs // groups):
+            raise ValueError(f"routed_experts: {outputs} experts in {groups} groups of which {keep} are kept, for {top} choices")
         self.groups, self.keep, self.route_scale = int(groups), int(keep), float(route_scale)
+        self.identity, self.outputs, self.group_by = int(identity), outputs, group_by
         self.gated = gate is not None
         self.width, self.inner, self.n_experts, self.top = width, inner, n_experts, top
         self.limit, self.alpha = float(limit), float(alpha)
@@ -185,7 +204,7 @@ class RoutedExperts(Part):
             self.router = Linear(width, n_experts + 1, router + "+gate", None, init_std=width ** -0.5,
                                  weight_sources=((router, n_experts), (self.token_gate, 1)))
         else:
-            self.router = Linear(width, n_experts, router, router_bias)
+            self.router = Linear(width, outputs, router, router_bias)
         if self.shared:
             sh = self.shared
             if self.gated:
@@ -205,7 +224,7 @@ class RoutedExperts(Part):
     def param_specs(self):
         specs = self.router.param_specs() + [self._stacked(w) for w in (("gate", "up", "down") if self.gated else ("up", "down"))]
         if self.correction_name:
-            specs.append(ParamSpec(self.correction_name, (self.n_experts,), "vector", ("normal", 0.0, 0.02)))
+            specs.append(ParamSpec(self.correction_name, (self.outputs,), "vector", ("normal", 0.0, 0.02)))
         if self.shared:
             specs += self.shared_up.param_specs() + self.shared_down.param_specs()
         return specs
@@ -237,13 +256,22 @@ class RoutedExperts(Part):
     def forward_apart(self, h, ctx):
         """-> (the chosen experts' results [T * top, width], their weights [T, top]): for whoever adds the weighted sum up in a kernel
         of its own (ops.streams_write's `weigh`); None where something else belongs to the result."""
-        if self.shared or self.weigh == "input":
+        if self.shared or self.weigh == "input" or self.identity:
             return None
-        _, out, wts, _ = self._experts(h)
+        _, out, wts, _, _ = self._experts(h)
         return out, wts
 
+    def forward_chosen(self, h, ctx):
+        """-> (the chosen experts' results [T * top, width], (weights [T, top], the chosen outputs' numbers [T, top], how many of the
+        outputs are experts)): for whoever adds the weighted sum up, with the row itself for an output that returns its input
+        (ops.post_norm's `chosen`); None where something else belongs to the result."""
+        if self.shared or self.weigh == "input":
+            return None
+        _, out, wts, ids, _ = self._experts(h)
+        return out, (wts, ids, self.n_experts)
+
     def _experts(self, h):
-        """-> (the router's result, the experts' results, the chosen ones' weights, h in the experts' precision)."""
+        """-> (the router's result, the experts' results, the chosen ones' weights and numbers, h in the experts' precision)."""
         T, top, dev = h.shape[0], self.top, h.device
         wdt = self.w_dtype
         if h.dtype != wdt:        # (experts stored in 32-bit in a bfloat16 engine: their products run on widened rows)
@@ -251,8 +279,8 @@ class RoutedExperts(Part):
         z = self.router(h, out_dtype=torch.float32)
         ids = torch.empty((T, top), dtype=torch.int32, device=dev)
         wts = torch.empty((T, top), dtype=torch.float32, device=dev)
-        ops.moe_route(z, self.correction, top, ids, wts, score=self.score, renorm=self.renorm, n_experts=self.n_experts,
-                      groups=self.groups, keep=self.keep, scale=self.route_scale)
+        ops.moe_route(z, self.correction, top, ids, wts, score=self.score, renorm=self.renorm, n_experts=self.outputs,
+                      groups=self.groups, keep=self.keep, scale=self.route_scale, group_by=self.group_by)
         offsets = torch.empty(self.n_experts + 1, dtype=torch.int32, device=dev)
         order = torch.empty(T * top, dtype=torch.int32, device=dev)
         ops.moe_plan(ids, self.n_experts, offsets, order)
@@ -262,14 +290,18 @@ class RoutedExperts(Part):
                    kind=self.act, in_scale=wts if on_input else None)
         out = torch.empty((T * top, self.width), dtype=torch.float32, device=dev)
         ops.moe_down(y, order, offsets, self.w_down, out, dims=self.down_dims)
-        return z, out, wts, h
+        return z, out, wts, ids, h
 
     def forward(self, h, ctx, accumulate_into):
         T, dev = h.shape[0], h.device
         returns = accumulate_into is None
         if returns:
             accumulate_into = torch.zeros((T, self.width), dtype=torch.float32, device=dev)
-        z, out, wts, h = self._experts(h)
+        row = h
+        z, out, wts, ids, h = self._experts(h)
+        if self.identity:
+            ops.moe_combine(out, wts, accumulate_into, ids=ids, n_experts=self.n_experts, h=row)
+            return accumulate_into if returns else None
         ops.moe_combine(out, None if self.weigh == "input" else wts, accumulate_into)
         if self.shared:
             n = self.shared["inner"]

@@ -7,7 +7,7 @@ import torch
 
 from ..kernels import ops
 from ..weights.spec import ParamSpec
-from .base import MIXERS, POSITIONS, PagedKV, Part
+from .base import MIXERS, POSITIONS, FixedState, PagedKV, Part
 from .linear import Linear
 
 
@@ -38,9 +38,11 @@ class CausalSelfAttention(Part):
     head_dim numbers that all heads share.  temp: the name of a number per head that multiplies its scores.  turn_values: the
     value of a position is turned by it over all its pairs (by position * base^(-2m/value_dim), base the encoding's, whatever
     scaling the keys' has) and kept so; a head's result is turned back by its own position.  entry_gate: the name of a matrix
-    [n_heads * value_dim, width]: the heads' results are multiplied entry by entry with sigmoid(W h).  Any of these four: one
+    [n_heads * value_dim, width]: the heads' results are multiplied entry by entry with sigmoid(W h).  position_temp = (coef, every):
+    queries are multiplied by 1 + coef ln(floor((position + 1) / every) + 1).  Any of these five: one
     kernel makes queries, keys and values from the projection's 32-bit result and puts keys and values into the cache
-    (ops.norm_turn_write), one turns the result back and gates it (ops.turn_back_gate)."""
+    (ops.norm_turn_write), one turns the result back and gates it (ops.turn_back_gate).
+    softcap > 0: a scaled score s becomes softcap * tanh(s / softcap)."""
     graph_safe = True
     returns_rows = True
 
@@ -48,20 +50,28 @@ class CausalSelfAttention(Part):
                  qkv_weight: str, qkv_bias, out_weight: str, out_bias, stored_in_out: bool = False,
                  window: int = 0, out_init_std: float = 0.02, position=None, qkv_weight_sources=None,
                  qkv_bias_sources=None, value_dim=None, exact_turn: bool = False, unit_eps=None, head_gate=None, sink=None,
-                 keep_first: int = 0, qk_norm=None, temp=None, turn_values: bool = False, entry_gate=None):
+                 keep_first: int = 0, qk_norm=None, temp=None, turn_values: bool = False, entry_gate=None, position_temp=None,
+                 softcap: float = 0.0):
         self.width, self.n_heads, self.n_kv_heads, self.head_dim = width, n_heads, n_kv_heads, head_dim
         self.value_dim = head_dim if value_dim is None else int(value_dim)
         self.unit_eps = None if unit_eps is None else float(unit_eps)
         self.head_gate, self.entry_gate = head_gate, entry_gate
         self.sink_name, self.temp_name, self.qk_norm, self.turn_values = sink, temp, (dict(qk_norm) if qk_norm else None), bool(turn_values)
         self.keep_first = int(keep_first) if window > 0 else 0
-        self.prepared = qk_norm is not None or temp is not None or self.turn_values or entry_gate is not None
+        self.position_temp = None if position_temp is None else (float(position_temp[0]), float(position_temp[1]))
+        if self.position_temp is not None and not self.position_temp[1] > 0:
+            raise ValueError(f"causal_attention: a temperature that grows every {position_temp[1]} positions")
+        self.softcap = float(softcap)
+        if not self.softcap >= 0:
+            raise ValueError(f"causal_attention: softcap {softcap}")
+        self.prepared = (qk_norm is not None or temp is not None or self.turn_values or entry_gate is not None
+                         or self.position_temp is not None)
         self.split = (bool(exact_turn) or self.value_dim != head_dim or self.unit_eps is not None or head_gate is not None
                       or self.prepared)
         if self.prepared:
             self.libraries = ("sequence",)
             if unit_eps is not None or head_gate is not None:
-                raise ValueError("causal_attention: unit_eps and head_gate do not go with qk_norm, temp, turn_values or entry_gate")
+                raise ValueError("causal_attention: unit_eps and head_gate do not go with qk_norm, temp, turn_values, entry_gate or position_temp")
             if self.turn_values and (self.value_dim % 2 != 0 or position is None or position[0] != "rotary_pairs"):
                 raise ValueError(f"causal_attention: values of {self.value_dim} numbers are turned in pairs, by the base of a rotary_pairs "
                                  "encoding of the layer's own")
@@ -148,7 +158,7 @@ class CausalSelfAttention(Part):
         q = new((T, H * hw), dtype=act, device=dev)
         kv = new((T, 2 * G * hw), dtype=act, device=dev)      # keys at column 0, values at G * hw
 
-        if turns and not hasattr(position, "freq"):
+        if turns and (not hasattr(position, "freq") or getattr(position, "halves", False)):
             raise TypeError(f"{type(position).__name__}: the 32-bit turn needs an encoding with a table of frequencies (rotary_pairs)")
         dims = position.dims if turns else 0
         freq = position.freq if turns else self.no_freq
@@ -162,7 +172,7 @@ class CausalSelfAttention(Part):
             ops.kv_write(kv, 0, G * hw, g.slot_map, cache.k, cache.v)
         o = torch.empty((T, H * hw), dtype=act, device=dev)
         ops.attention(q, o, cache.k, cache.v, g.block_tables, g.tiles, H, self.scale, self.window, tiles_wide=g.tiles_wide,
-                      single_rows=g.single_rows, max_context=g.max_context, sink=self.sink, keep_first=self.keep_first)
+                      single_rows=g.single_rows, max_context=g.max_context, sink=self.sink, keep_first=self.keep_first, softcap=self.softcap)
         if self.head_gate is not None:      # (the gate per head, and the heads' first value_dim columns on, in one launch)
             o = ops.head_gate(o, z[:, self.gate_col:self.gate_col + H], H, dv, torch.empty((T, H * dv), dtype=act, device=dev),
                               head_stride=hw)
@@ -180,15 +190,16 @@ class CausalSelfAttention(Part):
         act, T, dev = self.runtime.act_dtype, h.shape[0], h.device
         H, G, dv, hw = self.n_heads, self.n_kv_heads, self.value_dim, self.kept_dim
         turns = position is not None and getattr(position, "rotates", False)
-        if turns and (not hasattr(position, "freq") or position.mag != 1.0):
+        if turns and (not hasattr(position, "freq") or position.mag != 1.0 or getattr(position, "halves", False)):
             raise TypeError(f"{type(position).__name__}: this turn needs a table of frequencies and no factor on cos and sin (rotary_pairs)")
         z = self.qkv(h, out_dtype=torch.float32)
         q = ops.norm_turn_write(z, H, G, self.head_dim, dv, ctx.positions, torch.empty((T, H * hw), dtype=act, device=dev), g.slot_map,
                                 cache.k, cache.v, wq=self.wq, wk=self.wk, eps=self.qk_norm["eps"] if self.qk_norm else None,
-                                q_scale=self.temp, freq=position.freq if turns else None, v_freq=self.v_freq, write=cache.writes)
+                                q_scale=self.temp, freq=position.freq if turns else None, v_freq=self.v_freq, write=cache.writes,
+                                q_by_position=self.position_temp)
         o = torch.empty((T, H * hw), dtype=act, device=dev)
         ops.attention(q, o, cache.k, cache.v, g.block_tables, g.tiles, H, self.scale, self.window, tiles_wide=g.tiles_wide,
-                      single_rows=g.single_rows, max_context=g.max_context, sink=self.sink, keep_first=self.keep_first)
+                      single_rows=g.single_rows, max_context=g.max_context, sink=self.sink, keep_first=self.keep_first, softcap=self.softcap)
         if hw != dv or self.v_freq is not None or self.entry_gate is not None:
             o = ops.turn_back_gate(o, H, dv, torch.empty((T, H * dv), dtype=act, device=dev), positions=ctx.positions, freq=self.v_freq,
                                    gate=z[:, self.gate_col:self.gate_col + H * dv] if self.entry_gate is not None else None, head_stride=hw)
@@ -224,7 +235,7 @@ class CausalSelfAttention(Part):
             o = torch.empty((h.shape[0], self.q_width), dtype=act, device=h.device)
         ops.attention(q, o, cache.k, cache.v, g.block_tables, g.tiles, self.n_heads,
                       self.scale, self.window, tiles_wide=g.tiles_wide, single_rows=g.single_rows,
-                      max_context=g.max_context, sink=self.sink, keep_first=self.keep_first)
+                      max_context=g.max_context, sink=self.sink, keep_first=self.keep_first, softcap=self.softcap)
         if accumulate_into is None:
             return self.out(o, out_dtype=torch.float32)
         self.out(o, residual=accumulate_into, stats=stats, deferred=deferred)
@@ -488,12 +499,118 @@ class ChunkAttention(Part):
         self.out(o, residual=accumulate_into)
 
 
+class ConvHistory(Part):
+    """The state of a short convolution that a mixer with pages runs on its projections: the last taps - 1 rows, 32-bit."""
+
+    def __init__(self, channels: int, taps: int):
+        self.channels, self.taps = channels, taps
+
+    def cache_spec(self):
+        return FixedState(((self.taps - 1) * self.channels,))
+
+
+@MIXERS.register("conv_attention")
+class ConvAttention(Part):
+    """Causal softmax attention whose queries, keys and values pass a short causal convolution over time on every channel (no
+    activation; the last tap weighs the token's own).  Behind it q and k are each normed as one vector over all heads
+    (x / sqrt(mean(x^2) + eps) times a weight per entry), then turned by the position (position: the arguments of a "rotary_halves"
+    encoding, or None).  chunk > 0: position i reads j <= i of its own run of `chunk` positions (runs counted from the sequence's
+    position 0); the pages of runs that no later row reads are given back.  A name "g": a matrix [n_heads, width], head a's result
+    is multiplied by sigmoid(W_g h)_a.  Query head a reads key head a // (n_heads // n_kv_heads).  Then the output projection.
+
+    Two caches: the pages, and (with more than one tap) the projections' last rows (`ConvHistory`)."""
+    graph_safe = True
+    returns_rows = True
+    libraries = ("sequence",)
+    joinable = True      # (`proj` may be part of a product that several mixers share: parts.mixers.ParallelMixers)
+
+    def __init__(self, width: int, n_heads: int, n_kv_heads: int, head_dim: int, value_dim: int, taps: int, scale: float, eps: float,
+                 names: dict, chunk: int = 0, position=None):
+        """names: q, k, v, o and optionally g (matrices); q_conv, k_conv, v_conv ([channels, taps]); q_norm, k_norm (vectors over
+        all heads)."""
+        if n_heads % n_kv_heads != 0:
+            raise ValueError(f"conv_attention: {n_heads} heads cannot share {n_kv_heads} key heads")
+        if taps < 1 or chunk < 0:
+            raise ValueError(f"conv_attention: {taps} taps, chunks of {chunk}")
+        self.width, self.n_heads, self.n_kv_heads, self.head_dim, self.value_dim = width, n_heads, n_kv_heads, head_dim, value_dim
+        self.taps, self.scale, self.eps, self.chunk, self.names = int(taps), float(scale), eps, int(chunk), dict(names)
+        self.kept_dim = -(-max(head_dim, value_dim) // 16) * 16      # (keys and values in one width that every attention kernel takes)
+        if self.kept_dim > 256:
+            raise ValueError(f"conv_attention: keys of {head_dim} and values of {value_dim}: the attention kernels take up to 256")
+        self.q_width, self.kv_width, self.v_width = n_heads * head_dim, n_kv_heads * head_dim, n_kv_heads * value_dim
+        self.channels = self.q_width + self.kv_width + self.v_width
+        if self.channels > ops.CONV_TURN_CHANNELS_MAX:
+            raise ValueError(f"conv_attention: {self.channels} channels; its kernel keeps up to {ops.CONV_TURN_CHANNELS_MAX}")
+        n = names
+        self.gated = "g" in n
+        pieces = ((n["q"], self.q_width), (n["k"], self.kv_width), (n["v"], self.v_width)) + (((n["g"], n_heads),) if self.gated else ())
+        self.proj = Linear(width, sum(c for _, c in pieces), n["q"] + "+k+v" + ("+g" if self.gated else ""), None, init_std=width ** -0.5,
+                           weight_sources=pieces)
+        self.out = Linear(n_heads * value_dim, width, n["o"], None, init_std=(n_heads * value_dim) ** -0.5)
+        self.position = POSITIONS.make(("rotary_halves", dict(position, head_dim=head_dim))) if position is not None else None
+        self.history = ConvHistory(self.channels, self.taps) if self.taps > 1 else None
+        self.joined = False
+
+    def cache_parts(self):
+        return [self] + ([self.history] if self.history is not None else [])
+
+    def param_specs(self):
+        n = self.names
+        return ([] if self.joined else self.proj.param_specs()) + self.out.param_specs() + [
+            ParamSpec(n["q_conv"] + "+k+v", (self.channels, self.taps), "vector", ("normal", 0.3, 0.4),
+                      sources=((n["q_conv"], self.q_width), (n["k_conv"], self.kv_width), (n["v_conv"], self.v_width))),
+            ParamSpec(n["q_norm"], (self.q_width,), "vector", ("normal", 1.0, 0.1)),
+            ParamSpec(n["k_norm"], (self.kv_width,), "vector", ("normal", 1.0, 0.1))]
+
+    def cache_spec(self):
+        # (a row's run begins at most chunk - 1 positions before it: a window of that many keys never gives back too much)
+        return PagedKV(self.n_kv_heads, self.kept_dim, self.chunk)
+
+    def bind(self, tensors, runtime):
+        super().bind(tensors, runtime)
+        if not self.joined:
+            self.proj.bind(tensors)
+        self.out.bind(tensors)
+        n = self.names
+        self.conv = tensors[n["q_conv"] + "+k+v"].contiguous()
+        self.q_norm, self.k_norm = tensors[n["q_norm"]], tensors[n["k_norm"]]
+        if self.position is not None:
+            self.position.bind(tensors, runtime)
+
+    def forward(self, h, ctx, cache, accumulate_into, z=None):
+        """z: what `proj` gives for h, 32-bit, where a shared product has made it."""
+        act, T, dev = self.runtime.act_dtype, h.shape[0], h.device
+        H, G, dk, dv, hw, C = self.n_heads, self.n_kv_heads, self.head_dim, self.value_dim, self.kept_dim, self.channels
+        cache, past = cache if self.history is not None else ((cache[0] if isinstance(cache, (list, tuple)) else cache), None)
+        g = ctx.groups[cache.group]
+        if z is None:
+            z = self.proj(h, out_dtype=torch.float32)
+        single = ctx.single_rows and cache.writes
+        q = ops.conv_turn_write(z, H, G, dk, dv, self.conv, past.state if past is not None else None, ctx.row_start, ctx.state_slots,
+                                ctx.positions, torch.empty((T, H * hw), dtype=act, device=dev), g.slot_map, cache.k, cache.v, self.q_norm,
+                                self.k_norm, self.eps, freq=self.position.freq if self.position is not None else None, write=cache.writes,
+                                move_on=single)
+        if past is not None and cache.writes and not single:
+            ops.history_update(z[:, :C], past.state, ctx.row_start, ctx.state_slots)
+        o = torch.empty((T, H * hw), dtype=act, device=dev)
+        ops.attention(q, o, cache.k, cache.v, g.block_tables, g.tiles, H, self.scale, 0, tiles_wide=g.tiles_wide, single_rows=g.single_rows,
+                      max_context=g.max_context, chunk=self.chunk)
+        if self.gated:
+            o = ops.head_gate(o, z[:, C:C + H], H, dv, torch.empty((T, H * dv), dtype=act, device=dev), head_stride=hw)
+        elif hw != dv:
+            o = ops.turn_back_gate(o, H, dv, torch.empty((T, H * dv), dtype=act, device=dev), head_stride=hw)
+        if accumulate_into is None:
+            return self.out(o, out_dtype=torch.float32)
+        self.out(o, residual=accumulate_into)
+
+
 @MIXERS.register("parallel_mixers")
 class ParallelMixers(Part):
     """Several mixers side by side that read the same rows; each result is normed over the width (without a mean, with a
     weight per column of its own) and the result is their mean.  branches: [(kind name, arguments)] of mixers that can
-    return their result as rows (`returns_rows`); every branch keeps a cache or state of its own, so a LayerCall of a
-    layer with this mixer lists one cache per branch."""
+    return their result as rows (`returns_rows`); every branch keeps caches or states of its own, so a LayerCall of a
+    layer with this mixer lists those of the first branch (its `cache_parts`), then the second's, and so on.  Branches that are
+    `joinable` (their product of h is their `proj`, a Linear without a bias whose weight_sources name its pieces) share one product."""
     returns_rows = True
 
     def __init__(self, width: int, eps: float, branches, norm_names):
@@ -504,22 +621,47 @@ class ParallelMixers(Part):
         for b in self.branches:
             if not getattr(b, "returns_rows", False):
                 raise TypeError(f"parallel_mixers: {type(b).__name__} cannot return its result as rows")
+        self.joint = None
+        if len(self.branches) > 1 and all(getattr(b, "joinable", False) for b in self.branches):
+            pieces = tuple(p for b in self.branches for p in b.proj.weight_sources)
+            self.joint = Linear(width, sum(c for _, c in pieces), " | ".join(b.proj.weight_name for b in self.branches), None,
+                                init_std=width ** -0.5, weight_sources=pieces)
+            for b in self.branches:
+                b.joined = True
         self.graph_safe = all(getattr(b, "graph_safe", False) for b in self.branches)
         self.libraries = tuple(sorted({"sequence"} | {lib for b in self.branches for lib in getattr(b, "libraries", ())}))
 
     def cache_parts(self):
-        return list(self.branches)
+        return [p for b in self.branches for p in b.cache_parts()]
+
+    def _each(self, h, ctx, caches):
+        """The branches' results, one after the other."""
+        at = col = 0
+        z = self.joint(h, out_dtype=torch.float32) if self.joint is not None else None
+        for b in self.branches:
+            n = len(b.cache_parts())
+            mine = caches[at:at + n]
+            at += n
+            more = {}
+            if z is not None:
+                more["z"] = z[:, col:col + b.proj.out_features]
+                col += b.proj.out_features
+            yield b.forward(h, ctx, mine if n > 1 else mine[0], accumulate_into=None, **more)
 
     def param_specs(self):
         specs = [ParamSpec(n, (self.width,), "vector", ("normal", 1.0, 0.1)) for n in self.norm_names]
         for b in self.branches:
             specs += b.param_specs()
+        if self.joint is not None:
+            specs += self.joint.param_specs()
         return specs
 
     def bind(self, tensors, runtime):
         super().bind(tensors, runtime)
         for b in self.branches:
             b.bind(tensors, runtime)
+        if self.joint is not None:
+            self.joint.bind(tensors)
         self.norms = [tensors[n] for n in self.norm_names]
 
     def forward_pair(self, h, ctx, caches):
@@ -527,7 +669,7 @@ class ParallelMixers(Part):
         result into the stream norms and halves both in its own kernel (ops.streams_write's `branches`); None otherwise."""
         if len(self.branches) != 2:
             return None
-        a, b = (br.forward(h, ctx, cache, accumulate_into=None) for br, cache in zip(self.branches, caches))
+        a, b = self._each(h, ctx, caches)
         return a, (b, self.norms[0], self.norms[1], self.eps)
 
     def forward(self, h, ctx, caches, accumulate_into):
@@ -537,6 +679,6 @@ class ParallelMixers(Part):
         if y is None:
             y = torch.zeros((h.shape[0], self.width), dtype=torch.float32, device=h.device)
         share = 1.0 / len(self.branches)
-        for b, w, cache in zip(self.branches, self.norms, caches):
-            ops.rmsnorm_add(b.forward(h, ctx, cache, accumulate_into=None), w, None, share, self.eps, y)
+        for r, w in zip(self._each(h, ctx, caches), self.norms):
+            ops.rmsnorm_add(r, w, None, share, self.eps, y)
         return y if accumulate_into is None else None

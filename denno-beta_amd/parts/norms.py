@@ -111,3 +111,21 @@ def following_norm(norm, x, out_dtype):
     if norm is None or type(norm) is not RMSNorm or norm.width != x.shape[1] or out_dtype is None:
         return None
     return norm.weight, norm.eps, torch.empty(x.shape, dtype=out_dtype, device=x.device)
+
+
+@NORMS.register("layernorm_of_sum")
+class SumLayerNorm(LayerNorm):
+    """The norm that stands behind the sum of the stream and a sublayer's result: x <- LayerNorm(alpha * x + y), in place.
+    `replace(x, y)` does it in one kernel, where y may also come as two branches whose normed mean it is, or as experts' rows with
+    their weights (ops.post_norm); `forward` is the norm alone."""
+    libraries = ("sequence",)
+
+    def __init__(self, width: int, eps: float, weight_name: str, bias_name=None, alpha: float = 1.0):
+        super().__init__(width, eps, weight_name, bias_name)
+        self.alpha = float(alpha)
+
+    def replace(self, x, y, out_dtype, branches=None, chosen=None):
+        """-> the rows as they then stand, in out_dtype (x itself where that is the stream's own precision)."""
+        out = None if out_dtype == x.dtype else torch.empty(x.shape, dtype=out_dtype, device=x.device)
+        ops.post_norm(x, y, self.alpha, self.weight, self.bias, self.eps, out=out, branches=branches, chosen=chosen)
+        return x if out is None else out

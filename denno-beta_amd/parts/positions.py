@@ -144,3 +144,44 @@ class RotaryPairs(Part):
         for t in (q, k):
             self.turn(t, t, ctx.positions, t.shape[1] // self.head_dim, self.head_dim)
         return q, k
+
+
+@POSITIONS.register("rotary_halves")
+class RotaryHalves(Part):
+    """Of a vector's first `dims` entries, entry i and entry i + dims / 2 form a pair (u, v) that the position p turns by the angle
+    p * base^(-2i / dims) / factor (factor: positions stretched evenly, 1: not): (u cos - v sin, v cos + u sin).  The rest of the
+    vector passes.  Angles are 32-bit; the frequencies are made once, in 64-bit, and rounded.  head_dim: as in RotaryPairs."""
+    graph_safe = True
+    rotates = True
+    halves = True      # (kernels that turn neighbouring pairs are no way for this encoding)
+    mag = 1.0
+    libraries = ("sequence",)
+
+    def __init__(self, dims: int, base: float, head_dim: int = 0, factor: float = 1.0):
+        if dims % 2 != 0 or dims < 0:
+            raise ValueError(f"rotary_halves: {dims} dimensions cannot be paired")
+        self.dims, self.base, self.head_dim, self.factor = int(dims), float(base), int(head_dim or dims), float(factor)
+        if self.dims > self.head_dim:
+            raise ValueError(f"rotary_halves: {dims} dimensions in vectors of {self.head_dim}")
+        if not self.factor > 0:
+            raise ValueError(f"rotary_halves: factor {factor}")
+
+    def frequencies(self):
+        """The pairs' frequencies, 64-bit, on the CPU."""
+        i = torch.arange(self.dims // 2, dtype=torch.float64)
+        return torch.tensor(self.base, dtype=torch.float64) ** (-2.0 * i / max(self.dims, 1)) / self.factor
+
+    def bind(self, tensors, runtime):
+        super().bind(tensors, runtime)
+        self.freq = self.frequencies().to(torch.float32).to(runtime.device)
+
+    def table(self):
+        return None
+
+    def turn(self, src, dst, positions, n_vec, width, **layout):
+        return ops.rotary(src, dst, positions, self.freq, n_vec, self.dims, width, halves=True, **layout)
+
+    def rotate(self, q, k, ctx):
+        for t in (q, k):
+            self.turn(t, t, ctx.positions, t.shape[1] // self.head_dim, self.head_dim)
+        return q, k

@@ -263,6 +263,90 @@ class ChannelDelta(Part):
         self.out(y, residual=accumulate_into)
 
 
+@MIXERS.register("gated_delta")
+class GatedDelta(Part):
+    """The delta rule with one decay per head and token.  q and k (n_qk_heads heads of head_dim) and v (n_heads of value_dim)
+    each pass a short causal convolution over time on every channel and silu; q and k are made unit vectors per head
+    (x / sqrt(sum x^2 + unit_eps)), q times query_scale; head h reads q and k of head h // (n_heads // n_qk_heads).  beta =
+    sigmoid(W_b h) and the decay g = exp(-exp(A_log_h) * softplus(W_a h + dt_bias)), one number each per head.  Per head:
+    S <- g S; e = beta (v - S^T k); S <- S + k e^T; o = S^T q.  Each head's o is divided by its root mean square, times a weight
+    per value column that the heads share, times silu(W_g h); then the output projection.  State: S in 32-bit and the
+    convolutions' last taps - 1 inputs."""
+    graph_safe = True
+    returns_rows = True
+    libraries = ("sequence",)
+    joinable = True      # (see parts.mixers.ParallelMixers)
+
+    def __init__(self, width: int, n_heads: int, n_qk_heads: int, head_dim: int, value_dim: int, taps: int, eps: float, names: dict,
+                 unit_eps: float = 1e-6, query_scale=None):
+        """names: q, k, v, g, b, a, o (matrices); q_conv, k_conv, v_conv ([channels, taps]); A_log, dt_bias, norm.
+        unit_eps: what is added to the sum of squares under the unit vectors' root; query_scale: what the unit queries are
+        multiplied by (None: head_dim^(-1/2))."""
+        if n_heads % n_qk_heads != 0:
+            raise ValueError(f"gated_delta: {n_heads} heads cannot share {n_qk_heads} heads of queries and keys")
+        if taps < 1:
+            raise ValueError(f"gated_delta: {taps} taps")
+        self.width, self.n_heads, self.n_qk_heads, self.head_dim, self.value_dim = width, n_heads, n_qk_heads, head_dim, value_dim
+        self.taps, self.eps, self.names, self.unit_eps = taps, eps, dict(names), float(unit_eps)
+        self.query_scale = head_dim ** -0.5 if query_scale is None else float(query_scale)
+        self.qk, self.vw = n_qk_heads * head_dim, n_heads * value_dim
+        self.channels = 2 * self.qk + self.vw
+        n = names
+        # one product for everything that reads h; its 32-bit result feeds the recurrence
+        pieces = ((n["q"], self.qk), (n["k"], self.qk), (n["v"], self.vw), (n["g"], self.vw), (n["b"], n_heads), (n["a"], n_heads))
+        self.proj = Linear(width, sum(c for _, c in pieces), n["q"] + "+k+v+g+b+a", None, init_std=width ** -0.5, weight_sources=pieces)
+        self.out = Linear(self.vw, width, n["o"], None, init_std=self.vw ** -0.5)
+        self.joined = False
+
+    def param_specs(self):
+        n = self.names
+        return ([] if self.joined else self.proj.param_specs()) + self.out.param_specs() + [
+            ParamSpec(n["q_conv"] + "+k+v", (self.channels, self.taps), "vector", ("normal", 0.0, 0.4),
+                      sources=((n["q_conv"], self.qk), (n["k_conv"], self.qk), (n["v_conv"], self.vw))),
+            ParamSpec(n["A_log"], (self.n_heads,), "vector", ("uniform", -2.0, 0.5)),
+            ParamSpec(n["dt_bias"], (self.n_heads,), "vector", ("normal", -1.0, 1.0)),
+            ParamSpec(n["norm"], (self.value_dim,), "vector", ("normal", 1.0, 0.1))]
+
+    def cache_spec(self):
+        return FixedState((self.n_heads * self.head_dim * self.value_dim + (self.taps - 1) * self.channels,))
+
+    def bind(self, tensors, runtime):
+        super().bind(tensors, runtime)
+        if not self.joined:
+            self.proj.bind(tensors)
+        self.out.bind(tensors)
+        n = self.names
+        self.conv = tensors[n["q_conv"] + "+k+v"].contiguous()
+        self.dt_bias, self.norm = tensors[n["dt_bias"]], tensors[n["norm"]]
+        self.rate = torch.exp(tensors[n["A_log"]].to(F32)).contiguous()
+
+    def forward(self, h, ctx, cache, accumulate_into, z=None):
+        """z: what `proj` gives for h, 32-bit, where a shared product has made it."""
+        act, T, dev = self.runtime.act_dtype, h.shape[0], h.device
+        qk, vw, C, H = self.qk, self.vw, self.channels, self.n_heads
+        n_state = H * self.head_dim * self.value_dim
+        state, past = cache.state[:, :n_state], cache.state[:, n_state:]
+        if z is None:
+            z = self.proj(h, out_dtype=F32)
+        single = ctx.single_rows and cache.writes
+        x = torch.empty((T, C), dtype=F32, device=dev)
+        ops.conv_heads(z[:, :C], self.conv, past, ctx.row_start, ctx.state_slots, x, 2 * self.n_qk_heads, self.head_dim,
+                       self.n_qk_heads, self.query_scale, 1.0, self.unit_eps, H, self.value_dim, move_on=single)
+        if self.taps > 1 and cache.writes and not single:
+            ops.history_update(z[:, :C], past, ctx.row_start, ctx.state_slots)
+        gate, b = C, C + vw
+        o = torch.empty((T, vw), dtype=F32, device=dev)
+        # (beta and the decay are made from their arguments inside the scan)
+        ops.state_scan(x[:, :qk], x[:, qk:2 * qk], x[:, 2 * qk:], z[:, b + H:b + 2 * H], None, state, ctx.row_start, ctx.state_slots, H,
+                       self.head_dim, self.value_dim, o, beta=z[:, b:b + H], qk_heads=self.n_qk_heads, beta_logits=True, w_rows=True,
+                       w_rate=self.rate, w_bias=self.dt_bias)
+        y = torch.empty((T, vw), dtype=act, device=dev)
+        ops.head_norm(o, self.norm, self.eps, y, H, gate=z[:, gate:gate + vw], gate_kind="silu")
+        if accumulate_into is None:
+            return self.out(y, out_dtype=F32)
+        self.out(y, residual=accumulate_into)
+
+
 @MIXERS.register("min_gru")
 class MinGRU(Part):
     """A recurrence of single numbers whose gates read the token alone: z = sigmoid(W_z h + b_z); u = W_x h + b_x; the

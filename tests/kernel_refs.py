@@ -133,7 +133,7 @@ def linear_norm_in(copy, stats, c1, c2, eps, w, out, epilogue="none", kv=None, n
 
 
 def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, window=0, tiles_wide=None,
-              single_rows=False, max_context=0, decode_waves=None, chunk=0, bias=None, sink=False, keep_first=0):
+              single_rows=False, max_context=0, decode_waves=None, chunk=0, bias=None, sink=False, keep_first=0, softcap=0.0):
     n_pages, hkv, ps, dh = k_pool.shape
     group = n_heads // hkv
     tl = tiles.cpu().tolist()
@@ -156,6 +156,8 @@ def attention(q, out, k_pool, v_pool, block_tables, tiles, n_heads, scale, windo
                 v = vf[pages, h // group, :, offs]
                 qv = q[row0 + i, h * dh:(h + 1) * dh].float()
                 sc = (k @ qv) * scale
+                if softcap > 0:
+                    sc = softcap * torch.tanh(sc / softcap)
                 if bias is not None:
                     sc = sc + bias[h][torch.clamp(pos - keys, max=bias.shape[1] - 1)]
                 if sink is not False:      # (a key without a value: score 0, or the head's own)
@@ -331,7 +333,8 @@ def conv_rows(h, w, hist, row_start, slots, out, identity=True, act=None, bias=N
     return out
 
 
-def conv_heads(h, w, hist, row_start, slots, out, n_unit, unit_dim, n_first, scale_first, scale_rest, eps, n_rest, rest_dim):
+def conv_heads(h, w, hist, row_start, slots, out, n_unit, unit_dim, n_first, scale_first, scale_rest, eps, n_rest, rest_dim,
+               move_on=False):
     conv_rows(h, w, hist, row_start, slots, out, identity=False, act="silu")
     T = out.shape[0]
     if n_unit:
@@ -339,6 +342,8 @@ def conv_heads(h, w, hist, row_start, slots, out, n_unit, unit_dim, n_first, sca
         scale = torch.cat([torch.full((n_first,), float(scale_first)), torch.full((n_unit - n_first,), float(scale_rest))])
         y = v / torch.sqrt((v * v).sum(dim=-1, keepdim=True) + eps) * scale[None, :, None]
         out[:, :n_unit * unit_dim] = y.reshape(T, -1)
+    if move_on and w.shape[1] > 1:
+        history_update(h[:, :w.shape[0]], hist, row_start, slots)
     return out
 
 
@@ -369,16 +374,17 @@ def shift_mix(h, hist, mu, row_start, slots, out):
 
 
 def rotary(src, dst, positions, freq, n_vec, dims, width, src_off=0, src_stride=None, dst_off=0, dst_stride=None, mag=1.0,
-           unit_eps=None):
+           unit_eps=None, halves=False):
     src_stride = width if src_stride is None else src_stride
     dst_stride = width if dst_stride is None else dst_stride
     ang = positions.float()[:, None] * freq[None, :]
     cos, sin = torch.cos(ang) * mag, torch.sin(ang) * mag
     for n in range(n_vec):
         vec = src[:, src_off + n * src_stride: src_off + n * src_stride + width].float().clone()
-        a, b = vec[:, 0:dims:2].clone(), vec[:, 1:dims:2].clone()
-        vec[:, 0:dims:2] = a * cos - b * sin
-        vec[:, 1:dims:2] = b * cos + a * sin
+        lo, hi = (slice(0, dims // 2), slice(dims // 2, dims)) if halves else (slice(0, dims, 2), slice(1, dims, 2))
+        a, b = vec[:, lo].clone(), vec[:, hi].clone()
+        vec[:, lo] = a * cos - b * sin
+        vec[:, hi] = b * cos + a * sin
         if unit_eps is not None:      # (rotary_runs' norm behind the turn)
             vec = vec / torch.sqrt((vec * vec).mean(dim=-1, keepdim=True) + unit_eps)
         dst[:, dst_off + n * dst_stride: dst_off + n * dst_stride + width] = vec.to(dst.dtype)
@@ -397,8 +403,10 @@ def gated(x, g, kind, out):
 
 
 def state_scan(r, k, v, w, u, state, row_start, slots, n_heads, dk, dv, out, read_after=False, key_from_decay=False, beta=None,
-               w_head=None, qk_heads=None, beta_logits=False, w_rows=False):
+               w_head=None, qk_heads=None, beta_logits=False, w_rows=False, w_rate=None, w_bias=None):
     H = n_heads
+    if w_rate is not None:
+        w = torch.exp(-w_rate * torch.nn.functional.softplus(w + (w_bias if w_bias is not None else 0.0)))
     if beta is not None and beta_logits:
         beta = torch.sigmoid(beta)
     G = H if qk_heads is None else qk_heads
@@ -565,7 +573,7 @@ def _turned(x, positions, freq, sign=1.0):
 
 
 def norm_turn_write(z, n_heads, n_kv, dk, dv, positions, q_out, slot_map, k_pool, v_pool, wq=None, wk=None, eps=None, q_scale=None,
-                    freq=None, v_freq=None, write=True):
+                    freq=None, v_freq=None, write=True, q_by_position=None):
     T, kept, ps = z.shape[0], k_pool.shape[3], k_pool.shape[2]
     zd = z.double()
     q = zd[:, :n_heads * dk].reshape(T, n_heads, dk)
@@ -577,6 +585,9 @@ def norm_turn_write(z, n_heads, n_kv, dk, dv, positions, q_out, slot_map, k_pool
     q, k, v = _turned(q, positions, freq), _turned(k, positions, freq), _turned(v, positions, v_freq)
     if q_scale is not None:
         q = q * q_scale.double()[:, None]
+    if q_by_position is not None:
+        coef, every = q_by_position
+        q = q * (1.0 + coef * torch.log(torch.floor((positions.double() + 1.0) / every) + 1.0))[:, None, None]
     pad = lambda x: torch.nn.functional.pad(x, (0, kept - x.shape[-1]))      # noqa: E731
     q_out.copy_(pad(q).reshape(T, n_heads * kept))
     if write:
@@ -585,6 +596,62 @@ def norm_turn_write(z, n_heads, n_kv, dk, dv, positions, q_out, slot_map, k_pool
                 k_pool[slot // ps, :, slot % ps, :] = pad(k[t]).to(k_pool.dtype)
                 v_pool[slot // ps, :, :, slot % ps] = pad(v[t]).to(v_pool.dtype)
     return q_out
+
+
+def conv_turn_write(z, n_heads, n_kv, dk, dv, w, hist, row_start, slots, positions, q_out, slot_map, k_pool, v_pool, wq, wk, eps, freq=None,
+                    write=True, move_on=False):
+    T, kept, ps = z.shape[0], k_pool.shape[3], k_pool.shape[2]
+    C, taps = w.shape
+    qw, kw = n_heads * dk, n_kv * dk
+    x = conv_rows(z, w, hist, row_start, slots, torch.zeros((T, C)), identity=False).double()
+    unit = lambda v: v / torch.sqrt((v * v).mean(dim=-1, keepdim=True) + eps)      # noqa: E731
+    q, k = unit(x[:, :qw]) * wq.double(), unit(x[:, qw:qw + kw]) * wk.double()
+
+    def turned(v):
+        v = v.clone()
+        if freq is not None and freq.numel():
+            m = freq.numel()
+            ang = (positions.float()[:, None] * freq[None, :]).double()[:, None, :]
+            a, b = v[..., :m].clone(), v[..., m:2 * m].clone()
+            v[..., :m], v[..., m:2 * m] = a * torch.cos(ang) - b * torch.sin(ang), b * torch.cos(ang) + a * torch.sin(ang)
+        return v
+    pad = lambda v: torch.nn.functional.pad(v, (0, kept - v.shape[-1]))      # noqa: E731
+    q_out.copy_(pad(turned(q.view(T, n_heads, dk))).reshape(T, n_heads * kept))
+    keys, values = pad(turned(k.view(T, n_kv, dk))), pad(x[:, qw + kw:].reshape(T, n_kv, dv))
+    if write:
+        for t, slot in enumerate(slot_map.tolist()):
+            if slot >= 0:
+                k_pool[slot // ps, :, slot % ps, :] = keys[t].to(k_pool.dtype)
+                v_pool[slot // ps, :, :, slot % ps] = values[t].to(v_pool.dtype)
+    if move_on and taps > 1:
+        history_update(z[:, :C], hist, row_start, slots)
+    return q_out
+
+
+def clamped_glu(z, limit, alpha, out):
+    n = out.shape[1]
+    g, u = torch.clamp(z[:, :n], max=limit), torch.clamp(z[:, n:], min=-limit, max=limit)
+    out.copy_(g * torch.sigmoid(alpha * g) * (u + 1.0))
+    return out
+
+
+def post_norm(x, y, alpha, weight, bias, eps, out=None, branches=None, chosen=None):
+    xd, r = x.double(), y.double()
+    if branches is not None:
+        y2, w1, w2, beps = branches
+        unit = lambda v: v.double() / torch.sqrt((v.double() ** 2).mean(dim=-1, keepdim=True) + beps)      # noqa: E731
+        r = 0.5 * (unit(y) * w1.double() + unit(y2) * w2.double())
+    if chosen is not None:
+        wts, ids, n = chosen
+        rows = torch.where((ids >= n)[:, :, None], xd[:, None, :], y.double().view(x.shape[0], wts.shape[1], -1))
+        r = (rows * wts.double()[:, :, None]).sum(dim=1)
+    u = alpha * xd + r
+    d = u - u.mean(dim=-1, keepdim=True)
+    v = d / torch.sqrt((d * d).mean(dim=-1, keepdim=True) + eps) * weight.double()
+    x.copy_(v if bias is None else v + bias.double())
+    if out is not None:
+        out.copy_(x)
+    return x
 
 
 def turn_back_gate(o, n_heads, dv, out, positions=None, freq=None, gate=None, head_stride=None):
@@ -628,7 +695,7 @@ def heads_linear(a, w, out, a_off=0, a_stride=None, o_off=0, o_stride=None):
     return out
 
 
-def moe_route(z, correction, top, ids, wts, score="softmax", renorm=True, n_experts=None, groups=1, keep=1, scale=1.0):
+def moe_route(z, correction, top, ids, wts, score="softmax", renorm=True, n_experts=None, groups=1, keep=1, scale=1.0, group_by="two"):
     if n_experts is not None:
         z = z[:, :n_experts]
     E = z.shape[1]
@@ -638,7 +705,7 @@ def moe_route(z, correction, top, ids, wts, score="softmax", renorm=True, n_expe
         c = choice[t].clone()
         if keep < groups:
             per = E // groups
-            gs = c.view(groups, per).topk(min(2, per), dim=-1).values.sum(dim=-1)
+            gs = c.view(groups, per).topk(1 if group_by == "best" else min(2, per), dim=-1).values.sum(dim=-1)
             closed = torch.ones(groups, dtype=torch.bool)
             for _ in range(keep):
                 g = int(torch.argmax(torch.where(closed, gs, torch.full_like(gs, -float("inf")))))
@@ -658,7 +725,7 @@ def moe_plan(ids, n_experts, offsets, order):
     flat = ids.reshape(-1).long()
     idx = torch.sort(flat, stable=True).indices
     order.copy_(idx.to(torch.int32))
-    counts = torch.bincount(flat, minlength=n_experts)
+    counts = torch.bincount(flat, minlength=n_experts)[:n_experts]      # (choices of n_experts or more sort behind the experts')
     offsets[0] = 0
     offsets[1:] = torch.cumsum(counts, 0).to(torch.int32)
 
@@ -691,8 +758,10 @@ def moe_down(y, order, offsets, w_down, out, dims=None):
             out[int(order[p])] = w_down[e].float() @ y[p].float()
 
 
-def moe_combine(out, wts, x, logits=False):
+def moe_combine(out, wts, x, logits=False, ids=None, n_experts=0, h=None):
     T = x.shape[0]
+    if ids is not None:
+        out = torch.where((ids >= n_experts).view(-1, 1), h.float().repeat_interleave(ids.shape[1], dim=0), out)
     if logits:
         wts = torch.sigmoid(wts)
     if wts is None:

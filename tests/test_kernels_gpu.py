@@ -1146,3 +1146,44 @@ def test_attention_in_a_window_that_keeps_first_keys_with_a_sink_per_head(dtype,
         rows = torch.zeros(T, H * dh, dtype=dtype, device=DEV)
         ops().attention(q, rows, k, v, bt, tiles, H, scale, window, **kw)
         assert torch.equal(rows, out)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("H,Hkv,dh,ps", [(4, 2, 64, 16), (2, 1, 80, 16), (3, 3, 96, 32), (2, 2, 16, 16), (2, 1, 256, 16), (5, 1, 128, 16), (3, 1, 24, 8)])
+def test_attention_with_a_soft_cap(dtype, H, Hkv, dh, ps):
+    """Every kernel that `attention` may take, with scores well beyond the cap: a cap that is lost, or put before the scale, moves
+    the weights a lot.  Alone, with chunks whose pages behind are given back, and with a bias behind the cap."""
+    scale = 3 / math.sqrt(dh)
+    bias = torch.randn(H, 40, generator=torch.Generator().manual_seed(dh)).to(DEV)
+
+    def case(seq_lens, new_rows, seed, chunk):
+        q, k, v, bt, tiles, T = paged_case(seq_lens, new_rows, H, Hkv, dh, ps, dtype, seed=seed)
+        bt = bt.clone()
+        if chunk:
+            for s, (total, new) in enumerate(zip(seq_lens, new_rows)):
+                bt[s, :(total - new) // chunk * chunk // ps] = -1
+        return q[:, :H * dh], k, v, bt, tiles, T
+    for kw in (dict(softcap=1.5), dict(softcap=3.0, chunk=50), dict(softcap=1.0, bias=bias), dict(softcap=20.0)):
+        seq_lens, new_rows = [300, 70, 133, 1, 430], [1, 70, 21, 1, 300]
+        q, k, v, bt, tiles, T = case(seq_lens, new_rows, dh + H, kw.get("chunk", 0))
+        want = R.attention(q, torch.zeros(T, H * dh, device=DEV), k, v, bt, tiles, H, scale, 0, **kw)
+        if kw["softcap"] < 2 and "chunk" not in kw:      # (the test's own check: the cap shows)
+            uncapped = R.attention(q, torch.zeros(T, H * dh, device=DEV), k, v, bt, tiles, H, scale, 0, **{n: x for n, x in kw.items() if n != "softcap"})
+            assert (uncapped - want).abs().max() > 0.2
+        for wide in (None, paged_case.wide):
+            out = torch.zeros(T, H * dh, dtype=dtype, device=DEV)
+            ops().attention(q, out, k, v, bt, tiles, H, scale, 0, tiles_wide=wide, **kw)
+            assert torch.allclose(out.float(), want, **TOL[dtype]), ("portions", wide is not None, kw.keys())
+        seq_lens = [1, 49, 50, 51, 256, 257, 700, 1024]
+        q, k, v, bt, tiles, T = case(seq_lens, [1] * len(seq_lens), dh, kw.get("chunk", 0))
+        want = R.attention(q, torch.zeros(T, H * dh, device=DEV), k, v, bt, tiles, H, scale, 0, **kw)
+        for waves in (None, 4, 8, 16):
+            if waves and (dtype == torch.float32 or dh % 16 or ps % 16 or waves > (16 if dh <= 64 else 8 if dh <= 128 else 4)):
+                continue
+            out = torch.zeros(T, H * dh, dtype=dtype, device=DEV)
+            ops().attention(q, out, k, v, bt, tiles, H, scale, 0, tiles_wide=paged_case.wide, single_rows=True, max_context=1024, decode_waves=waves, **kw)
+            assert torch.allclose(out.float(), want, **TOL[dtype]), ("single rows", waves, kw.keys())
+        if dtype == torch.float32 and dh % 16 == 0:      # the kernels for single rows and for portions: the same bits
+            rows = torch.zeros(T, H * dh, dtype=dtype, device=DEV)
+            ops().attention(q, rows, k, v, bt, tiles, H, scale, 0, **kw)
+            assert torch.equal(rows, out)

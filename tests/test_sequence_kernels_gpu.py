@@ -850,3 +850,196 @@ def test_rows_of_a_table_stored_as_several_copies(dtype, E):
         assert torch.equal(out, (tables[0][ids[0].long()].float() * 2.0).expand(copies, T, E))
         ops.embed_sum([(tables[0], ids[0], 1.0), (tables[1], ids[1], 1.0)], out)
         assert torch.equal(out, (tables[0][ids[0].long()].float() + tables[1][ids[1].long()].float()).expand(copies, T, E))
+
+
+# ---- kernels behind a norm of sums, a pair of mixers and a router with outputs that return their input -------------------
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("T,width", [(1, 24), (9, 511), (5, 1000), (300, 1024), (3, 2000), (4, 4096), (2, 4500)])
+def test_a_norm_behind_the_sum(dtype, T, width):
+    """Every width's kernel: a plain result, two branches, a router's choices some of which give the row back; the rows of y that
+    such a choice has no use for hold no numbers and must not be read."""
+    x, y, y2 = torch.randn(T, width, device=DEV) * 2 + 0.5, torch.randn(T, width + 3, device=DEV)[:, :width], torch.randn(T, width, device=DEV) * 5
+    g, b, w1, w2 = (torch.randn(width, device=DEV) for _ in range(4))
+    out = lambda: torch.empty(T, width, dtype=dtype, device=DEV)      # noqa: E731
+    both("post_norm", lambda: (x.clone(), y, 2.5, g, None, 1e-5, out()), [0], torch.float32)
+    both("post_norm", lambda: (x.clone(), y, 0.7, g, b, 1e-2, out()), [0, 6], dtype)
+    both("post_norm", lambda: (x.clone(), y, 1.0, g, None, 1e-6, None), [0], torch.float32)
+    both("post_norm", lambda: (x.clone(), y, 1.5, g, None, 1e-5, out(), (y2, w1, w2, 1e-4)), [0, 6], dtype)
+    for top, n in ((1, 3), (4, 5), (6, 2), (3, 0)):
+        rows = torch.randn(T * top, width, device=DEV)
+        ids = torch.randint(0, 8, (T, top), dtype=torch.int32, device=DEV)
+        rows[(ids >= n).view(-1)] = float("nan")
+        wts = torch.rand(T, top, device=DEV)
+        both("post_norm", lambda: (x.clone(), rows, 2.0, g, None, 1e-5, out(), None, (wts, ids, n)), [0, 6], dtype)
+        # the same sum through moe_combine, the identity from the rows as the experts read them
+        a, s = x.clone(), torch.zeros(T, width, device=DEV)
+        ops.moe_combine(rows, wts, s, ids=ids, n_experts=n, h=a)
+        c = x.clone()
+        ops.post_norm(c, s, 2.0, g, None, 1e-5)
+        ops.post_norm(a, rows, 2.0, g, None, 1e-5, chosen=(wts, ids, n))
+        close(c, a)
+
+
+@pytest.mark.parametrize("T,E,extra,top,groups,keep", [(1, 4, 2, 2, 3, 2), (70, 12, 4, 4, 4, 3), (33, 60, 4, 3, 8, 1), (40, 5, 1, 6, 1, 1), (9, 2, 6, 3, 4, 2)])
+def test_choices_that_are_none_of_the_experts(T, E, extra, top, groups, keep):
+    """A router with outputs behind the experts': the groups judged by their best output; the plan leaves those choices out, and
+    the experts' products and the weighted sum take the rest."""
+    dtype, ff, width = torch.float32, 12, 20
+    n = E + extra
+    z, corr = torch.randn(T, n, device=DEV) * 2, torch.randn(n, device=DEV) * 0.3 - 0.2      # (choice scores of both signs)
+    ids, wts = torch.zeros(T, top, dtype=torch.int32, device=DEV), torch.zeros(T, top, device=DEV)
+    ops.moe_route(z, corr, top, ids, wts, renorm=False, groups=groups, keep=keep, group_by="best")
+    hi, hw = torch.zeros(T, top, dtype=torch.int32), torch.zeros(T, top)
+    ref.moe_route(z.cpu(), corr.cpu(), top, hi, hw, renorm=False, groups=groups, keep=keep, group_by="best")
+    assert torch.equal(ids.cpu(), hi)
+    close(wts, hw)
+    if T >= 9:
+        assert bool((ids >= E).any()) and bool((ids < E).any())
+    if keep < groups and T > 30:      # (judging groups by their two best would choose otherwise somewhere)
+        other = torch.zeros_like(hi)
+        ref.moe_route(z.cpu(), corr.cpu(), top, other, torch.zeros_like(hw), renorm=False, groups=groups, keep=keep)
+        assert not torch.equal(other, hi)
+    offsets = torch.full((E + 1,), -7, dtype=torch.int32, device=DEV)
+    order = torch.full((T * top,), -7, dtype=torch.int32, device=DEV)
+    ops.moe_plan(ids, E, offsets, order)
+    ho, hr = torch.zeros(E + 1, dtype=torch.int32), torch.zeros(T * top, dtype=torch.int32)
+    ref.moe_plan(hi, E, ho, hr)
+    used = int(ho[E])
+    assert used == int((hi < E).sum()) and torch.equal(offsets.cpu(), ho) and torch.equal(order.cpu()[:used], hr[:used])
+    assert bool((order.cpu()[used:] == -7).all())
+    h = torch.randn(T, width, device=DEV)
+    wu, wd = torch.randn(E, ff, width, device=DEV) / width ** 0.5, torch.randn(E, width, ff, device=DEV)
+    y, out = torch.zeros(T * top, ff, device=DEV), torch.full((T * top, width), float("nan"), device=DEV)
+    ops.moe_up(h, order, offsets, top, None, wu, 0.0, 1.0, y, kind="relu2")
+    ops.moe_down(y, order, offsets, wd, out)
+    x = torch.zeros(T, width, device=DEV)
+    ops.moe_combine(out, wts, x, ids=ids, n_experts=E, h=h.to(dtype))
+    want = torch.zeros(T, width, dtype=torch.float64)
+    for t in range(T):
+        for c in range(top):
+            e, row = int(hi[t, c]), h[t].cpu().double()
+            r = row if e >= E else wd[e].cpu().double() @ torch.relu(wu[e].cpu().double() @ row) ** 2
+            want[t] += float(hw[t, c]) * r
+    close(x / want.abs().max().float(), want.float() / want.abs().max().float())
+
+
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("T,n", [(1, 7), (5, 64), (300, 50), (9, 1030), (3, 2048)])
+def test_a_clamped_gate_of_both_halves_of_a_row(dtype, T, n):
+    z = torch.randn(T, 2 * n + 4, device=DEV)[:, :2 * n] * 4
+    for limit, alpha in ((1.5, 1.702), (7.0, 1.0)):
+        both("clamped_glu", lambda: (z, limit, alpha, torch.zeros(T, n, dtype=dtype, device=DEV)), [3], dtype)
+
+
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("dims,width", [(8, 8), (6, 10), (0, 4), (64, 96)])
+def test_rotary_of_halves(dtype, dims, width):
+    T, n = 5, 3
+    src = torch.randn(T, n * width + 2, device=DEV).to(dtype)
+    pos = torch.randint(0, 3000, (T,), dtype=torch.int32, device=DEV)
+    freq = torch.logspace(0, -3, dims // 2, device=DEV) if dims else torch.empty(0, device=DEV)
+    got = ops.rotary(src, torch.zeros(T, n * width, dtype=dtype, device=DEV), pos, freq, n, dims, width, halves=True)
+    want = ref.rotary(src.cpu(), torch.zeros(T, n * width, dtype=dtype), pos.cpu(), freq.cpu(), n, dims, width, halves=True)
+    close(got, want, dtype)
+
+
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("lengths", [[1, 7, 2, 3], [1, 1, 1, 1], [300, 2, 1, 40]])
+@pytest.mark.parametrize("taps", [1, 3, 4, 6])
+@pytest.mark.parametrize("H,G,dk,dv,dims,ps", [(4, 2, 16, 16, 16, 8), (3, 1, 10, 21, 6, 16), (5, 5, 48, 24, 0, 16), (12, 4, 96, 80, 64, 16), (2, 2, 256, 256, 256, 32)])
+def test_queries_keys_and_values_convolved_normed_whole_turned_and_kept(dtype, lengths, taps, H, G, dk, dv, dims, ps):
+    row_start, slots, T = tables(lengths, [2, 0, -1, 3])
+    C = (H + G) * dk + G * dv
+    kept = -(-max(dk, dv) // 16) * 16
+    z = torch.randn(T, C + 5, device=DEV)
+    w = torch.randn(C, taps, device=DEV)
+    hist = torch.randn(5, (taps - 1) * C + 3, device=DEV)
+    wq, wk = torch.randn(H * dk, device=DEV), torch.randn(G * dk, device=DEV)
+    pos = torch.randint(0, 4000, (T,), dtype=torch.int32, device=DEV)
+    freq = torch.logspace(0, -3, dims // 2, device=DEV) if dims else None
+    pages = -(-T // ps) + 2
+    slot_map = torch.randperm(pages * ps, device=DEV)[:T].int()
+    slot_map[0] = -1
+    k0, v0 = torch.zeros(pages, G, ps, kept, dtype=dtype, device=DEV), torch.zeros(pages, G, kept, ps, dtype=dtype, device=DEV)
+    single = T == len(lengths)
+    real = [t for s, (a, n) in enumerate(zip(row_start.tolist(), lengths)) for t in range(a, a + n) if int(slots[s]) >= 0]
+    dead = [t for t in range(T) if t not in real]
+    for write, move_on in ((True, False), (False, False)) + (((True, True),) if single else ()):
+        q, k, v, hs = torch.full((T, H * kept), 7.0, dtype=dtype, device=DEV), k0.clone(), v0.clone(), hist.clone()
+        # (a padding row has no place in the cache)
+        sm = slot_map.clone()
+        sm[dead] = -1
+        ops.conv_turn_write(z, H, G, dk, dv, w, hs[:, :(taps - 1) * C], row_start, slots, pos, q, sm, k, v, wq, wk, 1e-5, freq, write, move_on)
+        hq, hk, hv, hh = torch.zeros(T, H * kept, dtype=dtype), k0.cpu().clone(), v0.cpu().clone(), hist.cpu().clone()
+        ref.conv_turn_write(z.cpu(), H, G, dk, dv, w.cpu(), hh[:, :(taps - 1) * C], row_start.cpu(), slots.cpu(), pos.cpu(), hq, sm.cpu(), hk, hv,
+                            wq.cpu(), wk.cpu(), 1e-5, None if freq is None else freq.cpu(), write, move_on)
+        # (angles of thousands of turns: sin and cos of the device and the host part in their last bits)
+        close(q[real], hq[real], dtype, "q")
+        close(k, hk, dtype, "k"), close(v, hv, dtype, "v")
+        assert not bool(q[dead].any()) and torch.equal(hs.cpu(), hh)
+        assert move_on or torch.equal(hs, hist)
+    with pytest.raises(Exception):
+        ops.conv_turn_write(z, H, G, dk, dv, w, hist[:, :(taps - 1) * C], row_start, slots, pos, q, slot_map, k, v, wq, wk, 1e-5,
+                            torch.ones(dk // 2 + 1, device=DEV))
+
+
+@pytest.mark.parametrize("taps", [1, 2, 4, 7])
+def test_heads_convolved_and_the_history_moved_on_in_one_launch(taps):
+    row_start, slots, T = tables([1, 1, 1, 1, 1], [2, 0, -1, 3, 6])
+    n_unit, unit_dim, n_rest, rest_dim = 4, 10, 3, 70
+    C = n_unit * unit_dim + n_rest * rest_dim
+    z, w, hist = torch.randn(T, C + 5, device=DEV), torch.randn(C, taps, device=DEV), torch.randn(7, (taps - 1) * C + 2, device=DEV)
+    a, b = hist.clone(), hist.clone()
+    one, two = torch.zeros(T, C, device=DEV), torch.zeros(T, C, device=DEV)
+    args = lambda h, out: (z[:, :C], w, h[:, :(taps - 1) * C], row_start, slots, out, n_unit, unit_dim, 2, 0.3, 1.0, 1e-6, n_rest, rest_dim)   # noqa: E731
+    ops.conv_heads(*args(a, one), move_on=True)
+    ops.conv_heads(*args(b, two))
+    if taps > 1:
+        ops.history_update(z[:, :C], b[:, :(taps - 1) * C], row_start, slots)
+    assert torch.equal(one, two) and torch.equal(a, b)
+    close(one, ref.conv_heads(*[x.cpu() if isinstance(x, torch.Tensor) else x for x in args(hist, torch.zeros(T, C, device=DEV))]))
+
+
+@pytest.mark.parametrize("dk,dv,heads,qk_heads", [(16, 16, 2, 2), (48, 32, 4, 2), (5, 70, 1, 1), (64, 64, 4, 1), (100, 9, 2, 2), (130, 20, 3, 1),
+                                                  (32, 12, 6, 3), (128, 36, 1, 1), (252, 8, 1, 1), (64, 128, 2, 2), (6, 10, 2, 1)])
+@pytest.mark.parametrize("lengths", [[1, 12, 40], [1, 2, 1], [37, 5, 16]])
+def test_delta_rule_with_one_decay_a_row_and_head(dk, dv, heads, qk_heads, lengths):
+    """The decay given as it is, or as the argument that it is made from inside the scan; the same as a decay per channel."""
+    row_start, slots, T = tables(lengths, [2, -1, 0])
+    r, k = torch.randn(T, qk_heads * dk, device=DEV), torch.randn(T, qk_heads * dk, device=DEV)
+    k = torch.nn.functional.normalize(k.reshape(T, qk_heads, dk), dim=-1).reshape(T, -1).contiguous()
+    v = torch.randn(T, heads * dv, device=DEV)
+    zs = torch.randn(T, 2 * heads + 3, device=DEV) * 2                       # columns of wider rows
+    zb, zw = zs[:, :heads], zs[:, heads:2 * heads]
+    rate, bias = torch.rand(heads, device=DEV) + 0.1, torch.randn(heads, device=DEV)
+    state = torch.randn(3, heads * dk * dv + 11, device=DEV)
+
+    def make(w, w_rate, w_bias):
+        return lambda: (r, k, v, w, None, state.clone()[:, :heads * dk * dv], row_start, slots, heads, dk, dv, torch.zeros(T, heads * dv, device=DEV),
+                        False, False, zb, None, qk_heads, True, True, w_rate, w_bias)
+    both("state_scan", make(zw, rate, bias), [5, 11])
+    both("state_scan", make(zw, rate, None), [5, 11])
+    w = torch.exp(-rate * torch.nn.functional.softplus(zw + bias))
+    both("state_scan", make(w, None, None), [5, 11])
+    outs = []
+    for wide in (False, True):
+        st, o = state.clone()[:, :heads * dk * dv], torch.zeros(T, heads * dv, device=DEV)
+        ops.state_scan(r, k, v, w.repeat_interleave(dk, dim=1).contiguous() if wide else w, None, st, row_start, slots, heads, dk, dv, o, beta=zb,
+                       qk_heads=qk_heads, beta_logits=True, w_rows=not wide)
+        outs.append((st, o))
+    close(outs[0][0], outs[1][0]), close(outs[0][1], outs[1][1])
+
+
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("every", [1, 7, 128, 2.5])
+def test_queries_times_a_temperature_of_their_position(dtype, every):
+    T, H, G, dk, dv, ps = 40, 3, 1, 24, 40, 16
+    z = torch.randn(T, (H + G) * dk + G * dv, device=DEV)
+    # (the positions on both sides of where the temperature steps, and a large one)
+    steps = [int(m * every) for m in (1, 2, 3, 10)]
+    pos = torch.tensor(([0] + [max(0, s + d) for s in steps for d in (-2, -1, 0)] + [60000] * T)[:T], dtype=torch.int32, device=DEV)
+    k, v = torch.zeros(4, G, ps, 48, dtype=dtype, device=DEV), torch.zeros(4, G, 48, ps, dtype=dtype, device=DEV)
+    slot_map = torch.arange(T, dtype=torch.int32, device=DEV)
+    wq, wk = torch.randn(dk, device=DEV), torch.randn(dk, device=DEV)
+    both("norm_turn_write", lambda: (z, H, G, dk, dv, pos, torch.zeros(T, H * 48, dtype=dtype, device=DEV), slot_map, k, v, wq, wk, 1e-5, None, None,
+                                     None, True, (0.3, every)), [6, 8, 9], dtype)
