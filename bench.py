@@ -34,6 +34,11 @@ decode steps and prefill (`fp32`).  Peaks are the published ones of MI355X.
                                                              latent attention in a window, both again; a dense feed-forward, then
                                                              sixteen experts; the stream in four copies) beside four Nigilorn layers
                                                              of the same kinds and sizes: prefill and decode
+    python bench.py --only pepapel [--width 1024] [--kernel-times]   four Pepapel layers (a pair of attention in chunks and a delta rule,
+                                                             attention with a soft cap, the pair twice; a dense feed-forward, then
+                                                             sixteen experts and four outputs that return their input) beside
+                                                             seven Pafivik layers that hold the same mixers and as many
+                                                             feed-forwards: prefill and decode
 """
 import argparse
 import json
@@ -203,8 +208,8 @@ def main():
     ap.add_argument("--shape", choices=["xl", "large", "medium"], default=None,
                     help="--only decode / prefill / replay: the layer sizes of BASELINE.json's configs[2], [3] or [4] "
                          "(default xl; for replay medium)")
-    ap.add_argument("--width", type=int, default=0, help="--only ridopel, pafivik, dogalorn, nigilorn, fikupel: one width instead of 1,024 and 2,048")
-    ap.add_argument("--only", choices=["decode", "prefill", "serving", "replay", "ridopel", "pafivik", "dogalorn", "nigilorn", "fikupel"], default=None,
+    ap.add_argument("--width", type=int, default=0, help="--only ridopel, pafivik, dogalorn, nigilorn, fikupel, pepapel: one width instead of 1,024 and 2,048")
+    ap.add_argument("--only", choices=["decode", "prefill", "serving", "replay", "ridopel", "pafivik", "dogalorn", "nigilorn", "fikupel", "pepapel"], default=None,
                     help="run one workload and print a short line (decode, prefill: for profiling; serving: "
                          "BASELINE.json's configs[3], GPT-2 Large shape, 64 requests through the scheduler; replay: "
                          "configs[4], GPT-2 Medium shape, against the plain implementation)")
@@ -224,6 +229,8 @@ def main():
         return nigilorn(a)
     if a.only == "fikupel":
         return fikupel(a)
+    if a.only == "pepapel":
+        return pepapel(a)
     if a.only == "replay":
         a.shape = a.shape or "medium"      # (configs[4] as written; --shape xl: the same replay at configs[2]'s sizes)
         return replay(a)
@@ -407,6 +414,44 @@ def fikupel_configs(width, layers=4, vocab=32000, positions=2048):
                                                     rot=dict(base=10000.0, dims=32, scaling=stretch)))
     nig = dict(four(att(stretch), nlat, moe(scale=2.5, groups=dict(count=4, keep=2))), architecture="Nigilorn")
     return fik, nig
+
+
+def pepapel_configs(width, layers=4, vocab=32000, positions=2048):
+    """-> (a Pepapel config, a Pafivik config) of the same width, vocabulary and positions, with the same mixers and as many
+    feed-forwards.  The Pepapel layers: a pair of attention in chunks of 512 (heads of 64, a key head for every four, all dimensions
+    turned, four taps) and a delta rule (heads of 64 keys x 128 values, half as many heads of queries and keys, four taps);
+    attention over everything (the same heads, a temperature, a soft cap); the pair twice.  The first layer has a dense
+    feed-forward of four times the width (gated, with biases), the others sixteen experts of the model's width without a gate, in
+    groups with four outputs that return their input, two choices a token.  The Pafivik layers: for every pair an attention layer
+    without a feed-forward and a channel_delta layer with one, for every attention an attention layer; dense feed-forwards of
+    four times the width, or sixteen gated experts of the model's width of which a token uses two."""
+    H, Hd = width // 64, width // 128
+    ff = dict(kind="dense", ff=4 * width)
+    heads = dict(heads=H, kv_heads=max(1, H // 4), dim=64, vdim=64, scale=0.125)
+    delta = dict(heads=Hd, kv_heads=max(1, Hd // 2), dim=64, vdim=128, conv=4)
+    moe = dict(kind="moe", expert=dict(ff=width), router=dict(experts=16, identity=4, top=2, groups=dict(count=4, keep=3)))
+    pair = dict(type="parallel", mixer=dict(left=dict(heads, conv=4, mask=dict(size=512), rot=dict(base=10000.0, dims=64, scaling=dict(factor=2.0))),
+                                            right=delta))
+    att = dict(type="attention", mixer=dict(heads, q_temp=dict(coef=0.1, every=256), softcap=30.0))
+    kinds = [dict(pair, mlp=dict(ff, limit=7.0)), dict(att, mlp=moe), dict(pair, mlp=moe), dict(pair, mlp=moe)]
+    kinds = [kinds[i % 4] for i in range(layers)]
+    common = dict(vocab=vocab, width=width, norm=dict(eps=1e-5), embedding=dict(scale=1.0), max_positions=positions, n_positions=positions, vocab_size=vocab)
+    pep = dict(common, architecture="Pepapel", postln_alpha=2.5, layers=kinds)
+    pmoe = dict(kind="moe", expert=dict(ff=width), router=dict(experts=16, top=2))
+    patt = dict(type="attention", mixer=dict(heads, rot=dict(base=10000.0, dims=64)))
+    pdelta = dict(type="channel_delta", mixer=dict(delta, decay_rank=64, gate_rank=64))
+    others = []
+    for layer in kinds:
+        mlp = ff if layer["mlp"]["kind"] == "dense" else pmoe
+        others += [dict(patt, mlp=None), dict(pdelta, mlp=mlp)] if layer["type"] == "parallel" else [dict(patt, mlp=mlp)]
+    return pep, dict(common, architecture="Pafivik", residual_mult=0.5, layers=others)
+
+
+def pepapel(a):
+    """Prefill and decode steps of four Pepapel layers beside seven Pafivik layers with the same mixers and as many feed-forwards
+    (the closest of the framework's models: attention with grouped key heads, a delta rule with short convolutions, experts); with
+    --kernel-times each model's kernels."""
+    return side_by_side(a, ("pepapel", "pafivik"), pepapel_configs)
 
 
 def fikupel(a):
