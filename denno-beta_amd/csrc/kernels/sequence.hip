@@ -202,13 +202,13 @@ __global__ __launch_bounds__(64) void conv_heads_kernel(const float* h, size_t l
   const int dim = unit ? unit_dim : rest_dim;
   const int c0 = unit ? vec * unit_dim : n_unit * unit_dim + (vec - n_unit) * rest_dim;
   float* dst = out + static_cast<size_t>(t) * ldo + c0;
-  const int s = request_of(row_start, S, t);
+  const int s = move_on ? t : request_of(row_start, S, t);      // (a step of single rows: request t is row t)
   const int slot = slots[s];
-  if (slot < 0 || t >= row_start[S]) {      // a padding row: zeros
+  if (slot < 0 || (!move_on && t >= row_start[S])) {      // a padding row: zeros
     for (int j = lane; j < dim; j += 64) dst[j] = 0.f;
     return;
   }
-  const int row0 = row_start[s], i = t - row0;
+  const int row0 = move_on ? t : row_start[s], i = t - row0;
   float* past = hist + static_cast<size_t>(slot) * hist_stride;
   float ss = 0.f;
   for (int j = lane; j < dim; j += 64) {
@@ -1412,12 +1412,13 @@ __global__ __launch_bounds__(256) void norm_turn_write_kernel(NormTurnArgs a) {
 }
 
 // ---- the same behind a short convolution, with norms over all heads at once -------------------------------------------
-// A row of z is [q: H x dk | k: G x dk | v: G x dv].  Every channel passes a short causal convolution over time (no activation; w
-// [channels][taps], the last tap the row's own; rows before the step's from the history); q and k are each divided by their
+// A row of z is [q: H x dk | k: G x dk | v: G x dv].  Every channel passes a short causal convolution over time (no activation; the
+// last tap the row's own; rows before the step's from the history); q and k are each divided by their
 // root mean square as one vector over all heads and weighed entry by entry (wq: H x dk numbers, wk: G x dk); the first `dims`
 // entries of every head's q and k are turned by position * freq in pairs (i, i + dims / 2); then to their places as
-// norm_turn_write_kernel puts them.  move_on as in conv_heads_kernel.  One workgroup a row, the row in LDS; how many threads it
-// has follows from the sizes alone, so a row's sums do not depend on the step.
+// norm_turn_write_kernel puts them.  move_on as in conv_heads_kernel.  w is held [taps][channels] here.  One workgroup a row, the
+// row in LDS.  The squares are summed by runs of 64 channels (runs of q's and of k's, a wave a run), the runs in ascending order: the
+// same sums for any number of threads, so a row does not depend on the step.  LPV lanes share a vector on the way out.
 struct ConvTurnArgs {
   const float* z;
   size_t ldz;
@@ -1440,15 +1441,18 @@ struct ConvTurnArgs {
   int page_size, dt, write, move_on;
 };
 
-template <int THREADS>
+constexpr int CONV_TURN_RUNS = 256;      // runs of 64 channels of q and k in a row
+
+template <int THREADS, int LPV>
 __global__ __launch_bounds__(THREADS) void conv_turn_write_kernel(ConvTurnArgs a) {
   extern __shared__ float vals[];      // [channels]
-  __shared__ float cs[128], sn[128], sums[2][THREADS / 64];
-  const int t = blockIdx.x, tid = threadIdx.x;
+  __shared__ float cs[128], sn[128], sums[CONV_TURN_RUNS];
+  const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63;
   const int qw = a.H * a.dk, kw = a.G * a.dk, C = qw + kw + a.G * a.dv, half = a.dims / 2, pairs = a.kept / 2;
-  const int s = request_of(a.row_start, a.S, t);
-  const int slot = a.slots[s], row0 = a.row_start[s];
-  if (slot < 0 || t >= a.row_start[a.S]) {      // a padding row: zeros, so that what follows works on numbers
+  // (a step of single rows: request t is row t)
+  const int s = a.move_on ? t : request_of(a.row_start, a.S, t);
+  const int slot = a.slots[s], row0 = a.move_on ? t : a.row_start[s];
+  if (slot < 0 || (!a.move_on && t >= a.row_start[a.S])) {      // a padding row: zeros, so that what follows works on numbers
     for (int i = tid; i < a.H * pairs; i += THREADS) store_pair(a.q_out, t * a.ldq + 2 * i, a.dt, 0.f, 0.f);
     return;
   }
@@ -1458,48 +1462,76 @@ __global__ __launch_bounds__(THREADS) void conv_turn_write_kernel(ConvTurnArgs a
     sincosf(ang, &sn[tid], &cs[tid]);
   }
   float* past = a.hist + static_cast<size_t>(slot) * a.hist_stride;
-  float sq = 0.f, sk = 0.f;
-  for (int c = tid; c < C; c += THREADS) {
-    const float v = conv_channel(a.z + static_cast<size_t>(row0) * a.ldz, a.ldz, past, C, a.w + static_cast<size_t>(c) * a.taps, a.taps, t - row0, c);
-    if (a.move_on) history_move_on(past, C, a.taps, c, a.z[static_cast<size_t>(t) * a.ldz + c]);
-    if (c < qw) sq = fmaf(v, v, sq);
-    else if (c < qw + kw) sk = fmaf(v, v, sk);
-    vals[c] = v;
-  }
-  sq = wave_sum(sq), sk = wave_sum(sk);
-  if ((tid & 63) == 0) sums[0][tid >> 6] = sq, sums[1][tid >> 6] = sk;
-  __syncthreads();
-  sq = sk = 0.f;
+  const float* rows = a.z + static_cast<size_t>(row0) * a.ldz;
+  const int i = t - row0, taps = a.taps;
+  const int runs_q = (qw + 63) / 64, runs = runs_q + (kw + 63) / 64, all = runs + (a.G * a.dv + 63) / 64;
+  for (int run = __builtin_amdgcn_readfirstlane(tid >> 6); run < all; run += THREADS / 64) {
+    const int begin = run < runs_q ? 64 * run : run < runs ? qw + 64 * (run - runs_q) : qw + kw + 64 * (run - runs);
+    const int end = run < runs_q ? qw : run < runs ? qw + kw : C;
+    const int c = begin + lane;
+    float v = 0.f;
+    if (c < end) {
+      for (int q0 = 0; q0 < taps; q0 += 4) {
+        float x[4], wt[4];
 #pragma unroll
-  for (int u = 0; u < THREADS / 64; ++u) sq += sums[0][u], sk += sums[1][u];
-  const float iq = 1.0f / sqrtf(sq / static_cast<float>(qw) + a.eps), ik = 1.0f / sqrtf(sk / static_cast<float>(kw) + a.eps);
-  for (int c = tid; c < qw + kw; c += THREADS) vals[c] *= c < qw ? iq * a.wq[c] : ik * a.wk[c - qw];      // (the thread's own)
+        for (int u = 0; u < 4; ++u) {
+          const int q = min(q0 + u, taps - 1), src = i - taps + 1 + q;
+          x[u] = *(src >= 0 ? rows + static_cast<size_t>(src) * a.ldz + c : past + static_cast<size_t>(i + q) * C + c);
+          wt[u] = a.w[static_cast<size_t>(q) * C + c];
+        }
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          if (q0 + u < taps) v = fmaf(wt[u], x[u], v);
+      }
+      vals[c] = v;
+      if (a.move_on) history_move_on(past, C, taps, c, a.z[static_cast<size_t>(t) * a.ldz + c]);
+    }
+    if (run < runs) {
+      const float ss = wave_sum(v * v);
+      if (lane == 0) sums[run] = ss;
+    }
+  }
   __syncthreads();
+  float sq = 0.f, sk = 0.f;
+  for (int r = 0; r < runs_q; ++r) sq += sums[r];
+  for (int r = runs_q; r < runs; ++r) sk += sums[r];
+  const float iq = 1.0f / sqrtf(sq / static_cast<float>(qw) + a.eps), ik = 1.0f / sqrtf(sk / static_cast<float>(kw) + a.eps);
   const bool writes = a.write && place >= 0;
   const int page = writes ? place / a.page_size : 0, off = writes ? place % a.page_size : 0;
-  const int n = (writes ? a.H + 2 * a.G : a.H) * pairs;
-  for (int i = tid; i < n; i += THREADS) {
-    const int vec = i / pairs, e = 2 * (i % pairs);
-    const bool is_v = vec >= a.H + a.G;
-    const int width = is_v ? a.dv : a.dk;
-    const float* x = vals + (is_v ? qw + kw + (vec - a.H - a.G) * a.dv : vec * a.dk);
-    float out[2];
+  const int n_vec = writes ? a.H + 2 * a.G : a.H, sub = tid % LPV;
+  for (int vec = tid / LPV; vec < n_vec; vec += THREADS / LPV) {
+    const bool is_q = vec < a.H, is_v = vec >= a.H + a.G;
+    const int n = is_q ? vec : is_v ? vec - a.H - a.G : vec - a.H, width = is_v ? a.dv : a.dk;
+    const float* x = vals + (is_v ? qw + kw + n * a.dv : vec * a.dk);
+    const float* wn = is_q ? a.wq + n * a.dk : a.wk + n * a.dk;
+    const float inv = is_q ? iq : ik;
+    for (int m = sub; m < pairs; m += LPV) {
+      float out[2];
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      const int d = e + u;
-      float y = d < width ? x[d] : 0.f;
-      if (!is_v && d < 2 * half) y = d < half ? y * cs[d] - x[d + half] * sn[d] : y * cs[d - half] + x[d - half] * sn[d - half];
-      out[u] = y;
-    }
-    if (vec < a.H) {
-      store_pair(a.q_out, t * a.ldq + static_cast<size_t>(vec) * a.kept + e, a.dt, out[0], out[1]);
-    } else {
-      const size_t head = (static_cast<size_t>(page) * a.G + (vec - a.H) % a.G) * a.page_size * a.kept;
-      if (is_v) {
-        store_as(a.v_pool, head + static_cast<size_t>(e) * a.page_size + off, a.dt, out[0]);
-        store_as(a.v_pool, head + static_cast<size_t>(e + 1) * a.page_size + off, a.dt, out[1]);
+      for (int u = 0; u < 2; ++u) {
+        const int d = 2 * m + u;
+        float y = 0.f;
+        if (d < width) {
+          y = x[d];
+          if (!is_v) {
+            y *= inv * wn[d];
+            if (d < half) y = y * cs[d] - x[d + half] * (inv * wn[d + half]) * sn[d];
+            else if (d < 2 * half) y = y * cs[d - half] + x[d - half] * (inv * wn[d - half]) * sn[d - half];
+          }
+        }
+        out[u] = y;
+      }
+      const int e = 2 * m;
+      if (is_q) {
+        store_pair(a.q_out, t * a.ldq + static_cast<size_t>(n) * a.kept + e, a.dt, out[0], out[1]);
       } else {
-        store_pair(a.k_pool, head + static_cast<size_t>(off) * a.kept + e, a.dt, out[0], out[1]);
+        const size_t head = (static_cast<size_t>(page) * a.G + n) * a.page_size * a.kept;
+        if (is_v) {
+          store_as(a.v_pool, head + static_cast<size_t>(e) * a.page_size + off, a.dt, out[0]);
+          store_as(a.v_pool, head + static_cast<size_t>(e + 1) * a.page_size + off, a.dt, out[1]);
+        } else {
+          store_pair(a.k_pool, head + static_cast<size_t>(off) * a.kept + e, a.dt, out[0], out[1]);
+        }
       }
     }
   }
@@ -2341,8 +2373,17 @@ int dn_conv_turn_write(const float* z, long long ldz, int H, int G, int dk, int 
                        eps, freq, dims, positions, q_out, static_cast<size_t>(ldq), kept, slot_map, k_pool, v_pool, page_size, dt, write,
                        move_on && taps > 1};
   const size_t lds = static_cast<size_t>(C) * sizeof(float);
-  if (C <= 1024) hipLaunchKernelGGL(conv_turn_write_kernel<256>, dim3(T), dim3(256), lds, stream, a);
-  else hipLaunchKernelGGL(conv_turn_write_kernel<1024>, dim3(T), dim3(1024), lds, stream, a);
+  // (few rows: as many threads as a row's channels keep busy; many rows: more workgroups side by side.  The same bits either way)
+  const int threads = T > 256 || C <= 256 ? 256 : 1024;
+#define DN_CONV_TURN(N, L) hipLaunchKernelGGL((conv_turn_write_kernel<N, L>), dim3(T), dim3(N), lds, stream, a)
+  if (kept <= 64) {
+    if (threads == 256) DN_CONV_TURN(256, 32);
+    else DN_CONV_TURN(1024, 32);
+  } else {
+    if (threads == 256) DN_CONV_TURN(256, 64);
+    else DN_CONV_TURN(1024, 64);
+  }
+#undef DN_CONV_TURN
   return dn_launch_status();
 }
 

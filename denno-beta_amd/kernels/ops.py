@@ -153,6 +153,8 @@ def _declare(name, lib):
             "dn_conv_turn_write": [P, c_longlong, I, I, I, I, P, I, P, c_longlong, P, P, I, P, P, F, P, I, P, P, c_longlong, I, P, P, P, I, I, I, I, I, P],
             "dn_clamped_glu": [P, c_longlong, F, F, P, I, c_longlong, I, I, P],
             "dn_post_norm": [P, c_longlong, F, P, c_longlong, P, c_longlong, P, P, F, P, P, I, I, P, P, F, P, I, c_longlong, I, I, P],
+            "dn_delta_chunks": [P, c_longlong, P, c_longlong, P, c_longlong, P, c_longlong, P, c_longlong, P, P, P, c_longlong, P, P, I, I, I, I, I, I, P, P,
+                                c_longlong, P],
             "dn_turn_back_gate": [P, I, c_longlong, I, P, c_longlong, P, P, P, I, c_longlong, I, I, I, P],
             "dn_poly_norm": [P, c_longlong, P, F, P, I, c_longlong, I, I, P],
             "dn_head_gate": [P, I, c_longlong, I, P, c_longlong, P, I, c_longlong, I, I, I, P],
@@ -181,6 +183,9 @@ def _declare(name, lib):
         f = getattr(lib, fn)
         f.argtypes = args
         f.restype = c_int
+    if name == "sequence":
+        lib.dn_delta_chunks_floats.argtypes = [I, I, I, I, I]
+        lib.dn_delta_chunks_floats.restype = c_longlong
     if name == "gemm":
         lib.dn_gemm_work_floats.argtypes = [I, I, I, I]
         lib.dn_gemm_work_floats.restype = c_longlong
@@ -1278,6 +1283,38 @@ def state_scan(r, k, v, w, u, state, row_start, slots, n_heads, dk, dv, out, rea
     return out
 
 
+DELTA_CHUNKS_ROWS_MIN = 32      # rows a request, on average, from which the delta rule's chunks are worth their own kernels
+
+
+def delta_chunks_takes(T, S, dk):
+    """Whether a step of T rows of S requests is one for `delta_chunks` (portions, key heads of a size that it knows)."""
+    return T >= DELTA_CHUNKS_ROWS_MIN * S and dk % 16 == 0 and 16 <= dk <= 128
+
+
+def delta_chunks(r, k, v, beta, w, rate, bias, state, row_start, slots, n_heads, dk, dv, out, qk_heads=None):
+    """state_scan's delta rule with one decay per row and head (beta_logits, w_rows, w_rate = rate, w_bias = bias), 16 rows of a
+    request at a time on the matrix cores in 32-bit: the same recurrence, its sums in another order, so a row's result changes by
+    rounding with the place where its portion begins.  dk: a multiple of 16 up to 128; rows of r and k at multiples of 16 bytes."""
+    G = n_heads if qk_heads is None else qk_heads
+    _need(G >= 1 and n_heads % G == 0, lambda: f"delta_chunks: {n_heads} heads over {G} heads of queries and keys")
+    given = ((r, "r", G * dk), (k, "k", G * dk), (v, "v", n_heads * dv), (out, "out", n_heads * dv), (beta, "beta", n_heads), (w, "w", n_heads))
+    T = r.shape[0]
+    for t, name, n in given:
+        _dev(t, name, (torch.float32,), 2)
+        _need(tuple(t.shape) == (T, n), lambda: f"delta_chunks: {name} {tuple(t.shape)}")
+    S = _request_tables(row_start, slots, "delta_chunks")
+    _need(dk % 16 == 0 and 16 <= dk <= 128, lambda: f"delta_chunks: {dk} key channels a head; a multiple of 16 up to 128")
+    _need(rate is not None, "delta_chunks: rate")
+    _f32vec(rate, "rate", n_heads), _f32vec(bias, "bias", n_heads)
+    stride = _history(state, n_heads * dk * dv, "delta_chunks")
+    lib = _lib("sequence")
+    work = torch.empty(lib.dn_delta_chunks_floats(T, S, n_heads, dk, dv), dtype=torch.float32, device=r.device)
+    _ok(lib.dn_delta_chunks(r.data_ptr(), _rows(r, "r"), k.data_ptr(), _rows(k, "k"), v.data_ptr(), _rows(v, "v"), beta.data_ptr(), _rows(beta, "beta"),
+                            w.data_ptr(), _rows(w, "w"), rate.data_ptr(), _ptr(bias), state.data_ptr(), stride, row_start.data_ptr(), slots.data_ptr(),
+                            S, T, n_heads, G, dk, dv, work.data_ptr(), out.data_ptr(), _rows(out, "out"), _stream()), "delta_chunks")
+    return out
+
+
 def head_norm(o, weight, eps, out, n_heads, gate=None, gate_kind="silu", gate_first=False, skip=None, skip_scale=None):
     """y = o (+ skip * skip_scale, a second summand [T, n] with a number per run of n / len(skip_scale) columns); gate_first: y
     times act(gate) before the norm, else behind it; out[t, h, :] = y[t, h, :] / sqrt(mean(y[t, h, :]^2) + eps) * weight.
@@ -1531,7 +1568,7 @@ CONV_TURN_CHANNELS_MAX = 15000     # conv_turn_write keeps a row in LDS
 def conv_turn_write(z, n_heads, n_kv, dk, dv, w, hist, row_start, slots, positions, q_out, slot_map, k_pool, v_pool, wq, wk, eps, freq=None,
                     write=True, move_on=False):
     """A row of z (32-bit) begins with [q: n_heads x dk | k: n_kv x dk | v: n_kv x dv].  Every channel passes the short causal
-    convolution of conv_rows (identity=False, no activation; w [channels, taps], hist [slots, (taps - 1) * channels]); q and k are
+    convolution of conv_rows (identity=False, no activation; w here [taps, channels], hist [slots, (taps - 1) * channels]); q and k are
     each x / sqrt(mean(x^2) + eps) times a weight per entry as one vector over all heads; the first 2 len(freq) entries of every
     head's q and k are turned in pairs (i, i + len(freq)) by positions[t] * freq[i]; then to q_out and the pools as norm_turn_write
     puts them.  move_on: history_update in the same launch, for steps in which every request has one row."""
@@ -1539,7 +1576,7 @@ def conv_turn_write(z, n_heads, n_kv, dk, dv, w, hist, row_start, slots, positio
     _dev(slot_map, "slot_map", _I32, 1), _dev(positions, "positions", _I32, 1)
     _dev(k_pool, "k_pool", (q_out.dtype,), 4), _dev(v_pool, "v_pool", (q_out.dtype,), 4)
     T = z.shape[0]
-    C, taps = w.shape
+    taps, C = w.shape
     S = _request_tables(row_start, slots, "conv_turn_write")
     n_pages, Hkv, ps, kept = k_pool.shape
     _need(C == (n_heads + n_kv) * dk + n_kv * dv and w.is_contiguous() and z.shape[1] >= C and Hkv == n_kv and tuple(q_out.shape) == (T, n_heads * kept)

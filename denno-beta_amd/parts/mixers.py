@@ -572,7 +572,7 @@ class ConvAttention(Part):
             self.proj.bind(tensors)
         self.out.bind(tensors)
         n = self.names
-        self.conv = tensors[n["q_conv"] + "+k+v"].contiguous()
+        self.conv = tensors[n["q_conv"] + "+k+v"].t().contiguous()      # [taps, channels]
         self.q_norm, self.k_norm = tensors[n["q_norm"]], tensors[n["k_norm"]]
         if self.position is not None:
             self.position.bind(tensors, runtime)

@@ -336,10 +336,15 @@ class GatedDelta(Part):
             ops.history_update(z[:, :C], past, ctx.row_start, ctx.state_slots)
         gate, b = C, C + vw
         o = torch.empty((T, vw), dtype=F32, device=dev)
-        # (beta and the decay are made from their arguments inside the scan)
-        ops.state_scan(x[:, :qk], x[:, qk:2 * qk], x[:, 2 * qk:], z[:, b + H:b + 2 * H], None, state, ctx.row_start, ctx.state_slots, H,
-                       self.head_dim, self.value_dim, o, beta=z[:, b:b + H], qk_heads=self.n_qk_heads, beta_logits=True, w_rows=True,
-                       w_rate=self.rate, w_bias=self.dt_bias)
+        # (beta and the decay are made from their arguments inside the scan; the 32-bit engine walks a request's rows in order: its
+        # logits are the same bits however a prompt is cut)
+        if act != F32 and not single and qk % 4 == 0 and C % 4 == 0 and ops.delta_chunks_takes(T, ctx.S, self.head_dim):
+            ops.delta_chunks(x[:, :qk], x[:, qk:2 * qk], x[:, 2 * qk:], z[:, b:b + H], z[:, b + H:b + 2 * H], self.rate, self.dt_bias, state,
+                             ctx.row_start, ctx.state_slots, H, self.head_dim, self.value_dim, o, qk_heads=self.n_qk_heads)
+        else:
+            ops.state_scan(x[:, :qk], x[:, qk:2 * qk], x[:, 2 * qk:], z[:, b + H:b + 2 * H], None, state, ctx.row_start, ctx.state_slots, H,
+                           self.head_dim, self.value_dim, o, beta=z[:, b:b + H], qk_heads=self.n_qk_heads, beta_logits=True, w_rows=True,
+                           w_rate=self.rate, w_bias=self.dt_bias)
         y = torch.empty((T, vw), dtype=act, device=dev)
         ops.head_norm(o, self.norm, self.eps, y, H, gate=z[:, gate:gate + vw], gate_kind="silu")
         if accumulate_into is None:

@@ -434,6 +434,11 @@ def state_scan(r, k, v, w, u, state, row_start, slots, n_heads, dk, dv, out, rea
     return out
 
 
+def delta_chunks(r, k, v, beta, w, rate, bias, state, row_start, slots, n_heads, dk, dv, out, qk_heads=None):
+    return state_scan(r, k, v, w, None, state, row_start, slots, n_heads, dk, dv, out, beta=beta, qk_heads=qk_heads, beta_logits=True, w_rows=True,
+                      w_rate=rate, w_bias=bias)
+
+
 def head_norm(o, weight, eps, out, n_heads, gate=None, gate_kind="silu", gate_first=False, skip=None, skip_scale=None):
     T, n = o.shape
     dv = n // n_heads
@@ -601,7 +606,8 @@ def norm_turn_write(z, n_heads, n_kv, dk, dv, positions, q_out, slot_map, k_pool
 def conv_turn_write(z, n_heads, n_kv, dk, dv, w, hist, row_start, slots, positions, q_out, slot_map, k_pool, v_pool, wq, wk, eps, freq=None,
                     write=True, move_on=False):
     T, kept, ps = z.shape[0], k_pool.shape[3], k_pool.shape[2]
-    C, taps = w.shape
+    taps, C = w.shape
+    w = w.t().contiguous()
     qw, kw = n_heads * dk, n_kv * dk
     x = conv_rows(z, w, hist, row_start, slots, torch.zeros((T, C)), identity=False).double()
     unit = lambda v: v / torch.sqrt((v * v).mean(dim=-1, keepdim=True) + eps)      # noqa: E731

@@ -952,7 +952,7 @@ def test_queries_keys_and_values_convolved_normed_whole_turned_and_kept(dtype, l
     C = (H + G) * dk + G * dv
     kept = -(-max(dk, dv) // 16) * 16
     z = torch.randn(T, C + 5, device=DEV)
-    w = torch.randn(C, taps, device=DEV)
+    w = torch.randn(taps, C, device=DEV)
     hist = torch.randn(5, (taps - 1) * C + 3, device=DEV)
     wq, wk = torch.randn(H * dk, device=DEV), torch.randn(G * dk, device=DEV)
     pos = torch.randint(0, 4000, (T,), dtype=torch.int32, device=DEV)
@@ -978,6 +978,14 @@ def test_queries_keys_and_values_convolved_normed_whole_turned_and_kept(dtype, l
         close(k, hk, dtype, "k"), close(v, hv, dtype, "v")
         assert not bool(q[dead].any()) and torch.equal(hs.cpu(), hh)
         assert move_on or torch.equal(hs, hist)
+    if T > 256:      # (a row alone, in the kernel for few rows: the same bits)
+        t = int(row_start[3])
+        one, past = torch.empty(1, H * kept, dtype=dtype, device=DEV), torch.zeros(5, max(taps - 1, 1) * C, device=DEV)
+        for j in range(taps - 1):
+            past[3, j * C:(j + 1) * C] = hist[3, j * C:(j + 1) * C]
+        ops.conv_turn_write(z[t:t + 1].contiguous(), H, G, dk, dv, w, past[:, :(taps - 1) * C], torch.tensor([0, 1], dtype=torch.int32, device=DEV),
+                            slots[3:].contiguous(), pos[t:t + 1].contiguous(), one, sm[t:t + 1].contiguous(), k, v, wq, wk, 1e-5, freq, False, False)
+        assert torch.equal(one[0], q[t])
     with pytest.raises(Exception):
         ops.conv_turn_write(z, H, G, dk, dv, w, hist[:, :(taps - 1) * C], row_start, slots, pos, q, slot_map, k, v, wq, wk, 1e-5,
                             torch.ones(dk // 2 + 1, device=DEV))
@@ -1043,3 +1051,42 @@ def test_queries_times_a_temperature_of_their_position(dtype, every):
     wq, wk = torch.randn(dk, device=DEV), torch.randn(dk, device=DEV)
     both("norm_turn_write", lambda: (z, H, G, dk, dv, pos, torch.zeros(T, H * 48, dtype=dtype, device=DEV), slot_map, k, v, wq, wk, 1e-5, None, None,
                                      None, True, (0.3, every)), [6, 8, 9], dtype)
+
+
+@pytest.mark.parametrize("dk,dv,heads,qk_heads", [(16, 16, 2, 2), (64, 128, 4, 2), (48, 33, 3, 1), (128, 40, 2, 2), (80, 7, 2, 1), (32, 64, 6, 3), (96, 16, 1, 1),
+                                                  (112, 50, 2, 2)])
+@pytest.mark.parametrize("lengths", [[40], [16, 1, 33], [1, 15, 17, 200, 3], [2, 2, 5]])
+@pytest.mark.parametrize("fade", [0.02, 1.0, 30.0])
+def test_delta_rule_in_chunks(dk, dv, heads, qk_heads, lengths, fade):
+    """Sixteen rows at a time against row by row in 64-bit: decays near one (the state of long ago counts), ordinary ones, and
+    ones that leave nothing; keys that point almost the same way (the rows of a chunk then lean on each other the most); requests of
+    less than a chunk; padding left alone."""
+    slot_of = [4, 0, -1, 2, 1][:len(lengths)]
+    row_start, slots, T = tables(lengths, slot_of)
+    C = 2 * qk_heads * dk + heads * dv
+    x = torch.randn(T, C + (-C) % 4, device=DEV)
+    r, k, v = x[:, :qk_heads * dk], x[:, qk_heads * dk:2 * qk_heads * dk], x[:, 2 * qk_heads * dk:C]
+    shared = torch.randn(qk_heads, dk, device=DEV)
+    k.copy_(torch.nn.functional.normalize(k.reshape(T, qk_heads, dk) + 2.0 * shared, dim=-1).reshape(T, -1))
+    r.copy_(torch.nn.functional.normalize(r.reshape(T, qk_heads, dk), dim=-1).reshape(T, -1) * dk ** -0.5)
+    zs = torch.randn(T, 2 * heads + 3, device=DEV) * 2
+    zb, zw = zs[:, :heads], zs[:, heads:2 * heads]
+    rate, bias = (torch.rand(heads, device=DEV) + 0.1) * fade, torch.randn(heads, device=DEV)
+    state = torch.randn(5, heads * dk * dv + 11, device=DEV)
+    want_state, want = state.cpu().double(), torch.zeros(T, heads * dv, dtype=torch.float64)
+    d = lambda t: t.cpu().double()      # noqa: E731
+    ref.state_scan(d(r), d(k), d(v), d(zw), None, want_state[:, :heads * dk * dv], row_start.cpu(), slots.cpu(), heads, dk, dv, want, beta=d(zb),
+                   qk_heads=qk_heads, beta_logits=True, w_rows=True, w_rate=d(rate), w_bias=d(bias))
+    got_state, got = state.clone(), torch.full((T, heads * dv), 7.0, device=DEV)
+    ops.delta_chunks(r, k, v, zb, zw, rate, bias, got_state[:, :heads * dk * dv], row_start, slots, heads, dk, dv, got, qk_heads)
+    real = [t for s, n in enumerate(lengths) for t in range(int(row_start[s]), int(row_start[s]) + n) if slot_of[s] >= 0]
+    close(got[real], want[real]), close(got_state, want_state)
+    assert torch.equal(got_state[3], state[3])      # (a slot that no request of the step has)
+    # a state handed on at any row gives the same as one walk
+    cut = lengths[0] // 3
+    if cut:
+        st, one = state.clone(), torch.zeros(T, heads * dv, device=DEV)
+        for a, b in ((0, cut), (cut, lengths[0])):
+            ops.delta_chunks(r[a:b], k[a:b], v[a:b], zb[a:b], zw[a:b], rate, bias, st[:, :heads * dk * dv],
+                             torch.tensor([0, b - a], dtype=torch.int32, device=DEV), slots[:1].contiguous(), heads, dk, dv, one[a:b], qk_heads)
+        close(one[:lengths[0]], want[:lengths[0]]), close(st[4], want_state[4])
