@@ -135,8 +135,9 @@ __global__ __launch_bounds__(64) void route_wave_kernel(const float* z, size_t l
   const int t = blockIdx.x, lane = threadIdx.x;
   const float* row = z + static_cast<size_t>(t) * ldz;
   const float none = -__builtin_huge_valf();
-  __shared__ unsigned char open_group[8192];      // (groups <= experts <= 8,192)
-  __shared__ float group_score[8192];
+  // [groups] each, where there are groups (as much as they need: what a workgroup holds decides how many rows run side by side)
+  extern __shared__ float group_score[];
+  int* open_group = reinterpret_cast<int*>(group_score + groups);
   float m = none;
   for (int e = lane; e < E; e += 64) m = fmaxf(m, row[e]);
   m = wave_max(m);
@@ -742,7 +743,9 @@ int dn_moe_route(const float* z, long long ldz, const float* correction, int T, 
   if (groups < 1 || E % groups != 0 || keep < 1 || keep > groups || top > keep * (E / groups)) return DN_ERR_SHAPE;
   if (T == 0) return 0;
   if (E <= 8192 && top <= 64) {
-    hipLaunchKernelGGL(route_wave_kernel, dim3(T), dim3(64), 0, stream, z, static_cast<size_t>(ldz), correction, E, top, sigmoid, renorm,
+    const size_t lds = keep < groups ? groups * (sizeof(float) + sizeof(int)) : 0;
+    if (lds > 65536) return DN_ERR_SHAPE;
+    hipLaunchKernelGGL(route_wave_kernel, dim3(T), dim3(64), lds, stream, z, static_cast<size_t>(ldz), correction, E, top, sigmoid, renorm,
                        ids, wts, keep < groups ? groups : 1, keep, by_best, scale);
     return dn_launch_status();
   }
